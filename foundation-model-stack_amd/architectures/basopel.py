@@ -21,7 +21,7 @@ import torch
 
 from ..config import BasopelConfig
 from ..parts import LayerSpec, ModelSpec, PartSpec
-from ..weights.adapters import register_adapter, register_adapter_step
+from ..weights.adapters import pairs_to_neighbours, register_adapter, register_adapter_step
 from .registry import Architecture, register_architecture, register_model
 
 NAME = "basopel"
@@ -89,16 +89,6 @@ def basopel_spec(config: BasopelConfig) -> ModelSpec:
 
 
 # ---- the checkpoint's names -> the model's ----------------------------------------------------------------------
-def pairs_to_neighbours(t: torch.Tensor, heads: int, offset: int, dims: int) -> torch.Tensor:
-    """Rows of `heads` equal heads: in every head the run of `dims` rows from `offset` on is reordered so that row i and
-    row i + dims/2 of the run become rows 2i and 2i + 1."""
-    size = t.shape[0] // heads
-    rest = t.shape[1:]
-    v = t.reshape(heads, size, *rest)
-    run = v[:, offset : offset + dims].reshape(heads, 2, dims // 2, *rest).transpose(1, 2).reshape(heads, dims, *rest)
-    return torch.cat([v[:, :offset], run, v[:, offset + dims :]], dim=1).reshape(t.shape)
-
-
 def _layer_of(name: str, model_config) -> dict:
     return model_config.layers[int(re.match(r"l(\d+)\.", name).group(1))]
 

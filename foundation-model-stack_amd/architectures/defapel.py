@@ -20,7 +20,7 @@ import torch
 
 from ..config import DefapelConfig
 from ..parts import LayerSpec, ModelSpec, PartSpec
-from ..weights.adapters import register_adapter, register_adapter_step
+from ..weights.adapters import fuse_gated_delta, register_adapter, register_adapter_step
 from .registry import Architecture, register_architecture, register_model
 
 NAME = "defapel"
@@ -99,21 +99,6 @@ def defapel_spec(config: DefapelConfig) -> ModelSpec:
 _EXPERT = re.compile(r"^(l\d+\.mlp)\.e(\d+)\.(gate|up|down)$")
 
 
-def _fuse_delta(out: dict, p: str) -> None:
-    """The tensors of a gated delta rule under prefix p (which ends in a dot), in place."""
-    low_rank = p + "a1" in out
-    rows = [out.pop(p + n) for n in ("q", "k", "v", "b")]
-    rows.append(out.pop(p + ("a1" if low_rank else "a")))
-    rows.append(out.pop(p + ("g1" if low_rank else "g")))
-    out[p + "in_proj.weight"] = torch.cat(rows, dim=0)
-    out[p + "conv.weight"] = torch.cat([out.pop(p + n + ".conv") for n in ("q", "k", "v")], dim=0)
-    if low_rank:
-        out[p + "decay_up.weight"] = out.pop(p + "a2")
-        out[p + "gate_up.weight"] = out.pop(p + "g2")
-    out[p + "norm.weight"] = out.pop(p + "norm")
-    out[p + "out.weight"] = out.pop(p + "o")
-
-
 def _fuse_attention(out: dict, p: str) -> None:
     """The tensors of the windowed attention under prefix p, in place: queries, keys, values and the gate's rows are
     one projection (the gate has no bias: zeros)."""
@@ -138,7 +123,7 @@ def _to_model_names(sd, **kw):
     for (prefix, which), by_index in experts.items():
         out[f"{prefix}.experts.{which}"] = torch.stack([by_index[i] for i in sorted(by_index)], dim=0)
     for name in [n for n in out if n.endswith(".A_log")]:
-        _fuse_delta(out, name[: -len("A_log")])
+        fuse_gated_delta(out, name[: -len("A_log")])
     for name in [n for n in out if n.endswith(".mix.left.q")]:
         _fuse_attention(out, name[: -len("q")])
     renamed = {}

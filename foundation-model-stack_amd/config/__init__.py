@@ -3,6 +3,7 @@ from .basopel import BasopelConfig
 from .defapel import DefapelConfig
 from .llama import LLaMAConfig
 from .sidalorn import SidalornConfig
+from .zimorax import ZimoraxConfig
 from .zodolorn import ZodolornConfig
 
-__all__ = ["ModelConfig", "LLaMAConfig", "ZodolornConfig", "DefapelConfig", "SidalornConfig", "BasopelConfig"]
+__all__ = ["ModelConfig", "LLaMAConfig", "ZodolornConfig", "DefapelConfig", "SidalornConfig", "BasopelConfig", "ZimoraxConfig"]

@@ -3,6 +3,7 @@
 //                       at once, before they are cut into heads and rotated), or head by head with one weight for all
 //                       heads, from the float32 sums of the projection; the values are copied, or blended with the values
 //                       that an earlier layer left for the same token.  One rounding to the activation type.
+//   value_head_norm:    queries and keys copied, every head's value divided by its root mean square (no weight).
 //   gate_mul:           out = x * act(gate) * scale (gate: float32 logits, one a column or one a run of columns, or none),
 //                       into rows of any stride.
 //   cast_cols:          a run of columns of float32 rows as rows of their own, in the activation type.
@@ -97,6 +98,50 @@ extern "C" int fmsamd_qk_projection_norm(const float* proj, long ld, int nq, int
   else FMS_REQUIRE(false, "qk_projection_norm: unknown dtypes %d, %d", out_dtype, weight_dtype);
 #undef FMS_QKN
   FMS_LAUNCH_CHECK("qk_projection_norm");
+  return 0;
+}
+
+template <typename T>
+__global__ void __launch_bounds__(1024)
+    value_head_norm_kernel(const float* __restrict__ proj, long ld, int cols0, int heads, int dim, float eps, T* __restrict__ out, long ldo,
+                           const int* __restrict__ seq_of_token) {
+  const int t = blockIdx.x;
+  if (seq_of_token != nullptr && seq_of_token[t] < 0) return;
+  const float* row = proj + (size_t)t * ld;
+  T* o = out + (size_t)t * ldo;
+  const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, n_waves = blockDim.x / WAVE;
+  for (int head = wave; head < heads; head += n_waves) {
+    const float* x = row + cols0 + (size_t)head * dim;
+    float v[4], s = 0.f;  // a head has at most 256 entries
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = lane + e * WAVE;
+      v[e] = i < dim ? x[i] : 0.f;
+      s = fmaf(v[e], v[e], s);
+    }
+    const float inv = 1.f / sqrtf(wave_sum(s) / (float)dim + eps);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = lane + e * WAVE;
+      if (i < dim) o[cols0 + (size_t)head * dim + i] = from_f32<T>(v[e] * inv);
+    }
+  }
+  for (int i = threadIdx.x; i < cols0; i += blockDim.x) o[i] = from_f32<T>(row[i]);
+}
+
+extern "C" int fmsamd_value_head_norm(const float* proj, long ld, int cols0, int heads, int dim, float eps, void* out, int out_dtype,
+                                      long ldo, const int* seq_of_token, int n_tokens, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  FMS_REQUIRE(n_tokens > 0 && cols0 >= 0 && heads > 0 && dim > 0 && dim <= 4 * WAVE, "value_head_norm: bad sizes %d heads of %d", heads, dim);
+  FMS_REQUIRE(ld >= cols0 + (long)heads * dim && ldo >= cols0 + (long)heads * dim, "value_head_norm: the rows are too short");
+  const int threads = n_tokens <= 64 ? 1024 : 256;
+  if (out_dtype == FMS_F32)
+    value_head_norm_kernel<float><<<n_tokens, threads, 0, stream>>>(proj, ld, cols0, heads, dim, eps, (float*)out, ldo, seq_of_token);
+  else if (out_dtype == FMS_BF16)
+    value_head_norm_kernel<bf16><<<n_tokens, threads, 0, stream>>>(proj, ld, cols0, heads, dim, eps, (bf16*)out, ldo, seq_of_token);
+  else
+    FMS_REQUIRE(false, "value_head_norm: unknown dtype %d", out_dtype);
+  FMS_LAUNCH_CHECK("value_head_norm");
   return 0;
 }
 

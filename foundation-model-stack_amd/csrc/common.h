@@ -80,6 +80,10 @@ __device__ __forceinline__ float fms_activate(float x, int kind) {
       return x * tanhf(x > 20.f ? x : log1pf(expf(x)));
     case 7:  // gelu, tanh approximation
       return 0.5f * x * (1.f + tanhf(0.79788456080286536f * (x + 0.044715f * x * x * x)));
+    case 8: {  // the square of relu
+      const float r = fmaxf(x, 0.f);
+      return r * r;
+    }
     default:  // identity
       return x;
   }
@@ -93,6 +97,20 @@ __device__ __forceinline__ float wave_sum(float v) {
   for (int off = WAVE / 2; off > 0; off >>= 1) v += __shfl_xor(v, off, WAVE);
   return v;
 }
+
+// The sum over the 16 lanes of a row, in all of them, in the vector unit: two swaps inside quads, then the mirror of
+// a half row and of the row (a shuffle through LDS would put four round trips to LDS into a chain).
+__device__ __forceinline__ float row16_sum(float v) {
+#define FMS_DPP_ADD(ctrl) v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xF, 0xF, true))
+  FMS_DPP_ADD(0xB1);   // quad_perm [1, 0, 3, 2]
+  FMS_DPP_ADD(0x4E);   // quad_perm [2, 3, 0, 1]
+  FMS_DPP_ADD(0x141);  // row_half_mirror
+  FMS_DPP_ADD(0x140);  // row_mirror
+#undef FMS_DPP_ADD
+  return v;
+}
+
+__device__ __forceinline__ float softplus_f32(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 __device__ __forceinline__ float wave_max(float v) {
 #pragma unroll

@@ -26,7 +26,6 @@
 
 #define DELTA_MAX_TAPS CONV_MAX_TAPS
 
-__device__ __forceinline__ float softplus_f32(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.f / (1.f + expf(-z)); }
 
 // Blocks of 1024 threads for steps of few tokens (a decode step has a block per token and nothing else to hide a
@@ -117,18 +116,6 @@ struct DeltaArgs {
   const int* slot_ids;
   int H, G, D, Dv, per_channel;
 };
-
-// The sum over the 16 lanes of a row, in all of them, in the vector unit: two swaps inside quads, then the mirror of
-// a half row and of the row (a shuffle through LDS would put four round trips to LDS into every token's chain).
-__device__ __forceinline__ float row16_sum(float v) {
-#define FMS_DPP_ADD(ctrl) v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xF, 0xF, true))
-  FMS_DPP_ADD(0xB1);   // quad_perm [1, 0, 3, 2]
-  FMS_DPP_ADD(0x4E);   // quad_perm [2, 3, 0, 1]
-  FMS_DPP_ADD(0x141);  // row_half_mirror
-  FMS_DPP_ADD(0x140);  // row_mirror
-#undef FMS_DPP_ADD
-  return v;
-}
 
 // The sum over the PARTS lanes that share a column: a row of 16 lanes, or two rows (the second step swaps the odd rows
 // of one copy with the even rows of another, so that their sum is the pair's sum in both).

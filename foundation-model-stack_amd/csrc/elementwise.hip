@@ -53,7 +53,7 @@ extern "C" int fmsamd_embed(const int* ids, const void* table, int table_dtype, 
 
 // --------------------------------------------------------------------------
 // add + norm.  One block per output row.
-//   s = resid[r] (+ branch[r])            float32 sum, written back to resid
+//   s = resid[r] (+ branch[r] (* branch_scale))   float32 sum, written back to resid
 //   s = s - mean(s)                       if use_mean
 //   y = s * rsqrt(mean(s^2) + eps) (* weight) (+ bias)
 // With `rows`, output row i is computed from stream row rows[i] and the
@@ -86,6 +86,18 @@ __device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
   }
 }
 
+// VEC elements of a branch, times its factors per channel if it has them
+template <int VEC, typename T>
+__device__ __forceinline__ void load_branch(const T* p, const float* scale, float (&v)[VEC]) {
+  load_vec<VEC>(p, v);
+  if (scale != nullptr) {
+    float s[VEC];
+    load_vec<VEC>(scale, s);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] *= s[i];
+  }
+}
+
 // A thread keeps KEEP vectors of VEC elements in registers (and their weights, fetched before the
 // reduction so that they do not wait for it); a wider row is read again.  The loops over the kept
 // values have compile-time trip counts: the arrays must never be indexed by a run-time value, or
@@ -95,7 +107,7 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
                                                         const WeightT* __restrict__ weight,
                                                         const WeightT* __restrict__ bias, OutT* __restrict__ out,
                                                         const int* __restrict__ rows, int width, float eps,
-                                                        int use_mean) {
+                                                        int use_mean, const float* __restrict__ branch_scale) {
   __shared__ float scratch[17];
   const int r = rows ? rows[blockIdx.x] : blockIdx.x;
   float* x = resid + (size_t)r * width;
@@ -118,7 +130,7 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
       if (bias) load_vec<VEC>(bias + i, bkeep[n]);
       if (b) {
         float bv[VEC];
-        load_vec<VEC>(b + i, bv);
+        load_branch<VEC>(b + i, branch_scale ? branch_scale + i : nullptr, bv);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) keep[n][e] += bv[e];
         if (!rows) store_vec<VEC>(x + i, keep[n]);
@@ -135,7 +147,7 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
     load_vec<VEC>(x + i, v);
     if (b) {
       float bv[VEC];
-      load_vec<VEC>(b + i, bv);
+      load_branch<VEC>(b + i, branch_scale ? branch_scale + i : nullptr, bv);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] += bv[e];
       if (!rows) store_vec<VEC>(x + i, v);
@@ -164,7 +176,7 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
       load_vec<VEC>(x + i, v);
       if (reread_adds) {
         float bv[VEC];
-        load_vec<VEC>(b + i, bv);
+        load_branch<VEC>(b + i, branch_scale ? branch_scale + i : nullptr, bv);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) v[e] += bv[e];
       }
@@ -188,7 +200,7 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
     float v[VEC], wv[VEC], bv[VEC];
     load_vec<VEC>(x + i, v);
     if (reread_adds) {
-      load_vec<VEC>(b + i, bv);
+      load_branch<VEC>(b + i, branch_scale ? branch_scale + i : nullptr, bv);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] += bv[e];
     }
@@ -204,31 +216,32 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(float* __restrict__ resi
 
 template <typename BranchT, typename WeightT, typename OutT>
 static void launch_add_norm(float* resid, const void* branch, const void* weight, const void* bias, void* out,
-                            const int* rows, int n_out, int width, float eps, int use_mean, hipStream_t stream) {
-  const bool aligned = (((size_t)resid | (size_t)branch | (size_t)weight | (size_t)bias | (size_t)out) & 15) == 0;
+                            const int* rows, int n_out, int width, float eps, int use_mean, const float* branch_scale,
+                            hipStream_t stream) {
+  const bool aligned = (((size_t)resid | (size_t)branch | (size_t)weight | (size_t)bias | (size_t)out | (size_t)branch_scale) & 15) == 0;
   if (width % 4 == 0 && aligned) {
     // 4 vectors of 4 per thread cover the row up to 16 elements per thread; wider rows take more threads
     int threads = (width / 16 + 63) / 64 * 64;
     threads = threads < 64 ? 64 : (threads > 1024 ? 1024 : threads);
     add_norm_kernel<4, BranchT, WeightT, OutT><<<n_out, threads, 0, stream>>>(
         resid, (const BranchT*)branch, (const WeightT*)weight, (const WeightT*)bias, (OutT*)out, rows, width, eps,
-        use_mean);
+        use_mean, branch_scale);
   } else {
     const int threads = width > 4096 ? 1024 : (width >= 2048 ? 256 : (width >= 512 ? 128 : 64));
     add_norm_kernel<1, BranchT, WeightT, OutT><<<n_out, threads, 0, stream>>>(
         resid, (const BranchT*)branch, (const WeightT*)weight, (const WeightT*)bias, (OutT*)out, rows, width, eps,
-        use_mean);
+        use_mean, branch_scale);
   }
 }
 
 extern "C" int fmsamd_add_norm(float* resid, const void* branch, int act_dtype, const void* weight, const void* bias,
                                int weight_dtype, void* out, const int* rows, int n_out, int width, float eps,
-                               int use_mean, hipStream_t stream) {
+                               int use_mean, const float* branch_scale, hipStream_t stream) {
   if (n_out == 0) return 0;
   FMS_REQUIRE(n_out > 0 && width > 0, "add_norm: bad sizes rows=%d width=%d", n_out, width);
   FMS_REQUIRE(eps >= 0.f, "add_norm: eps %g is negative", (double)eps);
 #define FMS_AN(B, W, O)                                                                               \
-  launch_add_norm<B, W, O>(resid, branch, weight, bias, out, rows, n_out, width, eps, use_mean, stream)
+  launch_add_norm<B, W, O>(resid, branch, weight, bias, out, rows, n_out, width, eps, use_mean, branch_scale, stream)
   if (act_dtype == FMS_F32 && weight_dtype == FMS_F32)
     FMS_AN(float, float, float);
   else if (act_dtype == FMS_BF16 && weight_dtype == FMS_BF16)
@@ -241,6 +254,48 @@ extern "C" int fmsamd_add_norm(float* resid, const void* branch, int act_dtype, 
     FMS_REQUIRE(false, "add_norm: unknown dtypes act=%d weight=%d", act_dtype, weight_dtype);
 #undef FMS_AN
   FMS_LAUNCH_CHECK("add_norm");
+  return 0;
+}
+
+// --------------------------------------------------------------------------
+// the stream with what is still to be added, as rows of the activation type (the stream itself stays as it is)
+// --------------------------------------------------------------------------
+template <int VEC, typename T>
+__global__ void __launch_bounds__(256)
+    stream_rows_kernel(const float* __restrict__ resid, const T* __restrict__ branch, const float* __restrict__ branch_scale,
+                       T* __restrict__ out, long ldo, int width) {
+  const size_t t = blockIdx.x;
+  for (int i = threadIdx.x * VEC; i < width; i += blockDim.x * VEC) {
+    float v[VEC];
+    load_vec<VEC>(resid + t * width + i, v);
+    if (branch != nullptr) {
+      float bv[VEC];
+      load_branch<VEC>(branch + t * width + i, branch_scale ? branch_scale + i : nullptr, bv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += bv[e];
+    }
+    store_vec<VEC>(out + t * ldo + i, v);
+  }
+}
+
+extern "C" int fmsamd_stream_rows(const float* resid, const void* branch, const float* branch_scale, void* out, int act_dtype, long ldo,
+                                  int n_tokens, int width, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  FMS_REQUIRE(n_tokens > 0 && width > 0 && ldo >= width, "stream_rows: bad sizes T=%d width=%d", n_tokens, width);
+  const bool by_fours = width % 4 == 0 && ldo % 4 == 0 && (((size_t)resid | (size_t)branch | (size_t)branch_scale | (size_t)out) & 15) == 0;
+  const int threads = width >= 1024 ? 256 : 64;
+#define FMS_SR(V, T) stream_rows_kernel<V, T><<<n_tokens, threads, 0, stream>>>(resid, (const T*)branch, branch_scale, (T*)out, ldo, width)
+  if (act_dtype == FMS_F32) {
+    if (by_fours) FMS_SR(4, float);
+    else FMS_SR(1, float);
+  } else if (act_dtype == FMS_BF16) {
+    if (by_fours) FMS_SR(4, bf16);
+    else FMS_SR(1, bf16);
+  } else {
+    FMS_REQUIRE(false, "stream_rows: unknown dtype %d", act_dtype);
+  }
+#undef FMS_SR
+  FMS_LAUNCH_CHECK("stream_rows");
   return 0;
 }
 

@@ -6,7 +6,7 @@
 
 #include <hip/hip_runtime.h>
 
-#define FMSAMD_ABI_VERSION 10
+#define FMSAMD_ABI_VERSION 11
 
 // element types
 #define FMS_F32 0
@@ -21,7 +21,8 @@
 #define FMS_ACT_TANH 5
 #define FMS_ACT_MISH 6       // x tanh(log(1 + e^x))
 #define FMS_ACT_GELU_TANH 7  // the tanh approximation
-#define FMS_ACT_LAST FMS_ACT_GELU_TANH
+#define FMS_ACT_RELU2 8      // the square of relu
+#define FMS_ACT_LAST FMS_ACT_RELU2
 
 #ifdef __cplusplus
 extern "C" {
@@ -35,10 +36,15 @@ int fmsamd_embed(const int* ids, const void* table, int table_dtype, float* out,
                  float scale, hipStream_t stream);
 
 // resid += branch (float32 sum, written back unless `rows` is given); out = norm(resid) * weight + bias.
-// branch, weight, bias and rows may be null.  act_dtype is the type of branch and out.
+// branch, weight, bias and rows may be null.  act_dtype is the type of branch and out.  branch_scale (float32 [width] or
+// null): the branch is added times this vector, element by element.
 int fmsamd_add_norm(float* resid, const void* branch, int act_dtype, const void* weight, const void* bias,
                     int weight_dtype, void* out, const int* rows, int n_out, int width, float eps, int use_mean,
-                    hipStream_t stream);
+                    const float* branch_scale, hipStream_t stream);
+// out[t, 0:width] = resid[t] + branch[t] * branch_scale (branch and branch_scale may be null) in the activation type, rows
+// of out ldo apart; resid is left as it is
+int fmsamd_stream_rows(const float* resid, const void* branch, const float* branch_scale, void* out, int act_dtype, long ldo,
+                       int n_tokens, int width, hipStream_t stream);
 
 // out[t, j] = act(gu[t, j] + b[j]) * (gu[t, hidden + j] + b[hidden + j])
 int fmsamd_gated_act(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, int n_tokens, int hidden,
@@ -50,8 +56,8 @@ int fmsamd_advance_positions(int* positions, const int* seq_of_token, int n, hip
 int fmsamd_cast(const void* in, int in_dtype, void* out, int out_dtype, long n, hipStream_t stream);
 int fmsamd_bias_add(void* x, int dtype, const void* bias, int bias_dtype, int rows, int cols, hipStream_t stream);
 
-// cos/sin of position * freqs[i], float32, [max_pos, half]
-int fmsamd_rope_table(const float* freqs, float* cos_t, float* sin_t, int max_pos, int half, hipStream_t stream);
+// gain * cos/sin of position * freqs[i], float32, [max_pos, half]
+int fmsamd_rope_table(const float* freqs, float* cos_t, float* sin_t, int max_pos, int half, float gain, hipStream_t stream);
 
 // Rotate the queries of qkv in place; rotate the keys and write keys and values into the paged cache
 // (k_cache/v_cache null: queries only).  cos_t null: no rotation.  value_dim (0: head_dim): the size of a value if it
@@ -282,6 +288,10 @@ int fmsamd_qk_projection_norm(const float* proj, long ld, int nq, int nk, int nv
 // of x (a gate per head)
 int fmsamd_gate_mul(const void* x, long ldx, const float* gate, long ldg, int act, float scale, void* out, long ldo,
                     int dtype, int n_tokens, int cols, int group, hipStream_t stream);
+// out[t, 0:cols0] = proj[t, 0:cols0]; out[t, cols0 + h * dim + i] = proj[...] / rms over the head's dim entries, for `heads`
+// heads: values normed head by head without a weight.  proj: float32 rows; seq_of_token (or null): negative rows are skipped
+int fmsamd_value_head_norm(const float* proj, long ld, int cols0, int heads, int dim, float eps, void* out, int out_dtype, long ldo,
+                           const int* seq_of_token, int n_tokens, hipStream_t stream);
 int fmsamd_scale_f32(float* x, long n, float s, hipStream_t stream);
 // out[t, 0:n] = x[t, 0:n] (x: float32 rows ldx apart, already offset to the first column) in out_dtype
 int fmsamd_cast_cols(const float* x, long ldx, void* out, int out_dtype, long ldo, int n_tokens, int n, hipStream_t stream);
@@ -319,12 +329,12 @@ int fmsamd_gated_head_norm(const float* o, const float* gate, long ldg, const vo
 int fmsamd_group_norm_chain(float* resid, const void* branch, int act_dtype, const void* branch_weight, int branch_weight_dtype,
                             int branch_groups, float branch_eps, const void* weight, int weight_dtype, int groups, float eps,
                             void* out, int out_mode, const int* rows, int n_out, int width, hipStream_t stream);
-// out[t, c] = (x[t, c] if add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c] over a sequence's own tokens; the
+// out[t, c] = act((x[t, c] if add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c]) over a sequence's own tokens; the
 // inputs before the step come from conv_state [slots][taps-1][channels] (float32), which is then moved on.  x: float32 rows.
 // single_tokens: the caller knows that every sequence brings one token (a short step then needs no second kernel for the state).
 int fmsamd_short_conv(const float* x, long ld, int channels, const void* conv_w, const void* bias, int weight_dtype, int taps,
                       float* conv_state, const int* seq_of_token, const int* slot_ids, int add_input, void* out, int out_dtype,
-                      long ldo, int n_tokens, int single_tokens, hipStream_t stream);
+                      long ldo, int n_tokens, int single_tokens, int act, hipStream_t stream);
 
 // ---- the real-gated linear recurrent unit (rglru.hip) -------------------------------------------------------------------
 // u: float32 rows; ra_t, ri_t [blocks][in][out] (transposed square matrices), ra_b, ri_b, lam float32 [channels];
@@ -343,6 +353,26 @@ int fmsamd_rglru_scan_chunk(int n_tokens, int n_seqs);
 int fmsamd_rglru_scan_chunked(const float* a, const float* b, const float* y, long ldy, int act, float* state, const int* seq_starts,
                               const int* seq_of_token, const int* slot_ids, void* out, int out_dtype, long ldo, int n_tokens,
                               int n_seqs, int channels, int chunk, float* workspace, hipStream_t stream);
+
+// ---- attention whose scores are mixed over the heads (talking_attention.hip) ---------------------------------------------
+// score[h] = scale * sum_g talk[h, g] q_g . k_(kv head of g), talk float32 [nheads, nheads]; the softmax runs over the last
+// `window` keys (0: all) and, if given, the sink (float32 [nheads], a logit per head with neither key nor value).  Cache
+// layout as in rope.hip.  Any element type, any even head size.
+int fmsamd_talking_attn_generic(const void* q, long q_stride, void* out, long out_stride, int dtype, const int* positions,
+                                const int* seq_of_token, const int* block_table, int table_stride, const void* k_cache,
+                                const void* v_cache, const float* talk, const float* sink, int n_tokens, int nheads, int kvheads,
+                                int head_dim, int value_dim, float scale, int window, hipStream_t stream);
+
+// ---- the state-space recurrence (ssd.hip) --------------------------------------------------------------------------------
+// xbc: float32 rows [x: heads*vdim | B: groups*n_state | C: groups*n_state]; dt: float32 rows ld_dt apart, [T, heads]; with
+// d = softplus(dt + dt_bias): S <- exp(-exp(a_log) d) S + d x B^T, y = S C + skip x, over every sequence's tokens of the step,
+// from and into state [slots][heads][vdim][n_state]; y float32 [T, heads*vdim].
+int fmsamd_ssd_scan(const float* xbc, long ld, const float* dt, long ld_dt, const float* a_log, const float* dt_bias, const float* skip,
+                    float* state, float* y, const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
+                    int vdim, int groups, int n_state, hipStream_t stream);
+// out = N(y * silu(z)) * weight, N dividing each of `parts` equal parts of a row by its own root mean square; z: float32 rows
+int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void* weight, int weight_dtype, int parts, float eps,
+                            void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, hipStream_t stream);
 
 #ifdef __cplusplus
 }

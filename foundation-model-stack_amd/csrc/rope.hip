@@ -13,20 +13,20 @@
 // cos/sin of position * freq, float32: angle = float(p) * f, as the reference
 // builds its table (outer product of positions and frequencies, then cos/sin).
 __global__ void rope_table_kernel(const float* __restrict__ freqs, float* __restrict__ cos_t, float* __restrict__ sin_t,
-                                  int max_pos, int half) {
+                                  int max_pos, int half, float gain) {
   const int idx = blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= max_pos * half) return;
   const int p = idx / half, i = idx % half;
   const float angle = (float)p * freqs[i];
-  cos_t[idx] = cosf(angle);
-  sin_t[idx] = sinf(angle);
+  cos_t[idx] = gain * cosf(angle);
+  sin_t[idx] = gain * sinf(angle);
 }
 
 extern "C" int fmsamd_rope_table(const float* freqs, float* cos_t, float* sin_t, int max_pos, int half,
-                                 hipStream_t stream) {
+                                 float gain, hipStream_t stream) {
   FMS_REQUIRE(max_pos > 0 && half > 0, "rope_table: bad sizes max_pos=%d half=%d", max_pos, half);
   FMS_REQUIRE((long)max_pos * half < (1L << 31), "rope_table: table too large");
-  rope_table_kernel<<<ceil_div((long)max_pos * half, 256), 256, 0, stream>>>(freqs, cos_t, sin_t, max_pos, half);
+  rope_table_kernel<<<ceil_div((long)max_pos * half, 256), 256, 0, stream>>>(freqs, cos_t, sin_t, max_pos, half, gain);
   FMS_LAUNCH_CHECK("rope_table");
   return 0;
 }

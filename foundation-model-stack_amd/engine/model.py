@@ -38,6 +38,8 @@ class DecoderModel(Part):
             norms = {name: make_part("norm", n.kind, width=spec.width, **n.args) for name, n in zip(wanted, specs)}
             block = make_part("block", layer.block.kind, mixer=mixer, feed_forward=ff, **norms, **layer.block.args)
             self.layers.append(self.add_child(spec.layer_name.format(i=i), block))
+        # parts that replace the stream before certain schedule entries (a pass through looped layers)
+        self.entrances = {name: self.add_child(name, make_part("entrance", p.kind, width=spec.width, **p.args)) for name, p in spec.entrances.items()}
         self.final_norm = self.add_child(spec.final_norm_name, make_part("norm", spec.final_norm.kind, width=spec.width, **spec.final_norm.args))
         self.head = self.add_child(spec.head_name, make_part("head", spec.head.kind, width=spec.width, vocab=spec.vocab, **spec.head.args))
         # with tied heads the head's table is the embedding's (fms/models/llama.py:414-423)
@@ -133,18 +135,24 @@ class DecoderModel(Part):
         max_position = batch.max_context - 1
         batch.shared.clear()
         stream = ResidualStream(self.embedding.forward(batch.token_ids, batch))
+        for part in self.entrances.values():
+            part.begin(stream, batch, self.dtype)
         for n, entry in enumerate(self.schedule):
             block = self.layers[entry.layer]
             block.mixer.check_step(max_position)
+            if entry.enter is not None:
+                name, number = entry.enter
+                self.entrances[name].enter(number, stream, batch, self.dtype)
             owner = n if entry.cache_of is None else entry.cache_of
             if owner in cache.group_of_entry:
                 group, keys, values = cache.kv_of_entry(owner)
             else:
                 group, keys, values = -1, None, None
             view = LayerCache(group, keys, values, entry.cache_of is None, cache.state_of_entry(n))
-            if getattr(block, "fuses_next_norm", False) and n + 1 < len(self.schedule):
+            following = self.schedule[n + 1] if n + 1 < len(self.schedule) else None
+            if getattr(block, "fuses_next_norm", False) and following is not None and following.enter is None:
                 # the norm that reads the stream next, so that this block's last product can prepare its input
-                first_norm = getattr(self.layers[self.schedule[n + 1].layer], "first_norm", None)
+                first_norm = getattr(self.layers[following.layer], "first_norm", None)
                 block.forward(stream, batch, view, self.dtype, next_norm=first_norm() if first_norm else None)
             else:
                 block.forward(stream, batch, view, self.dtype)

@@ -17,7 +17,7 @@ import torch  # noqa: F401  (loads libamdhip64 before our library asks for it)
 
 from . import build as _build
 
-ABI_VERSION = 10
+ABI_VERSION = 11
 
 _lib: Optional[ctypes.CDLL] = None
 _lock = threading.Lock()
@@ -26,12 +26,13 @@ P, I, L, F = c_void_p, c_int, c_long, c_float
 
 _SIGNATURES = {
     "fmsamd_embed": [P, P, I, P, I, I, I, F, P],
-    "fmsamd_add_norm": [P, P, I, P, P, I, P, P, I, I, F, I, P],
+    "fmsamd_add_norm": [P, P, I, P, P, I, P, P, I, I, F, I, P, P],
+    "fmsamd_stream_rows": [P, P, P, P, I, L, I, I, P],
     "fmsamd_gated_act": [P, P, I, P, I, I, I, I, P],
     "fmsamd_cast": [P, I, P, I, L, P],
     "fmsamd_advance_positions": [P, P, I, P],
     "fmsamd_bias_add": [P, I, P, I, I, I, P],
-    "fmsamd_rope_table": [P, P, P, I, I, P],
+    "fmsamd_rope_table": [P, P, P, I, I, F, P],
     "fmsamd_rope_kv_write": [P, I, L, P, P, P, I, P, P, I, I, P, P, I, I, I, I, I, P],
     "fmsamd_attn_generic": [P, L, P, L, I, P, P, P, I, P, P, I, I, I, I, F, I, P, F, I, I, I, P, P, I, P],
     "fmsamd_attn_prefill_bf16": [P, L, P, L, P, P, P, P, I, I, P, I, P, P, I, I, I, I, F, I, F, I, P, I, P, I, P],
@@ -63,19 +64,23 @@ _SIGNATURES = {
     "fmsamd_moe_route_grouped": [P, L, I, I, I, P, I, I, F, P, P, P],
     "fmsamd_poly_norm": [P, L, I, F, F, F, F, F, P, I, L, I, P],
     "fmsamd_group_norm_chain": [P, P, I, P, I, I, F, P, I, I, F, P, I, P, I, I, P],
-    "fmsamd_short_conv": [P, L, I, P, P, I, I, P, P, P, I, P, I, L, I, I, P],
+    "fmsamd_short_conv": [P, L, I, P, P, I, I, P, P, P, I, P, I, L, I, I, I, P],
     "fmsamd_rglru_gates": [P, L, P, P, P, P, I, P, F, P, P, P, I, I, I, P],
     "fmsamd_rglru_scan": [P, P, P, L, I, P, P, P, P, P, I, L, I, I, P],
     "fmsamd_rglru_scan_chunk": [I, I],
     "fmsamd_rglru_scan_chunked": [P, P, P, L, I, P, P, P, P, P, I, L, I, I, I, I, P, P],
     "fmsamd_qk_projection_norm": [P, L, I, I, I, P, P, I, F, P, I, L, P, I, I, P, L, P, P],
     "fmsamd_gate_mul": [P, L, P, L, I, F, P, L, I, I, I, I, P],
+    "fmsamd_value_head_norm": [P, L, I, I, I, F, P, I, L, P, I, P],
     "fmsamd_scale_f32": [P, L, F, P],
     "fmsamd_cast_cols": [P, L, P, I, L, I, I, P],
     "fmsamd_delta_prepare": [P, L, I, P, L, I, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P],
     "fmsamd_delta_rule": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
     "fmsamd_gated_head_norm": [P, P, L, P, I, F, I, F, P, I, L, P, I, I, I, P],
     "fmsamd_moe_combine": [P, P, I, P, P, L, P, I, I, I, P, I, P, L, P],
+    "fmsamd_talking_attn_generic": [P, L, P, L, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
+    "fmsamd_ssd_scan": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P],
     "fmsamd_probe_read": [P, L, I, I, P, P],
     "fmsamd_probe_mfma": [I, I, I, P, P, P],
 }

@@ -20,7 +20,7 @@ from .library import check, load
 F32, BF16 = 0, 1
 # the names of the reference (fms/utils/activation.py:14-24) and "identity"; the numbers are FMS_ACT_* of csrc/fmsamd.h
 ACTIVATIONS = {"silu": 0, "swish": 0, "gelu": 1, "relu": 2, "identity": 3, "sigmoid": 4, "tanh": 5, "mish": 6,
-               "gelu-tanh": 7, "gelu_pytorch_tanh": 7}
+               "gelu-tanh": 7, "gelu_pytorch_tanh": 7, "relu2": 8}
 PAGE_TOKENS = 64
 
 
@@ -78,12 +78,14 @@ def add_norm(
     out_dtype: torch.dtype,
     rows: Optional[torch.Tensor] = None,
     use_mean: bool = False,
+    branch_scale: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
-    """resid += branch (in place, float32); returns norm(resid) * weight + bias in `out_dtype`.
+    """resid += branch (* branch_scale, float32 [width]) (in place, float32); returns norm(resid) * weight + bias in `out_dtype`.
 
     With `rows` (int32 indices) only those rows are produced and resid is left as it is.
     """
-    _need_cuda(resid, branch, weight, bias, rows)
+    _need_cuda(resid, branch, weight, bias, rows, branch_scale)
+    _check_branch_scale(branch_scale, resid)
     if resid.dtype != torch.float32 or resid.dim() != 2 or not resid.is_contiguous():
         raise ValueError("the residual stream must be a contiguous float32 [T, width] tensor")
     T, width = resid.shape
@@ -104,8 +106,28 @@ def add_norm(
         n_out = rows.numel()
     out = torch.empty(n_out, width, dtype=out_dtype, device=resid.device)
     check(load().fmsamd_add_norm(resid.data_ptr(), _ptr(branch), _code(out_dtype), _ptr(weight), _ptr(bias), _code(wdtype),
-                                 out.data_ptr(), _ptr(rows), n_out, width, float(eps), int(use_mean), _stream()))
+                                 out.data_ptr(), _ptr(rows), n_out, width, float(eps), int(use_mean),
+                                 _ptr(branch_scale), _stream()))
     return out
+
+
+def _check_branch_scale(branch_scale: Optional[torch.Tensor], resid: torch.Tensor) -> None:
+    if branch_scale is not None and (branch_scale.dtype != torch.float32 or tuple(branch_scale.shape) != (resid.shape[1],)
+                                     or not branch_scale.is_contiguous()):
+        raise ValueError(f"the branch's factors are a contiguous float32 [{resid.shape[1]}] tensor")
+
+
+def stream_rows(resid: torch.Tensor, branch: Optional[torch.Tensor], branch_scale: Optional[torch.Tensor], out: torch.Tensor) -> None:
+    """out = resid + branch (* branch_scale) in the type of out (the branch's too), rows of any stride; resid stays as it is."""
+    _need_cuda(resid, branch, branch_scale, out)
+    if resid.dtype != torch.float32 or resid.dim() != 2 or not resid.is_contiguous():
+        raise ValueError("the residual stream must be a contiguous float32 [T, width] tensor")
+    _rows2d("out", out)
+    _check_branch_scale(branch_scale, resid)
+    if out.shape != resid.shape or (branch is not None and (branch.shape != resid.shape or not branch.is_contiguous() or branch.dtype != out.dtype)):
+        raise ValueError(f"branch (contiguous) and out are {tuple(resid.shape)} of one type")
+    check(load().fmsamd_stream_rows(resid.data_ptr(), _ptr(branch), _ptr(branch_scale), out.data_ptr(), _code(out.dtype), out.stride(0),
+                                    resid.shape[0], resid.shape[1], _stream()))
 
 
 def gated_act(gu: torch.Tensor, bias: Optional[torch.Tensor], activation: str) -> torch.Tensor:
@@ -154,15 +176,15 @@ def bias_add_(x: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
 
 
 # --------------------------------------------------------------------------
-def rope_table(freqs: torch.Tensor, max_pos: int):
-    """cos and sin of position * freqs, float32 [max_pos, len(freqs)]."""
+def rope_table(freqs: torch.Tensor, max_pos: int, gain: float = 1.0):
+    """gain times cos and sin of position * freqs, float32 [max_pos, len(freqs)]."""
     _need_cuda(freqs)
     if freqs.dtype != torch.float32 or freqs.dim() != 1 or not freqs.is_contiguous():
         raise ValueError("freqs must be a contiguous float32 vector")
     half = freqs.numel()
     cos = torch.empty(max_pos, half, dtype=torch.float32, device=freqs.device)
     sin = torch.empty_like(cos)
-    check(load().fmsamd_rope_table(freqs.data_ptr(), cos.data_ptr(), sin.data_ptr(), max_pos, half, _stream()))
+    check(load().fmsamd_rope_table(freqs.data_ptr(), cos.data_ptr(), sin.data_ptr(), max_pos, half, float(gain), _stream()))
     return cos, sin
 
 
@@ -806,9 +828,9 @@ CONV_MAX_TAPS = 8
 
 def short_conv(x: torch.Tensor, col0: int, channels: int, conv_w: torch.Tensor, bias: Optional[torch.Tensor], conv_state: Optional[torch.Tensor],
                seq_of_token: torch.Tensor, slot_ids: torch.Tensor, out_dtype: torch.dtype, add_input: bool = False,
-               single_tokens: bool = False) -> torch.Tensor:
-    """A causal convolution over time on the channels col0 .. col0 + channels of float32 rows: out[t, c] = (x[t, c] if
-    add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c] over the sequence's own tokens -> [T, channels] in
+               single_tokens: bool = False, activation: str = "identity") -> torch.Tensor:
+    """A causal convolution over time on the channels col0 .. col0 + channels of float32 rows: out[t, c] = act((x[t, c] if
+    add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c]) over the sequence's own tokens -> [T, channels] in
     out_dtype.  The inputs before the step come from conv_state [slots, taps - 1, channels] (float32; zeros before a
     sequence's start), which is then moved on to the step's last inputs.  single_tokens: every sequence of the step
     brings exactly one token (a decode step); the kernel that convolves then moves the state on as well."""
@@ -831,7 +853,7 @@ def short_conv(x: torch.Tensor, col0: int, channels: int, conv_w: torch.Tensor, 
     view = x[:, col0 : col0 + channels]
     check(load().fmsamd_short_conv(view.data_ptr(), x.stride(0), channels, conv_w.data_ptr(), _ptr(bias), _code(conv_w.dtype), taps,
                                    _ptr(conv_state), seq_of_token.data_ptr(), slot_ids.data_ptr(), int(bool(add_input)), out.data_ptr(),
-                                   _code(out_dtype), out.stride(0), T, int(bool(single_tokens)), _stream()))
+                                   _code(out_dtype), out.stride(0), T, int(bool(single_tokens)), ACTIVATIONS[activation], _stream()))
     return out
 
 
@@ -1226,6 +1248,49 @@ def qk_projection_norm(proj: torch.Tensor, nq: int, nk: int, nv: int, q_weight: 
     return out
 
 
+def value_head_norm(proj: torch.Tensor, col0: int, heads: int, dim: int, eps: float, out_dtype: torch.dtype,
+                    seq_of_token: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """float32 rows -> [T, col0 + heads * dim] in out_dtype: the first col0 columns (queries and keys) as they are, then
+    `heads` values of `dim` entries, each divided by its root mean square."""
+    _need_cuda(proj, seq_of_token)
+    _rows2d("proj", proj)
+    n = col0 + heads * dim
+    if proj.dtype != torch.float32 or col0 < 0 or heads <= 0 or not 0 < dim <= 256 or proj.shape[1] < n:
+        raise ValueError("value_head_norm takes float32 rows that hold the columns asked for, and heads of at most 256 entries")
+    if seq_of_token is not None:
+        _need_i32("seq_of_token", seq_of_token)
+    out = torch.empty(proj.shape[0], n, dtype=out_dtype, device=proj.device)
+    check(load().fmsamd_value_head_norm(proj.data_ptr(), proj.stride(0), col0, heads, dim, float(eps), out.data_ptr(), _code(out_dtype),
+                                        out.stride(0), _ptr(seq_of_token), proj.shape[0], _stream()))
+    return out
+
+
+def talking_attention(q: torch.Tensor, positions, seq_of_token, block_table, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                      talk: torch.Tensor, sink: Optional[torch.Tensor], nheads: int, kvheads: int, head_dim: int, value_dim: int,
+                      scale: float, window: int = 0, *, decode: bool = False, max_context: int = 0) -> torch.Tensor:
+    """Causal attention of every token over the cache of its sequence with scores mixed over the heads before the softmax,
+    score_h = scale * sum_g talk[h, g] q_g . k_(kv head of g), over the last `window` keys (0: all) -> [T, nheads*value_dim].
+    talk: float32 [nheads, nheads]; sink: float32 [nheads], a logit per head in the denominator only, or None."""
+    _need_cuda(q, positions, seq_of_token, block_table, k_cache, v_cache, talk, sink)
+    _rows2d("q", q)
+    T = q.shape[0]
+    _check_batch_index(positions, seq_of_token, block_table, T)
+    _check_cache(k_cache, v_cache, kvheads, head_dim, q.dtype, value_dim)
+    if talk.dtype != torch.float32 or tuple(talk.shape) != (nheads, nheads) or not talk.is_contiguous():
+        raise ValueError(f"talk is a contiguous float32 [{nheads}, {nheads}] tensor")
+    if sink is not None and (sink.dtype != torch.float32 or tuple(sink.shape) != (nheads,) or not sink.is_contiguous()):
+        raise ValueError(f"sink must be a contiguous float32 [{nheads}] tensor")
+    out = torch.empty(T, nheads * value_dim, dtype=q.dtype, device=q.device)
+    lib = load()
+    for t0 in range(0, T, 65535):
+        n = min(65535, T - t0)
+        check(lib.fmsamd_talking_attn_generic(q[t0:].data_ptr(), q.stride(0), out[t0:].data_ptr(), out.stride(0), _code(q.dtype),
+                                              positions[t0:].data_ptr(), seq_of_token[t0:].data_ptr(), block_table.data_ptr(),
+                                              block_table.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), talk.data_ptr(), _ptr(sink), n,
+                                              nheads, kvheads, head_dim, value_dim, float(scale), int(window), _stream()))
+    return out
+
+
 def gate_mul(x: torch.Tensor, gate: Optional[torch.Tensor], activation: str = "sigmoid", scale: float = 1.0,
              out: Optional[torch.Tensor] = None, group: int = 1) -> torch.Tensor:
     """x * act(gate) * scale, elementwise over rows [T, cols]; gate: float32 logits (a view with contiguous rows) or None;
@@ -1372,6 +1437,63 @@ def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, e
     check(load().fmsamd_gated_head_norm(o.data_ptr(), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight.dtype), float(eps),
                                         ACTIVATIONS[activation], float(scale), out.data_ptr(), _code(out_dtype), out.stride(0),
                                         seq_of_token.data_ptr(), T, heads, vdim, _stream()))
+    return out
+
+
+# --------------------------------------------------------------------------
+# the state-space recurrence
+# --------------------------------------------------------------------------
+SSD_MAX_STATE = 256
+
+
+def ssd(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, skip: torch.Tensor, state: torch.Tensor,
+        seq_starts: torch.Tensor, seq_of_token: torch.Tensor, slot_ids: torch.Tensor, n_seqs: int, heads: int, vdim: int, groups: int,
+        n_state: int, longest: int) -> torch.Tensor:
+    """S <- exp(-exp(a_log) d) S + d x B^T, y = S C + skip x with d = softplus(dt + dt_bias), over the tokens of every sequence
+    of the step, from and into state [slots, heads, vdim, n_state] (float32) -> y float32 [T, heads*vdim].  xbc: float32 rows
+    [x: heads*vdim | B: groups*n_state | C: groups*n_state]; dt: float32 rows [T, heads] of any stride.  Sequence b owns the
+    token rows seq_starts[b] .. seq_starts[b + 1] and the state of slot_ids[b]; longest: the most tokens a sequence brings."""
+    _need_cuda(xbc, dt, a_log, dt_bias, skip, state, seq_starts, seq_of_token, slot_ids)
+    _rows2d("xbc", xbc)
+    _rows2d("dt", dt)
+    for name, t in (("seq_starts", seq_starts), ("seq_of_token", seq_of_token), ("slot_ids", slot_ids)):
+        _need_i32(name, t)
+    T = xbc.shape[0]
+    if xbc.dtype != torch.float32 or xbc.shape[1] != heads * vdim + 2 * groups * n_state:
+        raise ValueError(f"xbc is float32 [T, {heads * vdim + 2 * groups * n_state}], got {xbc.dtype} {tuple(xbc.shape)}")
+    if dt.dtype != torch.float32 or tuple(dt.shape) != (T, heads):
+        raise ValueError(f"dt is float32 [{T}, {heads}]")
+    for name, t in (("a_log", a_log), ("dt_bias", dt_bias), ("skip", skip)):
+        if t.dtype != torch.float32 or tuple(t.shape) != (heads,) or not t.is_contiguous():
+            raise ValueError(f"{name} is a contiguous float32 [{heads}] tensor")
+    if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, vdim, n_state) or not state.is_contiguous():
+        raise ValueError(f"the state is contiguous float32 [slots, {heads}, {vdim}, {n_state}]")
+    if not 0 < n_state <= SSD_MAX_STATE:
+        raise ValueError(f"the recurrence keeps at most {SSD_MAX_STATE} state rows a head, not {n_state}")
+    if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs or seq_of_token.numel() < T:
+        raise ValueError("the step's index arrays are shorter than its sequences or tokens")
+    y = torch.empty(T, heads * vdim, dtype=torch.float32, device=xbc.device)
+    check(load().fmsamd_ssd_scan(xbc.data_ptr(), xbc.stride(0), dt.data_ptr(), dt.stride(0), a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(),
+                                 state.data_ptr(), y.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(),
+                                 int(n_seqs), heads, vdim, groups, n_state, _stream()))
+    return y
+
+
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, parts: int, eps: float, out_dtype: torch.dtype,
+                     seq_of_token: torch.Tensor) -> torch.Tensor:
+    """y * silu(z), each of `parts` equal consecutive parts of a row divided by its own root mean square, times weight:
+    y float32 [T, cols] contiguous, z float32 rows [T, cols] of any stride -> [T, cols] in out_dtype."""
+    _need_cuda(y, z, weight, seq_of_token)
+    _rows2d("z", z)
+    _need_i32("seq_of_token", seq_of_token)
+    T, cols = y.shape
+    if y.dtype != torch.float32 or not y.is_contiguous() or z.dtype != torch.float32 or tuple(z.shape) != (T, cols):
+        raise ValueError("gated_group_norm takes float32 rows y (contiguous) and z of one shape")
+    if tuple(weight.shape) != (cols,) or not weight.is_contiguous() or parts < 1 or cols % parts or seq_of_token.numel() < T:
+        raise ValueError(f"gated_group_norm: a contiguous weight [{cols}], {parts} equal parts, a sequence index per token")
+    out = torch.empty(T, cols, dtype=out_dtype, device=y.device)
+    check(load().fmsamd_gated_group_norm(y.data_ptr(), z.data_ptr(), z.stride(0), weight.data_ptr(), _code(weight.dtype), int(parts), float(eps),
+                                         out.data_ptr(), _code(out_dtype), seq_of_token.data_ptr(), T, cols, _stream()))
     return out
 
 

@@ -65,9 +65,11 @@ class MultiHeadAttention(Mixer):
         output_gate=False,
         chunk: int = 0,
         keep_first: int = 0,
-        sink: bool = False,
+        sink=False,
         distance_bias: Optional[dict] = None,
         value_mix: Optional[str] = None,
+        value_norm: bool = False,
+        talking_heads: bool = False,
     ):
         """value_dim: the size of a value (and of an output head) if it is not head_dim.  qkv_bias, out_bias: biases of the
         input and the output projection (default: use_bias for both).  qk_norm "projection": queries and keys pass an RMS
@@ -78,11 +80,14 @@ class MultiHeadAttention(Mixer):
         chunk c > 0 (no window then): positions are cut into runs of c from the sequence's start, and a query sees the
         keys of its own run only.  keep_first: with a window, the sequence's first keys that every later query still sees
         (at their true positions).  sink: a learned logit per head in the softmax's denominator, with neither key nor
-        value.  distance_bias {"rows": B, "far": D}: a learned table [B, heads] added to the scores by bucketed distance
+        value (a number instead of True: that logit for every head, not learned).  distance_bias {"rows": B, "far": D}: a learned table [B, heads] added to the scores by bucketed distance
         n: row n below B/2, then B/2 + floor(log(n / (B/2)) / log(D / (B/2)) * (B - B/2)), at most B - 1.
         value_mix: "first": the step's values are handed to later layers as they are; "blend": the values become
         (1 - lambda) v + lambda v_first with a learned lambda and the values that the "first" layer left for the same
-        token (the blended values are what is cached)."""
+        token (the blended values are what is cached).
+        value_norm: every head's value is divided by its root mean square (norm_eps, no weight) before it is cached.
+        talking_heads: the heads' scores (scaled, before the mask and the softmax) are mixed by a learned matrix,
+        score_h <- sum_g talk[h, g] score_g."""
         super().__init__()
         if kvheads <= 0 or nheads % kvheads:
             raise ValueError(f"{nheads} query heads are no multiple of {kvheads} kv heads")
@@ -104,7 +109,9 @@ class MultiHeadAttention(Mixer):
             raise ValueError(f"output_gate {output_gate!r} is not one of False, True, 'element', 'head'")
         self.qk_norm, self.norm_eps, self.output_gate = qk_norm, float(norm_eps), bool(output_gate)
         self.gate_per_head = output_gate == "head"
-        self.chunk, self.keep_first, self.has_sink = int(chunk), int(keep_first), bool(sink)
+        self.chunk, self.keep_first = int(chunk), int(keep_first)
+        self.has_sink = sink is True
+        self.fixed_sink = float(sink) if isinstance(sink, (int, float)) and not isinstance(sink, bool) else None
         if self.chunk < 0 or self.keep_first < 0 or (self.chunk and (self.window or self.keep_first)):
             raise ValueError("chunks go with neither a window nor kept first keys, and no size is negative")
         if self.keep_first and not self.window:
@@ -117,10 +124,15 @@ class MultiHeadAttention(Mixer):
         if value_mix and not qk_norm:
             raise NotImplementedError("values are handed on and blended by the kernel that norms queries and keys")
         self.value_mix = value_mix
+        self.value_norm, self.talking_heads = bool(value_norm), bool(talking_heads)
+        if self.value_norm and (self.qk_norm or self.value_mix):
+            raise NotImplementedError("normed values go with neither normed queries and keys nor blended values")
+        if self.talking_heads and (self.soft_cap or self.chunk or self.keep_first or self.distance_bias is not None):
+            raise NotImplementedError("scores that are mixed over the heads carry no cap, no chunks, no kept keys and no distance table")
         qkv_bias = use_bias if qkv_bias is None else bool(qkv_bias)
         out_bias = use_bias if out_bias is None else bool(out_bias)
         # the steps beyond Llama's attention run a path of their own; without them nothing changes
-        self.extended = bool(self.qk_norm or self.output_gate or self.value_dim != head_dim or self.value_mix)
+        self.extended = bool(self.qk_norm or self.output_gate or self.value_dim != head_dim or self.value_mix or self.value_norm or self.talking_heads)
         self.n_q, self.n_k, self.n_v = nheads * head_dim, kvheads * head_dim, kvheads * self.value_dim
         in_proj = self.add_child("in_proj", Part())
         # with an output gate the gate's rows follow the values: everything that reads the mixer's input is one product
@@ -136,6 +148,9 @@ class MultiHeadAttention(Mixer):
             self.declare("rel", (self.distance_bias["rows"], nheads), init="normal", kind="scale")
         if self.value_mix:
             self.declare("vmix", (), init="zeros", kind="scale")  # the "first" layer has one too, and does not use it
+        if self.talking_heads:
+            self.declare("talk", (nheads, nheads), init="normal", kind="scale")
+        self._talk = None
         self._sink = self._bias_by_distance = self._lambda = None
         self.dense = self.add_child("dense", Linear(nheads * self.value_dim, width, out_bias))
 
@@ -160,6 +175,10 @@ class MultiHeadAttention(Mixer):
         distance (row n of every head for n up to the first distance of the last bucket, which serves all beyond)."""
         if self.has_sink:
             self._sink = self.w["sink"].to(torch.float32).contiguous()
+        elif self.fixed_sink is not None:
+            self._sink = torch.full((self.nheads,), self.fixed_sink, dtype=torch.float32, device=device)
+        if self.talking_heads:
+            self._talk = self.w["talk"].to(torch.float32).contiguous()
         if self.value_mix == "blend":
             self._lambda = self.w["vmix"].to(torch.float32).reshape(1).contiguous()
         if self.distance_bias is not None:
@@ -183,6 +202,8 @@ class MultiHeadAttention(Mixer):
         return self.position_encoder.score_slopes(self.nheads) if self.position_encoder is not None else None
 
     def prefill_qblock(self, n_tokens: int, dtype) -> int:
+        if self.talking_heads:
+            return 0
         if (dtype != torch.bfloat16 or self.head_dim % 16 or self._score_slopes() is not None or self.value_dim != self.head_dim
                 or ((self.keep_first or self.distance_bias is not None) and ops.prefill_extras_are_generic(self.head_dim))
                 or ops.prefill_cap_is_generic(self.head_dim, self.soft_cap)):
@@ -229,6 +250,8 @@ class MultiHeadAttention(Mixer):
                                              v_first=v_first, v_lambda=self._lambda if v_first is not None else None)
                 if self.value_mix == "first":
                     batch.shared["first_values"] = qkv[:, self.n_q + self.n_k :]
+            elif self.value_norm:
+                qkv = ops.value_head_norm(proj, self.n_q + self.n_k, K, self.value_dim, self.norm_eps, x.dtype, batch.seq_of_token)
             else:
                 qkv = ops.cast_cols(proj, 0, self.n_q + self.n_k + self.n_v, x.dtype)
             if self.output_gate:
@@ -249,6 +272,13 @@ class MultiHeadAttention(Mixer):
             ops.rope_kv_write(qkv, batch.positions, batch.seq_of_token, table, cos, sin, rot, keys, values, H, K, D)
         size = 0 if batch.is_decode else self.prefill_qblock(batch.n_tokens, x.dtype)
         qb_start, qb_len = batch.qblocks.get(size, (None, None))
+        if self.talking_heads:
+            mixed = ops.talking_attention(qkv, batch.positions, batch.seq_of_token, table, cache.keys, cache.values, self._talk, self._sink,
+                                          H, K, D, self.value_dim, self.scale, self.window, decode=batch.is_decode,
+                                          max_context=batch.context_bound)
+            if gate is not None or out is not None or out_scale != 1.0:
+                mixed = ops.gate_mul(mixed, gate, "sigmoid", out_scale, out=out, group=self.value_dim if self.gate_per_head else 1)
+            return BranchOutput(mixed, self.dense)
         mixed = ops.attention(
             qkv, batch.positions, batch.seq_of_token, table, cache.keys, cache.values, H, K, D, self.scale, self.window,
             decode=batch.is_decode, max_context=batch.context_bound,

@@ -142,10 +142,21 @@ class FeedForward(Part):
         return self.forward(x)
 
 
+class Entrance(Part):
+    """A part that replaces the residual stream before certain schedule entries run (a pass through looped layers)."""
+
+    def begin(self, stream, batch, act_dtype) -> None:
+        """Called once a step, when the stream holds the embedding's output and no layer has run."""
+
+    def enter(self, number: int, stream, batch, act_dtype) -> None:
+        """Replaces the stream for pass `number`, right before the pass's first layer."""
+        raise NotImplementedError
+
+
 # --------------------------------------------------------------------------
 # registries: category -> kind -> constructor
 # --------------------------------------------------------------------------
-CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head")
+CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "entrance", "embedding", "head")
 _registry: Dict[str, Dict[str, Callable[..., Part]]] = {c: {} for c in CATEGORIES}
 
 

@@ -32,6 +32,7 @@ class ResidualStream:
         self.resid = resid
         self.pending: Optional[torch.Tensor] = None
         self.pending_norm: Optional[Part] = None  # the norm that the pending branch passes before it is added
+        self.pending_scale: Optional[torch.Tensor] = None  # a factor per channel on the pending branch
         self.prepared: Optional[tuple] = None  # (norm, NormedRows) of the stream as it is now
 
     def normed(self, norm: Part, act_dtype: torch.dtype, deferred_ok: bool = False, rows: Optional[torch.Tensor] = None):
@@ -41,8 +42,11 @@ class ResidualStream:
             return prepared[1]
         pending, self.pending = self.pending, None
         pending_norm, self.pending_norm = self.pending_norm, None
+        pending_scale, self.pending_scale = self.pending_scale, None
         if pending_norm is not None:
             return norm.add_norm(self.resid, pending, act_dtype, rows, branch_norm=pending_norm)
+        if pending_scale is not None:
+            return norm.add_norm(self.resid, pending, act_dtype, rows, branch_scale=pending_scale)
         return norm.add_norm(self.resid, pending, act_dtype, rows)
 
     def rows(self, act_dtype: torch.dtype, want_rows: bool = True) -> Optional[torch.Tensor]:
@@ -62,15 +66,34 @@ class ResidualStream:
             return None
         return out if copy_wanted else self.resid
 
-    def add_branch(self, out, next_norm: Optional[Part] = None, post_norm: Optional[Part] = None) -> None:
+    def rows_into(self, out: torch.Tensor) -> None:
+        """The stream as it is, with what is pending added, into rows of the activation type and any stride.  The stream
+        itself is not brought up to date: for whoever replaces it next (replace)."""
+        if self.pending_norm is not None:
+            raise NotImplementedError("a branch with a norm of its own is added by the norm that reads the stream next")
+        ops.stream_rows(self.resid, self.pending, self.pending_scale, out)
+
+    def replace(self, resid: torch.Tensor) -> None:
+        """Another stream in the place of this one; what was pending goes with the old one."""
+        self.resid = resid
+        self.pending = self.pending_norm = self.pending_scale = self.prepared = None
+
+    def add_branch(self, out, next_norm: Optional[Part] = None, post_norm: Optional[Part] = None,
+                   scale: Optional[torch.Tensor] = None) -> None:
         """Takes a branch's output: a tensor (added when the stream is next read) or a BranchOutput.  post_norm: the
-        branch joins the stream through that norm (the norm that reads the stream next applies both)."""
+        branch joins the stream through that norm (the norm that reads the stream next applies both).  scale: the branch
+        joins times this vector (float32 [width])."""
         if self.pending is not None:
             raise RuntimeError("a branch output is still to be added: read the stream through a norm between two branches")
         if post_norm is not None:
             # the branch's norm needs the whole row of the branch: its last product cannot add into the stream
             self.pending = out.value() if isinstance(out, BranchOutput) else out
             self.pending_norm = post_norm
+            self.prepared = None
+            return
+        if scale is not None:
+            self.pending = out.value() if isinstance(out, BranchOutput) else out
+            self.pending_scale = scale
             self.prepared = None
             return
         if isinstance(out, BranchOutput):
@@ -92,8 +115,10 @@ class PreNormBlock(Part):
     norm_arguments = ("norm1", "norm2")  # the norms the block is built with, by constructor argument
 
     def __init__(self, mixer: Part, feed_forward: Optional[Part], norm1: Part, norm2: Part,
-                 names=("ln", "attn", "ff_ln", "ff_sub_layer")):
-        """The feed-forward may be absent (None): the block is then its mixer branch alone, and has no second norm."""
+                 names=("ln", "attn", "ff_ln", "ff_sub_layer"), branch_scales=None, width: int = 0):
+        """The feed-forward may be absent (None): the block is then its mixer branch alone, and has no second norm.
+        branch_scales (two names; width: the stream's): every branch's result is multiplied by a learned vector of that
+        name, element by element, before it joins the stream."""
         super().__init__()
         self.norm1 = self.add_child(names[0], norm1)
         self.mixer = self.add_child(names[1], mixer)
@@ -101,6 +126,14 @@ class PreNormBlock(Part):
         if feed_forward is not None:
             self.norm2 = self.add_child(names[2], norm2)
             self.add_child(names[3], feed_forward)
+        self.branch_scales = tuple(branch_scales)[: 1 if feed_forward is None else 2] if branch_scales else ()
+        for name in self.branch_scales:
+            self.declare(name, (width,), init="ones", kind="scale")
+        self._scales = [None, None]
+
+    def finalize(self, device, dtype) -> None:
+        for i, name in enumerate(self.branch_scales):
+            self._scales[i] = self.w[name].to(torch.float32).contiguous()
 
     def first_norm(self) -> Part:
         return self.norm1
@@ -111,13 +144,13 @@ class PreNormBlock(Part):
         h = stream.normed(self.norm1, act_dtype, mixer_takes is not None and mixer_takes(T, act_dtype, batch))
         branch = getattr(self.mixer, "forward_branch", self.mixer.forward)
         if self.feed_forward is None:
-            stream.add_branch(branch(h, batch, cache), next_norm)
+            stream.add_branch(branch(h, batch, cache), next_norm, scale=self._scales[0])
             return
-        stream.add_branch(branch(h, batch, cache), self.norm2)
+        stream.add_branch(branch(h, batch, cache), self.norm2, scale=self._scales[0])
         ff_takes = getattr(self.feed_forward, "accepts_normed_rows", None)
         h = stream.normed(self.norm2, act_dtype, ff_takes is not None and ff_takes(T, act_dtype))
         branch = getattr(self.feed_forward, "forward_branch", self.feed_forward.forward)
-        stream.add_branch(branch(h), next_norm)
+        stream.add_branch(branch(h), next_norm, scale=self._scales[1])
 
 
 class SandwichNormBlock(Part):

@@ -1,6 +1,6 @@
 """Feed-forwards beside the gated linear unit: a plain two-layer one, and a mixture of small experts.
 
-``MLP``: down(act(up(x))).
+``MLP``: down(act(up(x))), with or without biases.
 
 ``ExpertsFeedForward``: a router gives every token float32 logits over the experts; the `top` largest are its
 experts, weighted by the softmax over those logits alone (`score` "softmax"), by each one's sigmoid ("sigmoid") or by

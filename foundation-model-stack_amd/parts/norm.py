@@ -61,10 +61,14 @@ class ParameterizedNorm(Part):
         out_dtype: torch.dtype,
         rows: Optional[torch.Tensor] = None,
         branch_norm: Optional["ParameterizedNorm"] = None,
+        branch_scale: Optional[torch.Tensor] = None,
     ) -> torch.Tensor:
         """resid += branch (float32, in place); returns norm(resid) in out_dtype (only `rows` if given).
         branch_norm: the branch goes through that norm first (a block that norms its branches before they join the
-        stream); both norms and the sum are then one kernel."""
+        stream); both norms and the sum are then one kernel.
+        branch_scale (float32 [width]): the branch joins the stream times this vector, element by element."""
+        if branch_scale is not None and (branch_norm is not None or self.groups > 1):
+            raise NotImplementedError("a branch with a scale of its own joins the stream without a norm, and is read through a norm of one group")
         grouped = self.groups > 1 or (branch_norm is not None and branch_norm.groups > 1)
         if grouped:
             if not self._plain_rms() or (branch_norm is not None and not branch_norm._plain_rms()):
@@ -86,7 +90,7 @@ class ParameterizedNorm(Part):
         bias = self.w.get("bias")
         if bias is not None and self._scale is not None:
             bias = bias.to(torch.float32)  # the kernel takes scale and shift of one type
-        return ops.add_norm(resid, branch, self.scale_weight(), bias, self.eps, out_dtype, rows, self.use_mean)
+        return ops.add_norm(resid, branch, self.scale_weight(), bias, self.eps, out_dtype, rows, self.use_mean, branch_scale)
 
     def join(self, resid: torch.Tensor, branch: torch.Tensor, act_dtype: torch.dtype, want_rows: bool) -> Optional[torch.Tensor]:
         """resid += norm(branch) (float32, in place), for a block whose norms sit behind its branches; returns the stream

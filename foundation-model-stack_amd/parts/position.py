@@ -40,6 +40,8 @@ def rope_frequencies(dim: int, theta: float, scaling: Optional[dict] = None, alp
     regular: fms/modules/positions.py:124-132.  llama3: fms/modules/positions.py:171-196.
     ntk: fms/modules/positions.py:161-168, theta * alpha^(dim / (dim - 2)) for the power of two `alpha`.
     linear: every frequency divided by scaling["factor"].
+    yarn: frequency i divided by the factor where its dimension turns fewer than `beta_slow` times over the original
+    length, kept where it turns more than `beta_fast` times, and a straight line between the two in i in between.
     """
     scaling = dict(scaling or {})
     kind = scaling.get("rope_type", "regular")
@@ -55,6 +57,14 @@ def rope_frequencies(dim: int, theta: float, scaling: Optional[dict] = None, alp
         return freqs.to(torch.float32)
     if kind == "linear":  # positions counted in steps of 1 / factor: every frequency divided by the factor
         return (freqs / float(scaling["factor"])).to(torch.float32)
+    if kind == "yarn":
+        def dim_of(turns):  # the (real) index of the dimension pair that turns so many times over the original length
+            return dim * math.log(scaling["original_max_position_embeddings"] / (2 * math.pi * turns)) / (2 * math.log(theta))
+
+        lo = max(math.floor(dim_of(scaling["beta_fast"])), 0)
+        hi = min(math.ceil(dim_of(scaling["beta_slow"])), dim - 1)
+        ramp = ((torch.arange(dim // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        return (freqs / float(scaling["factor"]) * ramp + freqs * (1 - ramp)).to(torch.float32)
     if kind == "llama3":
         factor = scaling["factor"]
         low_freq_factor = scaling["low_freq_factor"]
@@ -66,7 +76,13 @@ def rope_frequencies(dim: int, theta: float, scaling: Optional[dict] = None, alp
         smoothed = (1 - smooth) * scaled / factor + smooth * scaled
         medium = ~(wavelen < old_len / high_freq_factor) * ~(wavelen > old_len / low_freq_factor)
         return torch.where(medium, smoothed, scaled).to(torch.float32)
-    raise ValueError(f"rope_type {kind!r} is not supported (regular, linear, llama3, ntk)")
+    raise ValueError(f"rope_type {kind!r} is not supported (regular, linear, yarn, llama3, ntk)")
+
+
+def rope_gain(scaling: Optional[dict]) -> float:
+    """The factor on cosines and sines that goes with a scaling: 0.1 ln(factor) + 1 for yarn, else 1."""
+    scaling = scaling or {}
+    return 0.1 * math.log(scaling["factor"]) + 1.0 if scaling.get("rope_type") == "yarn" else 1.0
 
 
 class PositionEncoding(Part):
@@ -127,7 +143,7 @@ class RotaryEncoding(PositionEncoding):
         while True:
             length = min(self.max_seq_len * alpha, self.max_positions)
             freqs = rope_frequencies(self.rot_dim, self.theta, self.scaling, alpha, exact=self.exact_frequencies)
-            self.tables[alpha] = ops.rope_table(freqs.to(device), length)
+            self.tables[alpha] = ops.rope_table(freqs.to(device), length, rope_gain(self.scaling))
             if self.max_seq_len * alpha >= self.max_positions:
                 break
             alpha *= 2

@@ -10,7 +10,7 @@ twice or let an entry read the cache of an earlier entry.
 from __future__ import annotations
 
 import dataclasses
-from typing import Dict, List, Optional
+from typing import Dict, List, Optional, Tuple
 
 
 @dataclasses.dataclass
@@ -33,6 +33,8 @@ class LayerSpec:
 class ScheduleEntry:
     layer: int  # index into ModelSpec.layers
     cache_of: Optional[int] = None  # earlier schedule entry whose cache this entry reads instead of owning one
+    # (key into ModelSpec.entrances, number of the pass): what replaces the residual stream right before this entry runs
+    enter: Optional[Tuple[str, int]] = None
 
 
 @dataclasses.dataclass
@@ -46,6 +48,7 @@ class ModelSpec:
     head: PartSpec = dataclasses.field(default_factory=lambda: PartSpec("linear"))
     positions: Dict[str, PartSpec] = dataclasses.field(default_factory=dict)
     schedule: Optional[List[ScheduleEntry]] = None  # default: every layer once, in order
+    entrances: Dict[str, PartSpec] = dataclasses.field(default_factory=dict)  # by the name their parameters start with
     tie_heads: bool = False
     # parameter name prefixes (the reference's names by default)
     embedding_name: str = "base_model.embedding"
@@ -59,6 +62,8 @@ class ModelSpec:
         for n, entry in enumerate(self.schedule):
             if not 0 <= entry.layer < len(self.layers):
                 raise ValueError(f"schedule entry {n} names layer {entry.layer}, the model has {len(self.layers)}")
+            if entry.enter is not None and entry.enter[0] not in self.entrances:
+                raise ValueError(f"schedule entry {n} is entered through {entry.enter[0]!r}, which the model does not have")
             if entry.cache_of is not None:
                 if not 0 <= entry.cache_of < n:
                     raise ValueError(f"schedule entry {n} reads the cache of entry {entry.cache_of}, which does not run before it")

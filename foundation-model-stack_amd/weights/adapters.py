@@ -122,3 +122,29 @@ def fuse_glu_step(sd, **kw):
             out[f"{prefix}.wg1_fused.{kind}"] = torch.cat([sd[name], sd[up]], dim=0)
             del out[name], out[up]
     return out
+
+
+def pairs_to_neighbours(t: torch.Tensor, heads: int, offset: int, dims: int) -> torch.Tensor:
+    """For checkpoints that pair rotated entry i with entry i + dims/2, where the rotation kernels turn neighbouring pairs.
+    Rows of `heads` equal heads: in every head the run of `dims` rows from `offset` on is reordered so that row i and
+    row i + dims/2 of the run become rows 2i and 2i + 1."""
+    size = t.shape[0] // heads
+    rest = t.shape[1:]
+    v = t.reshape(heads, size, *rest)
+    run = v[:, offset : offset + dims].reshape(heads, 2, dims // 2, *rest).transpose(1, 2).reshape(heads, dims, *rest)
+    return torch.cat([v[:, :offset], run, v[:, offset + dims :]], dim=1).reshape(t.shape)
+
+
+def fuse_gated_delta(out: dict, p: str) -> None:
+    """The tensors of a gated delta rule under prefix p (which ends in a dot), in place."""
+    low_rank = p + "a1" in out
+    rows = [out.pop(p + n) for n in ("q", "k", "v", "b")]
+    rows.append(out.pop(p + ("a1" if low_rank else "a")))
+    rows.append(out.pop(p + ("g1" if low_rank else "g")))
+    out[p + "in_proj.weight"] = torch.cat(rows, dim=0)
+    out[p + "conv.weight"] = torch.cat([out.pop(p + n + ".conv") for n in ("q", "k", "v")], dim=0)
+    if low_rank:
+        out[p + "decay_up.weight"] = out.pop(p + "a2")
+        out[p + "gate_up.weight"] = out.pop(p + "g2")
+    out[p + "norm.weight"] = out.pop(p + "norm")
+    out[p + "out.weight"] = out.pop(p + "o")
