@@ -362,6 +362,24 @@ int fmsamd_talking_attn_generic(const void* q, long q_stride, void* out, long ou
                                 const int* seq_of_token, const int* block_table, int table_stride, const void* k_cache,
                                 const void* v_cache, const float* talk, const float* sink, int n_tokens, int nheads, int kvheads,
                                 int head_dim, int value_dim, float scale, int window, hipStream_t stream);
+// The same for bfloat16 on the matrix cores, for sizes of which ..._fits says so (rows: multiples of 8; the scale positive).
+// Prompts: the step is cut into query blocks of at most ..._qblock(...) consecutive tokens of one sequence; sizes that fit
+// the decode kernel only (prefill_fits says 0) run prompts through it.  Decode: a block per (token, 16 heads, split), the
+// visible keys of every sequence dealt over the splits; more than one split needs a workspace of ..._workspace(...) bytes.
+int fmsamd_talking_attn_mfma_fits(int kvheads, int head_dim, int value_dim);
+int fmsamd_talking_attn_prefill_fits(int kvheads, int head_dim, int value_dim);
+int fmsamd_talking_attn_qblock(int nheads, int kvheads);
+int fmsamd_talking_attn_prefill(const void* q, long q_stride, void* out, long out_stride, const int* positions,
+                                const int* seq_of_token, const int* qblock_start, const int* qblock_len, int n_qblocks,
+                                int qblock_tokens, const int* block_table, int table_stride, const void* k_cache,
+                                const void* v_cache, const float* talk, const float* sink, int n_tokens, int nheads, int kvheads,
+                                int head_dim, int value_dim, float scale, int window, hipStream_t stream);
+long fmsamd_talking_attn_workspace(int n_tokens, int nheads, int value_dim, int n_splits);
+int fmsamd_talking_attn_decode(const void* q, long q_stride, void* out, long out_stride, void* workspace, long workspace_bytes,
+                               const int* positions, const int* seq_of_token, const int* block_table, int table_stride,
+                               const void* k_cache, const void* v_cache, const float* talk, const float* sink, int n_tokens,
+                               int nheads, int kvheads, int head_dim, int value_dim, float scale, int window, int n_splits,
+                               hipStream_t stream);
 
 // ---- the state-space recurrence (ssd.hip) --------------------------------------------------------------------------------
 // xbc: float32 rows [x: heads*vdim | B: groups*n_state | C: groups*n_state]; dt: float32 rows ld_dt apart, [T, heads]; with
@@ -370,6 +388,13 @@ int fmsamd_talking_attn_generic(const void* q, long q_stride, void* out, long ou
 int fmsamd_ssd_scan(const float* xbc, long ld, const float* dt, long ld_dt, const float* a_log, const float* dt_bias, const float* skip,
                     float* state, float* y, const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
                     int vdim, int groups, int n_state, hipStream_t stream);
+// The same for long steps, in chunks of 64 tokens as float32 matrix products.  longest: the most tokens a sequence brings;
+// workspace of fmsamd_ssd_chunk_workspace(...) bytes.
+long fmsamd_ssd_chunk_workspace(int n_tokens, int n_seqs, int heads);
+int fmsamd_ssd_chunked(const float* xbc, long ld, const float* dt, long ld_dt, const float* a_log, const float* dt_bias, const float* skip,
+                       float* state, float* y, const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
+                       int vdim, int groups, int n_state, int n_tokens, int longest, float* workspace, long workspace_bytes,
+                       hipStream_t stream);
 // out = N(y * silu(z)) * weight, N dividing each of `parts` equal parts of a row by its own root mean square; z: float32 rows
 int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void* weight, int weight_dtype, int parts, float eps,
                             void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, hipStream_t stream);

@@ -6,6 +6,14 @@
 //
 //   ssd_scan:         token by token (decode steps, short portions).  The rows of S never mix, so 16 lanes share a value
 //                     channel, each with a run of its N entries in registers.
+//   ssd_chunk_scores, ssd_chunk_walk: long steps, in chunks of 64 tokens as matrix products (float32 matrix instructions:
+//                     true 32-bit products and sums).  With l_t the sum of the chunk's log decays up to and with token t,
+//                       y_t = exp(l_t) S C_t + sum_{s <= t} M_ts x_s + skip x_t,    M_ts = (C_t . B_s) exp(l_t - l_s) d_s
+//                       S  <- exp(l_end) S + sum_s d_s exp(l_end - l_s) x_s B_s^T
+//                     The first kernel makes every chunk's M (side by side, nothing depends on the state); the second walks
+//                     a sequence's chunks with the state in accumulators, 16 value channels of a head a block.  The sums
+//                     l are kept in float64 until their differences are taken: a chunk may decay by hundreds of e-folds,
+//                     and neighbours' differences are small.
 //   gated_group_norm: y * silu(z), each of `parts` equal parts of the row over its own root mean square, times a weight.
 //
 // The state is kept [slot][head][value channel][state row], so that a lane's entries are contiguous.
@@ -91,6 +99,274 @@ extern "C" int fmsamd_ssd_scan(const float* xbc, long ld, const float* dt, long 
   else if (n_state <= 128) ssd_scan_kernel<8><<<grid, 256, 0, stream>>>(a);
   else ssd_scan_kernel<16><<<grid, 256, 0, stream>>>(a);
   FMS_LAUNCH_CHECK("ssd_scan");
+  return 0;
+}
+
+// ---- long steps, in chunks -------------------------------------------------------------------------------------------------
+#define SSD_CHUNK 64
+#define SSD_HEADS 8  // heads of a block of ssd_chunk_scores, at most
+
+// What the chunks of a step leave for the walk, by chunk slot and head: M [64][64], the weights of the tokens in the state
+// d_s exp(l_end - l_s) [64], and exp(l_t) [64].  Chunk i of sequence b has the slot seq_starts[b] / 64 + b + i.
+struct SsdChunks {
+  float *m, *w, *e;
+};
+__device__ __forceinline__ int ssd_chunk_slot(int start, int b, int i) { return start / SSD_CHUNK + b + i; }
+
+// Four entries n .. n + 3 of a row of B or C (zeros from N on).
+template <bool VEC>
+__device__ __forceinline__ f32x4 ssd_row4(const float* row, int n, int N) {
+  if (VEC) return n < N ? *reinterpret_cast<const f32x4*>(row + n) : f32x4{0.f, 0.f, 0.f, 0.f};
+  f32x4 v;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = n + i < N ? row[n + i] : 0.f;
+  return v;
+}
+
+// The float32 product: lane (r = lane % 16, g = lane / 16) holds A[row r][k g] and B[k g][column r], and rows 4 g + i of
+// column r of the result.  Which k a step takes is free as long as both operands agree: four steps take the k's
+// 4 g + i, i = 0 .. 3, of sixteen, so that a lane's operands of four steps are four neighbours in memory.
+#define SSD_MFMA(a, b, c) __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0)
+
+template <bool VEC>
+__global__ void __launch_bounds__(256) ssd_chunk_scores_kernel(SsdArgs a, SsdChunks out, int subsets) {
+  __shared__ double ls[SSD_HEADS][SSD_CHUNK];
+  __shared__ float ds[SSD_HEADS][SSD_CHUNK];
+  const int b = blockIdx.y;
+  const int start = a.seq_starts[b], t1 = a.seq_starts[b + 1];
+  const int t0 = start + blockIdx.x * SSD_CHUNK;
+  if (t0 >= t1 || a.seq_of_token[start] < 0) return;
+  const int group = blockIdx.z / subsets, subset = blockIdx.z % subsets;
+  const int per = a.H / a.G;
+  const int h0 = group * per + subset * SSD_HEADS;
+  const int nh = min(SSD_HEADS, per - subset * SSD_HEADS);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const size_t slot = ssd_chunk_slot(start, b, blockIdx.x);
+  const int last = t1 - 1;
+  // decays: a lane a token, a wave a head
+  for (int hh = wave; hh < nh; hh += 4) {
+    const int h = h0 + hh, t = t0 + lane;
+    float d = 0.f;  // past the sequence's end: a token that changes nothing
+    if (t <= last) d = softplus_f32(a.dt[(size_t)t * a.ld_dt + h] + a.dt_bias[h]);
+    double l = -(double)(expf(a.a_log[h]) * d);
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const double o = __shfl_up(l, off, WAVE);
+      if (lane >= off) l += o;
+    }
+    const double end = __shfl(l, 63, WAVE);
+    ls[hh][lane] = l;
+    ds[hh][lane] = d;
+    out.w[(slot * a.H + h) * SSD_CHUNK + lane] = d * expf((float)(end - l));
+    out.e[(slot * a.H + h) * SSD_CHUNK + lane] = expf((float)l);
+  }
+  // C_t . B_s for the wave's 16 tokens t and all tiles of s up to its own
+  const size_t col_b = (size_t)a.H * a.P + (size_t)group * a.N, col_c = col_b + (size_t)a.G * a.N;
+  const float* crow = a.xbc + (size_t)min(t0 + 16 * wave + r, last) * a.ld + col_c;
+  const float* brow[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) brow[j] = a.xbc + (size_t)min(t0 + 16 * j + r, last) * a.ld + col_b;
+  f32x4 cb[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) cb[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int n0 = 0; n0 < a.N; n0 += 16) {
+    const f32x4 c = ssd_row4<VEC>(crow, n0 + 4 * g, a.N);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j <= wave) {
+        const f32x4 bv = ssd_row4<VEC>(brow[j], n0 + 4 * g, a.N);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) cb[j] = SSD_MFMA(c[i], bv[i], cb[j]);
+      }
+    }
+  }
+  __syncthreads();
+  for (int hh = 0; hh < nh; ++hh) {
+    float* m = out.m + (slot * a.H + h0 + hh) * (SSD_CHUNK * SSD_CHUNK);
+    double lt[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) lt[i] = ls[hh][16 * wave + 4 * g + i];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j <= wave) {
+        const int s = 16 * j + r;
+        const double lsj = ls[hh][s];
+        const float d = ds[hh][s];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = 16 * wave + 4 * g + i;
+          m[t * SSD_CHUNK + s] = s <= t ? cb[j][i] * expf((float)(lt[i] - lsj)) * d : 0.f;
+        }
+      }
+    }
+  }
+}
+
+// KT: tiles of 16 state rows a wave owns (N <= 64 KT)
+template <int KT, bool VEC>
+__global__ void __launch_bounds__(256) ssd_chunk_walk_kernel(SsdArgs a, SsdChunks in, int p_tiles, int n_seqs) {
+  constexpr int NT = 4 * KT;
+  __shared__ f32x4 states[2][NT * 64];  // the state as the chunk finds it: [tile][lane]
+  // Blocks are dealt over the chip's eight dies in turn, each with a cache of its own: a run of neighbouring heads (which
+  // share B and C, and a head's blocks its M) goes to one die.
+  const int per_seq = a.H * p_tiles;
+  const int b = blockIdx.x / per_seq;
+  int id = blockIdx.x % per_seq;
+  if (a.H % 8 == 0) id = (id % 8) * (per_seq / 8) + id / 8;
+  const int h = id / p_tiles, p0 = (id % p_tiles) * 16;
+  const int t0 = a.seq_starts[b], t1 = a.seq_starts[b + 1];
+  if (t0 >= t1 || a.seq_of_token[t0] < 0) return;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const int N = a.N, P = a.P, last = t1 - 1;
+  const int p = p0 + r;
+  const bool live = p < P;
+  const int group = h / (a.H / a.G);
+  const size_t col_x = (size_t)h * P + (live ? p : 0);
+  const size_t col_b = (size_t)a.H * P + (size_t)group * N, col_c = col_b + (size_t)a.G * N;
+  float* srow = a.state + (((size_t)a.slot_ids[b] * a.H + h) * P + (live ? p : 0)) * N;
+  const float skip = a.skip[h];
+
+  f32x4 S[KT];  // state rows 16 (wave + 4 k) + 4 g + i of channel p
+#pragma unroll
+  for (int k = 0; k < KT; ++k) S[k] = ssd_row4<VEC>(srow, 16 * (wave + 4 * k) + 4 * g, live ? N : 0);
+
+  struct Operands {
+    f32x4 c[NT], m[4], w[4], e;
+    float x[4][4], bb[KT][4][4], end;
+  };
+  auto load = [&](Operands& o, int chunk) {
+    const int tc = t0 + chunk * SSD_CHUNK;
+    const size_t slot = (size_t)ssd_chunk_slot(t0, b, chunk) * a.H + h;
+    const float* crow = a.xbc + (size_t)min(tc + 16 * wave + r, last) * a.ld + col_c;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) o.c[n] = ssd_row4<VEC>(crow, 16 * n + 4 * g, N);
+    const float* m = in.m + slot * (SSD_CHUNK * SSD_CHUNK) + (16 * wave + r) * SSD_CHUNK + 4 * g;
+    const float* w = in.w + slot * SSD_CHUNK + 4 * g;
+    const float* e = in.e + slot * SSD_CHUNK;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      o.m[j] = *reinterpret_cast<const f32x4*>(m + (j <= wave ? 16 * j : 0));  // tiles above the diagonal are not there
+      o.w[j] = *reinterpret_cast<const f32x4*>(w + 16 * j);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float* row = a.xbc + (size_t)min(tc + 16 * j + 4 * g + i, last) * a.ld;
+        o.x[j][i] = row[col_x];
+#pragma unroll
+        for (int k = 0; k < KT; ++k) {
+          const int n = 16 * (wave + 4 * k) + r;
+          o.bb[k][j][i] = n < N ? row[col_b + n] : 0.f;
+        }
+      }
+    }
+    o.e = *reinterpret_cast<const f32x4*>(e + 16 * wave + 4 * g);
+    o.end = e[SSD_CHUNK - 1];
+  };
+  auto work = [&](const Operands& o, int chunk) {
+    f32x4* st = states[chunk & 1];  // the other buffer may still be read by a wave of the chunk before
+#pragma unroll
+    for (int k = 0; k < KT; ++k) st[(wave + 4 * k) * 64 + lane] = S[k];
+    block_sync_lds();
+    f32x4 y0 = f32x4{0.f, 0.f, 0.f, 0.f}, y1 = y0;
+#pragma unroll
+    for (int n = 0; n < NT; n += 2) {
+      const f32x4 s0 = st[n * 64 + lane], s1 = st[(n + 1) * 64 + lane];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        y0 = SSD_MFMA(o.c[n][i], s0[i], y0);
+        y1 = SSD_MFMA(o.c[n + 1][i], s1[i], y1);
+      }
+    }
+    f32x4 y = (y0 + y1) * o.e;
+    f32x4 xt = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j <= wave) {  // uniform over the wave
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y = SSD_MFMA(o.m[j][i], o.x[j][i], y);
+      }
+      if (j == wave) xt = f32x4{o.x[j][0], o.x[j][1], o.x[j][2], o.x[j][3]};
+    }
+#pragma unroll
+    for (int k = 0; k < KT; ++k) S[k] *= o.end;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float xw = o.x[j][i] * o.w[j][i];
+#pragma unroll
+        for (int k = 0; k < KT; ++k) S[k] = SSD_MFMA(o.bb[k][j][i], xw, S[k]);
+      }
+    }
+    const int t = t0 + chunk * SSD_CHUNK + 16 * wave + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (live && t + i <= last) a.y[(size_t)(t + i) * a.H * P + (size_t)h * P + p] = fmaf(skip, xt[i], y[i]);
+  };
+  // the next chunk's operands are asked for before this one is worked on
+  const int chunks = (t1 - t0 + SSD_CHUNK - 1) / SSD_CHUNK;
+  Operands oa, ob;
+  load(oa, 0);
+  for (int c = 0; c < chunks; c += 2) {
+    load(ob, c + 1 < chunks ? c + 1 : c);
+    work(oa, c);
+    if (c + 1 < chunks) {
+      load(oa, c + 2 < chunks ? c + 2 : c + 1);
+      work(ob, c + 1);
+    }
+  }
+  if (live) {
+#pragma unroll
+    for (int k = 0; k < KT; ++k) {
+      const int n = 16 * (wave + 4 * k) + 4 * g;
+      if (VEC) {
+        if (n < N) *reinterpret_cast<f32x4*>(srow + n) = S[k];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (n + i < N) srow[n + i] = S[k][i];
+      }
+    }
+  }
+}
+
+extern "C" long fmsamd_ssd_chunk_workspace(int n_tokens, int n_seqs, int heads) {
+  const long slots = n_tokens / SSD_CHUNK + n_seqs + 1;
+  return slots * heads * (SSD_CHUNK * SSD_CHUNK + 2 * SSD_CHUNK) * (long)sizeof(float);
+}
+
+extern "C" int fmsamd_ssd_chunked(const float* xbc, long ld, const float* dt, long ld_dt, const float* a_log, const float* dt_bias,
+                                  const float* skip, float* state, float* y, const int* seq_starts, const int* seq_of_token,
+                                  const int* slot_ids, int n_seqs, int heads, int vdim, int groups, int n_state, int n_tokens, int longest,
+                                  float* workspace, long workspace_bytes, hipStream_t stream) {
+  if (n_seqs == 0 || n_tokens == 0) return 0;
+  SsdArgs a{xbc, ld, dt, ld_dt, a_log, dt_bias, skip, state, y, seq_starts, seq_of_token, slot_ids, heads, vdim, groups, n_state};
+  if (ssd_check("ssd_chunked", a, n_seqs)) return -1;
+  FMS_REQUIRE(longest > 0 && longest <= n_tokens, "ssd_chunked: a longest sequence of %d in %d tokens", longest, n_tokens);
+  FMS_REQUIRE(workspace != nullptr && workspace_bytes >= fmsamd_ssd_chunk_workspace(n_tokens, n_seqs, heads) && (uintptr_t)workspace % 16 == 0,
+              "ssd_chunked: the workspace is too small");
+  const long slots = n_tokens / SSD_CHUNK + n_seqs + 1;
+  SsdChunks c{workspace, workspace + slots * heads * SSD_CHUNK * SSD_CHUNK,
+              workspace + slots * heads * (SSD_CHUNK * SSD_CHUNK + SSD_CHUNK)};
+  const int subsets = ceil_div(heads / groups, SSD_HEADS);
+  FMS_REQUIRE(n_seqs <= 65535 && (long)groups * subsets <= 65535, "ssd_chunked: too many sequences or groups for one launch");
+  const int p_tiles = ceil_div(vdim, 16);
+  const long blocks = (long)n_seqs * heads * p_tiles;
+  FMS_REQUIRE(blocks < (1L << 31), "ssd_chunked: too many blocks");
+  const bool vec = n_state % 4 == 0 && ((long)heads * vdim) % 4 == 0 && ld % 4 == 0 && (uintptr_t)xbc % 16 == 0 && (uintptr_t)state % 16 == 0;
+  const dim3 grid(ceil_div(longest, SSD_CHUNK), n_seqs, groups * subsets);
+  if (vec) ssd_chunk_scores_kernel<true><<<grid, 256, 0, stream>>>(a, c, subsets);
+  else ssd_chunk_scores_kernel<false><<<grid, 256, 0, stream>>>(a, c, subsets);
+  FMS_LAUNCH_CHECK("ssd_chunk_scores");
+#define FMS_SSD_WALK(KT)                                                                                       \
+  do {                                                                                                         \
+    if (vec) ssd_chunk_walk_kernel<KT, true><<<(unsigned)blocks, 256, 0, stream>>>(a, c, p_tiles, n_seqs);     \
+    else ssd_chunk_walk_kernel<KT, false><<<(unsigned)blocks, 256, 0, stream>>>(a, c, p_tiles, n_seqs);        \
+  } while (0)
+  if (n_state <= 64) FMS_SSD_WALK(1);
+  else if (n_state <= 128) FMS_SSD_WALK(2);
+  else FMS_SSD_WALK(4);
+#undef FMS_SSD_WALK
+  FMS_LAUNCH_CHECK("ssd_chunk_walk");
   return 0;
 }
 

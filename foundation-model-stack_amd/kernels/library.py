@@ -79,7 +79,13 @@ _SIGNATURES = {
     "fmsamd_gated_head_norm": [P, P, L, P, I, F, I, F, P, I, L, P, I, I, I, P],
     "fmsamd_moe_combine": [P, P, I, P, P, L, P, I, I, I, P, I, P, L, P],
     "fmsamd_talking_attn_generic": [P, L, P, L, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
+    "fmsamd_talking_attn_mfma_fits": [I, I, I],
+    "fmsamd_talking_attn_prefill_fits": [I, I, I],
+    "fmsamd_talking_attn_qblock": [I, I],
+    "fmsamd_talking_attn_prefill": [P, L, P, L, P, P, P, P, I, I, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
+    "fmsamd_talking_attn_decode": [P, L, P, L, P, L, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P],
     "fmsamd_ssd_scan": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "fmsamd_ssd_chunked": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, L, P],
     "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P],
     "fmsamd_probe_read": [P, L, I, I, P, P],
     "fmsamd_probe_mfma": [I, I, I, P, P, P],
@@ -124,6 +130,10 @@ def load(verbose: bool = True) -> ctypes.CDLL:
         lib.fmsamd_latent_attn_workspace.argtypes = [I, I, I, I]
         lib.fmsamd_latent_attn_mfma_fits.restype = c_int
         lib.fmsamd_latent_attn_mfma_fits.argtypes = [I, I]
+        lib.fmsamd_ssd_chunk_workspace.restype = c_long
+        lib.fmsamd_ssd_chunk_workspace.argtypes = [I, I, I]
+        lib.fmsamd_talking_attn_workspace.restype = c_long
+        lib.fmsamd_talking_attn_workspace.argtypes = [I, I, I, I]
         lib.fmsamd_moe_max_tiles.restype = c_int
         lib.fmsamd_moe_max_tiles.argtypes = [I, I, I]
         lib.fmsamd_moe_tile_rows.restype = c_int

@@ -1267,10 +1267,16 @@ def value_head_norm(proj: torch.Tensor, col0: int, heads: int, dim: int, eps: fl
 
 def talking_attention(q: torch.Tensor, positions, seq_of_token, block_table, k_cache: torch.Tensor, v_cache: torch.Tensor,
                       talk: torch.Tensor, sink: Optional[torch.Tensor], nheads: int, kvheads: int, head_dim: int, value_dim: int,
-                      scale: float, window: int = 0, *, decode: bool = False, max_context: int = 0) -> torch.Tensor:
+                      scale: float, window: int = 0, *, decode: bool = False, max_context: int = 0,
+                      qblock_start: Optional[torch.Tensor] = None, qblock_len: Optional[torch.Tensor] = None, qblock_tokens: int = 0,
+                      n_splits: int = 0, force_generic: bool = False) -> torch.Tensor:
     """Causal attention of every token over the cache of its sequence with scores mixed over the heads before the softmax,
     score_h = scale * sum_g talk[h, g] q_g . k_(kv head of g), over the last `window` keys (0: all) -> [T, nheads*value_dim].
-    talk: float32 [nheads, nheads]; sink: float32 [nheads], a logit per head in the denominator only, or None."""
+    talk: float32 [nheads, nheads]; sink: float32 [nheads], a logit per head in the denominator only, or None.
+
+    float32, and bfloat16 of sizes that the matrix-core kernels do not take, run the generic kernel.  bfloat16 prompts run
+    in query blocks (of talking_qblock(...) tokens), decode steps (max_context bounds the contexts) deal the visible keys
+    over n_splits blocks a token (default: as many as fill the GPU)."""
     _need_cuda(q, positions, seq_of_token, block_table, k_cache, v_cache, talk, sink)
     _rows2d("q", q)
     T = q.shape[0]
@@ -1282,6 +1288,31 @@ def talking_attention(q: torch.Tensor, positions, seq_of_token, block_table, k_c
         raise ValueError(f"sink must be a contiguous float32 [{nheads}] tensor")
     out = torch.empty(T, nheads * value_dim, dtype=q.dtype, device=q.device)
     lib = load()
+    if q.dtype == torch.bfloat16 and not force_generic and scale > 0 and q.stride(0) % 8 == 0 and lib.fmsamd_talking_attn_mfma_fits(kvheads, head_dim, value_dim):
+        common = (positions.data_ptr(), seq_of_token.data_ptr())
+        if not decode and qblock_start is not None:
+            _need_i32("qblock_start", qblock_start)
+            _need_i32("qblock_len", qblock_len)
+            if qblock_start.numel() != qblock_len.numel():
+                raise ValueError("a length per query block is needed")
+            check(lib.fmsamd_talking_attn_prefill(q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), *common, qblock_start.data_ptr(),
+                                                  qblock_len.data_ptr(), qblock_start.numel(), int(qblock_tokens), block_table.data_ptr(),
+                                                  block_table.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), talk.data_ptr(), _ptr(sink), T,
+                                                  nheads, kvheads, head_dim, value_dim, float(scale), int(window), _stream()))
+            return out
+        if n_splits <= 0:
+            n_splits = 1
+            if decode:
+                if max_context <= 0:
+                    raise ValueError("decode attention needs max_context (an upper bound of every context length)")
+                n_splits = talking_splits(T, nheads, max_context, window)
+        ws_bytes = lib.fmsamd_talking_attn_workspace(T, nheads, value_dim, n_splits)
+        ws = torch.empty(max(ws_bytes // 4, 1), dtype=torch.float32, device=q.device) if ws_bytes else None
+        check(lib.fmsamd_talking_attn_decode(q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), _ptr(ws), ws_bytes, *common,
+                                             block_table.data_ptr(), block_table.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
+                                             talk.data_ptr(), _ptr(sink), T, nheads, kvheads, head_dim, value_dim, float(scale), int(window),
+                                             int(n_splits), _stream()))
+        return out
     for t0 in range(0, T, 65535):
         n = min(65535, T - t0)
         check(lib.fmsamd_talking_attn_generic(q[t0:].data_ptr(), q.stride(0), out[t0:].data_ptr(), out.stride(0), _code(q.dtype),
@@ -1289,6 +1320,21 @@ def talking_attention(q: torch.Tensor, positions, seq_of_token, block_table, k_c
                                               block_table.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), talk.data_ptr(), _ptr(sink), n,
                                               nheads, kvheads, head_dim, value_dim, float(scale), int(window), _stream()))
     return out
+
+
+def talking_splits(n_tokens: int, nheads: int, max_context: int, window: int) -> int:
+    """How many blocks share a (token, 16 heads) of the decode kernel: enough for some 256 blocks in all, but no wave of a
+    block's four without a tile of 32 keys at the most keys that a query can see."""
+    seen = min(int(max_context), int(window)) if window > 0 else int(max_context)
+    tiles = -(-seen // 32) + 1
+    return max(1, min(-(-256 // (n_tokens * -(-nheads // 16))), -(-tiles // 4), 64))
+
+
+def talking_qblock(nheads: int, kvheads: int, head_dim: int, value_dim: int) -> int:
+    """The number of consecutive query tokens of one sequence that a block of the bfloat16 prompt kernel takes; 0: sizes that
+    it does not take."""
+    lib = load()
+    return lib.fmsamd_talking_attn_qblock(nheads, kvheads) if lib.fmsamd_talking_attn_prefill_fits(kvheads, head_dim, value_dim) else 0
 
 
 def gate_mul(x: torch.Tensor, gate: Optional[torch.Tensor], activation: str = "sigmoid", scale: float = 1.0,
@@ -1444,15 +1490,18 @@ def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, e
 # the state-space recurrence
 # --------------------------------------------------------------------------
 SSD_MAX_STATE = 256
+SSD_CHUNK_FROM = 16  # tokens a sequence: from there on a step runs the recurrence in chunks
 
 
 def ssd(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, skip: torch.Tensor, state: torch.Tensor,
         seq_starts: torch.Tensor, seq_of_token: torch.Tensor, slot_ids: torch.Tensor, n_seqs: int, heads: int, vdim: int, groups: int,
-        n_state: int, longest: int) -> torch.Tensor:
+        n_state: int, longest: int, chunked: Optional[bool] = None) -> torch.Tensor:
     """S <- exp(-exp(a_log) d) S + d x B^T, y = S C + skip x with d = softplus(dt + dt_bias), over the tokens of every sequence
     of the step, from and into state [slots, heads, vdim, n_state] (float32) -> y float32 [T, heads*vdim].  xbc: float32 rows
     [x: heads*vdim | B: groups*n_state | C: groups*n_state]; dt: float32 rows [T, heads] of any stride.  Sequence b owns the
-    token rows seq_starts[b] .. seq_starts[b + 1] and the state of slot_ids[b]; longest: the most tokens a sequence brings."""
+    token rows seq_starts[b] .. seq_starts[b + 1] and the state of slot_ids[b]; longest: the most tokens a sequence brings.
+    chunked: in chunks of 64 tokens as matrix products (default: from SSD_CHUNK_FROM tokens a sequence on), else token by
+    token; the two differ by rounding."""
     _need_cuda(xbc, dt, a_log, dt_bias, skip, state, seq_starts, seq_of_token, slot_ids)
     _rows2d("xbc", xbc)
     _rows2d("dt", dt)
@@ -1473,6 +1522,14 @@ def ssd(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, dt_bias: torch
     if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs or seq_of_token.numel() < T:
         raise ValueError("the step's index arrays are shorter than its sequences or tokens")
     y = torch.empty(T, heads * vdim, dtype=torch.float32, device=xbc.device)
+    if longest >= SSD_CHUNK_FROM if chunked is None else chunked:
+        lib = load()
+        ws_bytes = lib.fmsamd_ssd_chunk_workspace(T, int(n_seqs), heads)
+        ws = torch.empty(ws_bytes // 4, dtype=torch.float32, device=xbc.device)
+        check(lib.fmsamd_ssd_chunked(xbc.data_ptr(), xbc.stride(0), dt.data_ptr(), dt.stride(0), a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(),
+                                     state.data_ptr(), y.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(),
+                                     int(n_seqs), heads, vdim, groups, n_state, T, int(longest), ws.data_ptr(), ws_bytes, _stream()))
+        return y
     check(load().fmsamd_ssd_scan(xbc.data_ptr(), xbc.stride(0), dt.data_ptr(), dt.stride(0), a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(),
                                  state.data_ptr(), y.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(),
                                  int(n_seqs), heads, vdim, groups, n_state, _stream()))

@@ -203,7 +203,7 @@ class MultiHeadAttention(Mixer):
 
     def prefill_qblock(self, n_tokens: int, dtype) -> int:
         if self.talking_heads:
-            return 0
+            return ops.talking_qblock(self.nheads, self.kvheads, self.head_dim, self.value_dim) if dtype == torch.bfloat16 and self.scale > 0 else 0
         if (dtype != torch.bfloat16 or self.head_dim % 16 or self._score_slopes() is not None or self.value_dim != self.head_dim
                 or ((self.keep_first or self.distance_bias is not None) and ops.prefill_extras_are_generic(self.head_dim))
                 or ops.prefill_cap_is_generic(self.head_dim, self.soft_cap)):
@@ -273,9 +273,12 @@ class MultiHeadAttention(Mixer):
         size = 0 if batch.is_decode else self.prefill_qblock(batch.n_tokens, x.dtype)
         qb_start, qb_len = batch.qblocks.get(size, (None, None))
         if self.talking_heads:
+            size = 0 if batch.is_decode else self.prefill_qblock(batch.n_tokens, x.dtype)
+            qb_start, qb_len = batch.qblocks.get(size, (None, None))
             mixed = ops.talking_attention(qkv, batch.positions, batch.seq_of_token, table, cache.keys, cache.values, self._talk, self._sink,
                                           H, K, D, self.value_dim, self.scale, self.window, decode=batch.is_decode,
-                                          max_context=batch.context_bound)
+                                          max_context=batch.context_bound, qblock_start=qb_start, qblock_len=qb_len,
+                                          qblock_tokens=size)
             if gate is not None or out is not None or out_scale != 1.0:
                 mixed = ops.gate_mul(mixed, gate, "sigmoid", out_scale, out=out, group=self.value_dim if self.gate_per_head else 1)
             return BranchOutput(mixed, self.dense)

@@ -2,8 +2,8 @@
 
 It is the yardstick of the tests and shares nothing with the library.  `weights` maps the checkpoint's tensor names to
 tensors, `config` is the dictionary of config.json.  Everything runs in float64 unless the caller asks for the
-roundings of a bfloat16 model (`rounding="bfloat16"`: what a product or an activation leaves is stored in bfloat16;
-scores, softmax, norms, angles, decays, step sizes, the recurrences with their states and the residual sum stay as they
+roundings of a bfloat16 model (`rounding="bfloat16"`: what a product or an activation leaves is stored in bfloat16, or a
+number: in its place random errors of that size, drawn from that seed; scores, softmax, norms, angles, decays, step sizes, the recurrences with their states and the residual sum stay as they
 are).
 
 Notation: x is the residual stream [T, width]; h what a mixer or a feed-forward reads; t, i a token's position, j a
@@ -23,6 +23,12 @@ _store = lambda x: x  # noqa: E731
 
 def _bf16(x):
     return x.to(torch.bfloat16).to(x.dtype)
+
+
+def _noise(seed):
+    """In the place of rounding: random errors of the size that bfloat16 storage makes."""
+    gen = torch.Generator().manual_seed(seed)
+    return lambda x: x * (1 + (torch.rand(x.shape, generator=gen, dtype=x.dtype) * 2 - 1) * (0.75 * 2.0 ** -8))
 
 
 def load_model_folder(folder):
@@ -218,7 +224,7 @@ def under(weights, prefix):
 def forward(config, weights, ids, rounding=None, layers_out=None):
     """Logits [T, vocab] of one sequence of token ids; `layers_out` (a list) receives the stream after every layer run."""
     global _store
-    _store = _bf16 if rounding == "bfloat16" else (lambda t: t)
+    _store = _bf16 if rounding == "bfloat16" else (_noise(rounding) if isinstance(rounding, int) else (lambda t: t))
     try:
         eps = config["norm"]["eps"]
         ids = torch.as_tensor(ids, dtype=torch.long)
