@@ -29,6 +29,12 @@ is the same comparison for Basopel (attention in chunks with a sink, in a window
 distance, and over a latent; layer norms on both sides of every branch) beside Llama of the same width, depth, heads and
 gated feed-forward; every attention call is priced by the keys its own mask shows.
 
+    python bench.py --zimorax [--layers N]
+
+is the same comparison for Zimorax (the Mamba-2 recurrence, a gated delta rule, windowed attention whose scores are mixed
+over the heads, looped layers, a plain feed-forward) beside Defapel, the closest model of the library (windowed attention
+beside a gated delta rule), with the same width, depth, heads, window and delta sizes.
+
     python bench.py --sidalorn [--layers N]
 
 is the same comparison for Sidalorn (attention without positions over a latent, a real-gated recurrent block, norms in
@@ -78,6 +84,7 @@ def main() -> int:
     ap.add_argument("--zodolorn", action="store_true",
                     help="another workload: Zodolorn beside Llama at equal layer sizes, with every kernel class's distance from its roofline")
     ap.add_argument("--basopel", action="store_true", help="another workload: Basopel beside Llama at equal layer sizes, likewise")
+    ap.add_argument("--zimorax", action="store_true", help="another workload: Zimorax beside Defapel at equal layer sizes, likewise")
     ap.add_argument("--defapel", action="store_true", help="another workload: Defapel beside Llama at equal layer sizes, likewise")
     ap.add_argument("--sidalorn", action="store_true", help="another workload: Sidalorn beside Zodolorn at equal layer sizes, likewise")
     args = ap.parse_args()
@@ -91,8 +98,9 @@ def main() -> int:
         print(f"bench.py measures one GPU: this library runs on a single MI355X, --gpus {args.gpus} is not supported")
         return 2
 
-    if args.zodolorn or args.defapel or args.sidalorn or args.basopel:
-        return design_comparison(args, "zodolorn" if args.zodolorn else ("defapel" if args.defapel else ("sidalorn" if args.sidalorn else "basopel")))
+    for design in ("zodolorn", "defapel", "sidalorn", "basopel", "zimorax"):
+        if getattr(args, design):
+            return design_comparison(args, design)
 
     import torch
 
@@ -334,6 +342,15 @@ DEFAPEL_SIZES = [
 ]
 
 
+# (name, width, layer pattern (m: mamba2, d: delta, a: attention with mixed scores), heads, kv heads, head size, window,
+#  feed-forward, (mamba2 heads, channels a head, state, groups), delta heads, delta q/k heads, key channels, value channels;
+#  of the model beside it: experts, top, expert ff), vocabulary
+ZIMORAX_SIZES = [
+    ("w2048", 2048, "mmda", 16, 4, 128, 1024, 8192, (64, 64, 128, 8), 16, 8, 128, 128, 32, 4, 1024, 32768),
+    ("w4096", 4096, "mmda", 32, 8, 128, 1024, 12288, (128, 64, 128, 8), 32, 16, 128, 128, 64, 6, 1536, 32768),
+]
+
+
 # (name, width, layer pattern, heads, [dim, vdim, kv_rank], recurrent channels, blocks, dense ff, experts, identity experts, top,
 #  expert ff, shared ff, groups, groups kept, norm groups, vocabulary)
 SIDALORN_SIZES = [
@@ -406,6 +423,14 @@ def design_comparison(args, design) -> int:
             vector_flops = 8.0 * qkv.shape[0] * H * D * V
             # priced at the float32 vector rate (the recurrence runs there), in units of the matrix rate the ideal is formed with
             return nbytes(qkv, a[1], a[2], out) + 2 * n_seqs * (st.numel() // st.shape[0]) * 4, vector_flops * mfma_flops / PEAK_FLOPS["fp32"]
+        if name == "talking_attention":  # scores of every head, mixed over the heads (heads x heads a key), values
+            H, K, D, V = a[8:12]
+            read, loaded = keys_of_call([None] * 10 + [a[13]], {})
+            return 2 * loaded * K * (D + V) + nbytes(a[0][:, : H * D], out), 2.0 * read * H * (D + H + V)
+        if name == "ssd":  # state read and written once a sequence; per token and head 3 passes over vdim x state in float32
+            st, n_seqs, H, P, N = a[5], a[9], a[10], a[11], a[13]
+            vector_flops = 5.0 * a[0].shape[0] * H * P * N
+            return nbytes(a[0], a[1], out) + 2 * n_seqs * (st.numel() // st.shape[0]) * 4, vector_flops * mfma_flops / PEAK_FLOPS["fp32"]
         if name == "latent_attention":  # one row of rank + rot a key, and the latent once more as values
             H, R, P = a[6], a[7], a[8]
             read, loaded = keys_of_call(a, kw)
@@ -431,11 +456,12 @@ def design_comparison(args, design) -> int:
                "moe_route", "moe_combine", "add_norm", "norm_add_norm", "rms_norm_cols", "rope_kv_write", "qkv_rope_write",
                "latent_kv_write", "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "norm_add_norm_affine",
                "delta_rule", "delta_prepare", "gated_head_norm", "qk_projection_norm", "gate_mul", "scale_", "cast", "cast_cols",
-               "rglru_gates", "rglru_scan", "short_conv", "group_norm_chain", "poly_norm", "moe_route_grouped"]
+               "rglru_gates", "rglru_scan", "short_conv", "group_norm_chain", "poly_norm", "moe_route_grouped", "talking_attention", "ssd",
+               "gated_group_norm", "value_head_norm", "stream_rows"]
     small = {"moe_route", "moe_combine", "add_norm", "norm_add_norm", "norm_add_norm_affine", "rms_norm_cols", "rope_kv_write", "latent_kv_write",
              "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "delta_prepare", "gated_head_norm",
              "qk_projection_norm", "gate_mul", "scale_", "cast", "cast_cols", "short_conv", "group_norm_chain", "poly_norm",
-             "moe_route_grouped"}
+             "moe_route_grouped", "gated_group_norm", "value_head_norm", "stream_rows"}
 
     def classes_of_a_step(run):
         """{class: (ms, ms at the roofline)} of the kernels of `run()`, by events around every call into the library."""
@@ -533,9 +559,40 @@ def design_comparison(args, design) -> int:
             torch.cuda.empty_cache()
         return out
 
-    record = {"workload": f"{design} beside {'zodolorn' if design == 'sidalorn' else 'llama'} at equal layer sizes", "layers": layers, "dtype": "bf16",
+    beside = {"sidalorn": "zodolorn", "zimorax": "defapel"}.get(design, "llama")
+    record = {"workload": f"{design} beside {beside} at equal layer sizes", "layers": layers, "dtype": "bf16",
               "data": "synthetic: random weights N(0, 0.02), uniform random token ids",
               "peak_measured": {"read_gbs": round(read_bps / 1e9, 1), "mfma_tflops": round(mfma_flops / 1e12, 1)}, "sizes": {}}
+    if design == "zimorax":
+        from fms_amd.architectures.defapel import make_config as make_defapel
+        from fms_amd.architectures.zimorax import make_config as make_zimorax
+
+        for (name, width, pattern, heads, kv, dim, window, ff, (mheads, mvdim, mstate, mgroups), dheads, dkv, ddim, dvdim, experts, top,
+             expert_ff, vocab) in ZIMORAX_SIZES:
+            pattern = (pattern * layers)[:layers]
+            loop = {"start": 1, "stop": layers, "times": 1} if layers > 1 else None  # every layer runs once, as the other model's do
+            config = make_zimorax(width=width, vocab=vocab, pattern=pattern, heads=heads, kv_heads=kv, dim=dim, vdim=dim, window=window, ff=ff,
+                                  mamba_heads=mheads, mamba_vdim=mvdim, state=mstate, groups=mgroups, norm_groups=mgroups, delta_heads=dheads,
+                                  delta_kv_heads=dkv, delta_dim=ddim, delta_vdim=dvdim, rot_dims=dim // 2, loop=loop, max_positions=context)
+            model = fms_amd.from_config(config, "zimorax", data_type="bf16", random_seed=args.seed)
+            mine = measure(model, vocab, per_call_masks=True)
+            del model
+            torch.cuda.empty_cache()
+            other = make_defapel(width=width, vocab=vocab, pattern=("pppc" * layers)[:layers], heads=heads, kv_heads=kv, dim=dim, vdim=dim,
+                                 window=window, delta_heads=dheads, delta_kv_heads=dkv, delta_dim=ddim, delta_vdim=dvdim, experts=experts,
+                                 top=top, expert_ff=expert_ff, max_positions=context)
+            defapel = fms_amd.from_config(other, "defapel", data_type="bf16", random_seed=args.seed)
+            theirs = measure(defapel, vocab, per_call_masks=True)
+            del defapel
+            torch.cuda.empty_cache()
+            record["sizes"][name] = {"zimorax": dict(config=dict(width=width, pattern=pattern, heads=heads, kv_heads=kv, dim=dim, window=window, ff=ff,
+                                                                   mamba_heads=mheads, mamba_vdim=mvdim, state=mstate, groups=mgroups,
+                                                                   delta_heads=dheads, delta_kv_heads=dkv, delta_dim=ddim, delta_vdim=dvdim,
+                                                                   vocab=vocab), **mine),
+                                     "defapel": dict(config=dict(width=width, heads=heads, kv_heads=kv, dim=dim, window=window, delta_heads=dheads,
+                                                                   experts=experts, top=top, expert_ff=expert_ff, vocab=vocab), **theirs)}
+        print(json.dumps(record))
+        return 0
     if design == "basopel":
         from fms_amd.architectures.basopel import make_config as make_basopel
 
