@@ -431,6 +431,11 @@ def design_comparison(args, design) -> int:
             st, n_seqs, H, P, N = a[5], a[9], a[10], a[11], a[13]
             vector_flops = 5.0 * a[0].shape[0] * H * P * N
             return nbytes(a[0], a[1], out) + 2 * n_seqs * (st.numel() // st.shape[0]) * 4, vector_flops * mfma_flops / PEAK_FLOPS["fp32"]
+        if name == "ssd_step":  # the same for one token a sequence, with the convolution in front of it (its state read once)
+            st, conv, n_seqs, H, P, N = a[9], a[5], a[13], a[14], a[15], a[17]
+            channels = H * P + 2 * a[16] * N
+            state_bytes = 2 * n_seqs * (st.numel() // st.shape[0]) * 4 + (n_seqs * (conv.numel() // conv.shape[0]) * 4 if conv is not None else 0)
+            return state_bytes + a[0].shape[0] * 4 * channels + nbytes(a[3], a[4], out), 5.0 * n_seqs * H * P * N * mfma_flops / PEAK_FLOPS["fp32"]
         if name == "latent_attention":  # one row of rank + rot a key, and the latent once more as values
             H, R, P = a[6], a[7], a[8]
             read, loaded = keys_of_call(a, kw)
@@ -456,7 +461,7 @@ def design_comparison(args, design) -> int:
                "moe_route", "moe_combine", "add_norm", "norm_add_norm", "rms_norm_cols", "rope_kv_write", "qkv_rope_write",
                "latent_kv_write", "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "norm_add_norm_affine",
                "delta_rule", "delta_prepare", "gated_head_norm", "qk_projection_norm", "gate_mul", "scale_", "cast", "cast_cols",
-               "rglru_gates", "rglru_scan", "short_conv", "group_norm_chain", "poly_norm", "moe_route_grouped", "talking_attention", "ssd",
+               "rglru_gates", "rglru_scan", "short_conv", "group_norm_chain", "poly_norm", "moe_route_grouped", "talking_attention", "ssd", "ssd_step",
                "gated_group_norm", "value_head_norm", "stream_rows"]
     small = {"moe_route", "moe_combine", "add_norm", "norm_add_norm", "norm_add_norm_affine", "rms_norm_cols", "rope_kv_write", "latent_kv_write",
              "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "delta_prepare", "gated_head_norm",

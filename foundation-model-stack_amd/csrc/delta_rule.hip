@@ -309,7 +309,7 @@ extern "C" int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const
                                     int conv_dtype, int taps, const float* a_log, const float* dt_bias, float* conv_state,
                                     const int* seq_of_token, const int* slot_ids, float* qkv, float* beta, float* decay,
                                     float* kq, int n_tokens, int heads, int kv_heads, int dim, int vdim, int per_channel,
-                                    float q_scale, hipStream_t stream) {
+                                    float q_scale, const int* seq_starts, int n_seqs, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   FMS_REQUIRE(n_tokens > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0,
               "delta_prepare: bad sizes heads=%d kv_heads=%d dim=%d vdim=%d", heads, kv_heads, dim, vdim);
@@ -318,6 +318,7 @@ extern "C" int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const
   FMS_REQUIRE(ld >= C && col_b >= 0 && col_b + heads <= ld, "delta_prepare: rows of %ld for %ld channels", ld, C);
   FMS_REQUIRE(C * 4 <= 64 * 1024, "delta_prepare: %ld channels do not fit one block's LDS", C);
   FMS_REQUIRE(col_a >= 0 && col_a + heads * (per_channel ? dim : 1) <= lda, "delta_prepare: the decay's columns leave its rows");
+  FMS_REQUIRE(seq_starts == nullptr || n_seqs > 0, "delta_prepare: no sequences");
   const size_t lds = (size_t)C * sizeof(float);
   const int threads = n_tokens <= 64 ? 1024 : 256;
 #define FMS_PREP(W)                                                                                                   \
@@ -330,7 +331,7 @@ extern "C" int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const
 #undef FMS_PREP
   FMS_LAUNCH_CHECK("delta_prepare");
   if (taps > 1) {
-    conv_state_kernel<<<n_tokens, threads, 0, stream>>>(proj, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, (int)C);
+    move_conv_state(proj, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, (int)C, threads, seq_starts, n_seqs, stream);
     FMS_LAUNCH_CHECK("conv_state");
   }
   return 0;

@@ -223,6 +223,8 @@ static void launch_add_norm(float* resid, const void* branch, const void* weight
     // 4 vectors of 4 per thread cover the row up to 16 elements per thread; wider rows take more threads
     int threads = (width / 16 + 63) / 64 * 64;
     threads = threads < 64 ? 64 : (threads > 1024 ? 1024 : threads);
+    // few rows (a decode step): a vector a thread, so that no thread makes several passes one after the other
+    if (n_out <= 256 && width <= 4096) threads = (width / 4 + 63) / 64 * 64;
     add_norm_kernel<4, BranchT, WeightT, OutT><<<n_out, threads, 0, stream>>>(
         resid, (const BranchT*)branch, (const WeightT*)weight, (const WeightT*)bias, (OutT*)out, rows, width, eps,
         use_mean, branch_scale);

@@ -128,9 +128,10 @@ typedef struct {
 
 // At most 192 rows: the weights stream once through MFMA registers.  From 17 rows on the product needs a
 // workspace of fmsamd_gemm_skinny_workspace(M, rows of W, K) bytes (slices of K meet there).
+// out = act(x W^T + bias), act FMS_ACT_IDENTITY, _RELU or _RELU2.
 long fmsamd_gemm_skinny_workspace(int M, int rows, int K);
 int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
-                            int out_dtype, long ldo, int M, int N, int K, const fmsamd_row_scale* row_scale,
+                            int out_dtype, long ldo, int M, int N, int K, int act, const fmsamd_row_scale* row_scale,
                             void* workspace, long workspace_bytes, hipStream_t stream);
 int fmsamd_gemm_skinny_gated_bf16(const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
                                   int out_dtype, long ldo, int M, int hidden, int K, int act,
@@ -301,12 +302,13 @@ int fmsamd_cast_cols(const float* x, long ldx, void* out, int out_dtype, long ld
 // convolution and whose columns col_b .. col_b + heads are the logits of beta; a: rows with the decay's input at col_a
 // (heads columns, or heads*dim if per_channel); conv_w [C, taps]; conv_state [slots][taps-1][C] is read, then updated.
 // Writes qkv [T, C] (convolved, silu, q and k unit vectors per head, q times q_scale), beta [T, heads] and
+// (seq_starts [n_seqs + 1] or null: where the sequences start; the state is then moved on by their last tokens' blocks only)
 // decay [T, heads (*dim)] = exp(-exp(a_log) softplus(a + dt_bias)), and kq [T, kv_heads] = k . q of the finished vectors.
 int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const float* a, long lda, int col_a, const void* conv_w,
                          int conv_dtype, int taps, const float* a_log, const float* dt_bias, float* conv_state,
                          const int* seq_of_token, const int* slot_ids, float* qkv, float* beta, float* decay, float* kq,
                          int n_tokens, int heads, int kv_heads, int dim, int vdim, int per_channel, float q_scale,
-                         hipStream_t stream);
+                         const int* seq_starts, int n_seqs, hipStream_t stream);
 // The recurrence over every sequence's tokens of the step (seq_starts [n_seqs + 1]); state [slots][heads][vdim][dim]
 // is read and written; out [T, heads*vdim].  single_tokens != 0: the caller knows that no sequence brings more than one
 // token, and the kernel stages accordingly (the result is the same either way).
@@ -331,10 +333,12 @@ int fmsamd_group_norm_chain(float* resid, const void* branch, int act_dtype, con
                             void* out, int out_mode, const int* rows, int n_out, int width, hipStream_t stream);
 // out[t, c] = act((x[t, c] if add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c]) over a sequence's own tokens; the
 // inputs before the step come from conv_state [slots][taps-1][channels] (float32), which is then moved on.  x: float32 rows.
+// act: FMS_ACT_IDENTITY or FMS_ACT_SILU.  seq_starts [n_seqs + 1] (or null): the sequences' first token rows; the state is
+// then moved on by blocks for the sequences' last tokens only, not by one for every token.
 // single_tokens: the caller knows that every sequence brings one token (a short step then needs no second kernel for the state).
 int fmsamd_short_conv(const float* x, long ld, int channels, const void* conv_w, const void* bias, int weight_dtype, int taps,
                       float* conv_state, const int* seq_of_token, const int* slot_ids, int add_input, void* out, int out_dtype,
-                      long ldo, int n_tokens, int single_tokens, int act, hipStream_t stream);
+                      long ldo, int n_tokens, int single_tokens, int act, const int* seq_starts, int n_seqs, hipStream_t stream);
 
 // ---- the real-gated linear recurrent unit (rglru.hip) -------------------------------------------------------------------
 // u: float32 rows; ra_t, ri_t [blocks][in][out] (transposed square matrices), ra_b, ri_b, lam float32 [channels];
@@ -363,11 +367,9 @@ int fmsamd_talking_attn_generic(const void* q, long q_stride, void* out, long ou
                                 const void* v_cache, const float* talk, const float* sink, int n_tokens, int nheads, int kvheads,
                                 int head_dim, int value_dim, float scale, int window, hipStream_t stream);
 // The same for bfloat16 on the matrix cores, for sizes of which ..._fits says so (rows: multiples of 8; the scale positive).
-// Prompts: the step is cut into query blocks of at most ..._qblock(...) consecutive tokens of one sequence; sizes that fit
-// the decode kernel only (prefill_fits says 0) run prompts through it.  Decode: a block per (token, 16 heads, split), the
+// Prompts: the step is cut into query blocks of at most ..._qblock(...) consecutive tokens of one sequence.  Decode: a block per (token, 16 heads, split), the
 // visible keys of every sequence dealt over the splits; more than one split needs a workspace of ..._workspace(...) bytes.
 int fmsamd_talking_attn_mfma_fits(int kvheads, int head_dim, int value_dim);
-int fmsamd_talking_attn_prefill_fits(int kvheads, int head_dim, int value_dim);
 int fmsamd_talking_attn_qblock(int nheads, int kvheads);
 int fmsamd_talking_attn_prefill(const void* q, long q_stride, void* out, long out_stride, const int* positions,
                                 const int* seq_of_token, const int* qblock_start, const int* qblock_len, int n_qblocks,
@@ -395,9 +397,18 @@ int fmsamd_ssd_chunked(const float* xbc, long ld, const float* dt, long ld_dt, c
                        float* state, float* y, const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
                        int vdim, int groups, int n_state, int n_tokens, int longest, float* workspace, long workspace_bytes,
                        hipStream_t stream);
-// out = N(y * silu(z)) * weight, N dividing each of `parts` equal parts of a row by its own root mean square; z: float32 rows
+// One token a sequence (a decode step), with the convolution (bias, silu) that makes xbc: proj float32 rows with the channels
+// [x | B | C] before the convolution at col_x and dt at col_dt.  conv_state [slots][taps-1][channels] is read and not moved.
+int fmsamd_ssd_step(const float* proj, long ld, int col_x, int col_dt, const void* conv_w, const void* conv_b, int weight_dtype, int taps,
+                    const float* conv_state, const float* a_log, const float* dt_bias, const float* skip, float* state, float* y,
+                    const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads, int vdim, int groups,
+                    int n_state, hipStream_t stream);
+// out = N(y * silu(z)) * weight, N dividing each of `parts` equal parts of a row by its own root mean square; z: float32 rows.
+// conv_x (or null): the same launch moves the state of a convolution on by one token a sequence (float32 rows ld_conv apart,
+// conv_state [slots][taps-1][channels]).
 int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void* weight, int weight_dtype, int parts, float eps,
-                            void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, hipStream_t stream);
+                            void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, const float* conv_x, long ld_conv,
+                            int channels, int taps, float* conv_state, const int* slot_ids, hipStream_t stream);
 
 #ifdef __cplusplus
 }

@@ -510,7 +510,7 @@ __global__ void __launch_bounds__(SK_WAVES* WAVE)
     } else {
       if (!live) continue;
       if (bias) v += to_f32(bias[n]);
-      out[(size_t)m * ldo + n] = from_f32<OutT>(v);
+      out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v, act));
     }
   }
 }
@@ -588,12 +588,13 @@ static int row_scale_of(const fmsamd_row_scale* in, int K, RowScale* out) {
   return 0;
 }
 
-// out[M, N] = x[M, K] w[N, K]^T (+ bias).  M <= 192.
+// out[M, N] = act(x[M, K] w[N, K]^T (+ bias)).  M <= 192.
 extern "C" int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, const void* bias, int bias_dtype,
-                                       void* out, int out_dtype, long ldo, int M, int N, int K,
+                                       void* out, int out_dtype, long ldo, int M, int N, int K, int act,
                                        const fmsamd_row_scale* row_scale, void* workspace, long workspace_bytes,
                                        hipStream_t stream) {
   if (M == 0 || N == 0) return 0;
+  FMS_REQUIRE(act == FMS_ACT_IDENTITY || act == FMS_ACT_RELU || act == FMS_ACT_RELU2, "gemm_skinny_bf16: activation %d is none that it finishes with", act);
   RowScale scale;
   if (row_scale_of(row_scale, K, &scale)) return -1;
   FMS_REQUIRE(M > 0 && M <= FMS_SKINNY_MAX_ROWS && N > 0 && K > 0, "gemm_skinny_bf16: bad sizes M=%d N=%d K=%d (M <= 192)", M, N, K);
@@ -601,11 +602,11 @@ extern "C" int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, c
   FMS_REQUIRE(ldx >= K && ldo >= N, "gemm_skinny_bf16: leading dimensions too small");
   FMS_REQUIRE(out_dtype == FMS_BF16 || out_dtype == FMS_F32, "gemm_skinny_bf16: unknown output dtype %d", out_dtype);
   if (M > 16 && !skinny_takes_many_rows(M, N, K))
-    return wide_product(EPI_PLAIN, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, 0, scale, RopeEpilogue{},
+    return wide_product(EPI_PLAIN, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, act, scale, RopeEpilogue{},
                         ResidEpilogue{}, workspace, workspace_bytes, stream);
   const int rows = skinny_rows_per_block(N, M);
 #define FMS_LS(NTB, MT) \
-  launch_skinny<NTB, MT, EPI_PLAIN>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, 0, rows, stream, scale)
+  launch_skinny<NTB, MT, EPI_PLAIN>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, act, rows, stream, scale)
 #define FMS_LS_MT(NTB)  \
   do {                  \
     if (M <= 16)        \

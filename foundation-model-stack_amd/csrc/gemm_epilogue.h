@@ -10,8 +10,16 @@ __device__ __forceinline__ float sk_activate(float x, int kind) {
   return fms_activate(x, kind);
 }
 
+// The activations that a plain product finishes with (the others are a kernel of their own behind it: a switch over all of
+// them at every store would cost every product).
+__device__ __forceinline__ float sk_plain(float x, int act) {
+  if (act == FMS_ACT_IDENTITY) return x;
+  const float r = fmaxf(x, 0.f);
+  return act == FMS_ACT_RELU2 ? r * r : r;
+}
+
 // What the skinny kernel does with a finished output element.
-#define EPI_PLAIN 0  // store (+ bias)
+#define EPI_PLAIN 0  // store act(product + bias), act one of identity, relu and its square
 #define EPI_GATED 1  // the block's second tile is the "up" half: out = act(first) * second, N is the hidden size
 #define EPI_ROPE 2   // the output row is [queries | keys | values] of attention: rotate q and k, store q, and
                      // write k and v into their cache pages (layout: see rope.hip)

@@ -332,6 +332,7 @@ __global__ void __launch_bounds__(512)
         for (int e = 0; e < 4; ++e) {
           v[e] *= rs;
           if (o.bias != nullptr && n + e < n_lim) v[e] += wide_bias(o, n + e);
+          v[e] = sk_plain(v[e], o.act);
         }
         OutT* const out = (OutT*)o.out;
         if (o.vec && n + 3 < n_lim) {
@@ -475,7 +476,7 @@ __global__ void __launch_bounds__(256)
     if ((lane & 15) == 0 && n / 16 < res.tiles) res.partials[(size_t)m * res.tiles + n / 16] = sq;
   } else {
     if (!live) return;
-    out[(size_t)m * ldo + n] = from_f32<OutT>(v + bias_v);
+    out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v + bias_v, act));
   }
 }
 
@@ -617,7 +618,7 @@ int wide_product(int epi, const void* x, long ldx, const void* w, const void* bi
   FMS_LAUNCH_CHECK("wide product");
   switch (epi) {
     case EPI_PLAIN:
-      launch_finish<EPI_PLAIN>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, 0, scale, rope, res, stream);
+      launch_finish<EPI_PLAIN>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, act, scale, rope, res, stream);
       break;
     case EPI_GATED:
       launch_finish<EPI_GATED>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, tile2_offset, act, scale,

@@ -238,11 +238,18 @@ extern "C" int fmsamd_group_norm_chain(float* resid, const void* branch, int act
 }
 
 // A block per token, a thread per channel and pass; all taps of a channel are asked for before any is used.
-template <typename W, typename T>
+// What a convolution's sum passes (known at compile time: a switch over every activation, unrolled over a tile's rows and
+// channels, would fill the instruction cache).
+template <bool SILU>
+__device__ __forceinline__ float conv_act(float v) {
+  return SILU ? v / (1.f + expf(-v)) : v;
+}
+
+template <typename W, typename T, bool SILU>
 __global__ void __launch_bounds__(1024)
     short_conv_kernel(const float* __restrict__ x, long ld, int C, const W* __restrict__ conv_w, const W* __restrict__ bias,
                       int taps, float* __restrict__ conv_state, const int* __restrict__ seq_of_token,
-                      const int* __restrict__ slot_ids, int add_input, T* __restrict__ out, long ldo, int move_state, int act) {
+                      const int* __restrict__ slot_ids, int add_input, T* __restrict__ out, long ldo, int move_state) {
   const int t = blockIdx.x;
   const int seq = seq_of_token[t];
   T* o = out + (size_t)t * ldo;
@@ -267,7 +274,7 @@ __global__ void __launch_bounds__(1024)
 #pragma unroll
     for (int j = 0; j < CONV_MAX_TAPS; ++j) acc = fmaf(ws[j], xs[j], acc);
     if (add_input) acc += x[(size_t)t * ld + c];
-    o[c] = from_f32<T>(fms_activate(acc, act));
+    o[c] = from_f32<T>(conv_act<SILU>(acc));
     if (move_state) {
       // every sequence brings one token (have == 0): xs[0 .. taps - 2] are the channel's old entries, all read above by
       // this thread, which is their only reader in the step; the new ones are the old ones moved up and the token's own
@@ -284,11 +291,11 @@ __global__ void __launch_bounds__(1024)
 // convolution is run as one of CONV_MAX_TAPS taps whose first weights are zero: every register has a fixed place.
 #define CONV_TILE 16
 
-template <typename W, typename T, int VEC>
+template <typename W, typename T, int VEC, bool SILU>
 __global__ void __launch_bounds__(256)
     short_conv_tile_kernel(const float* __restrict__ x, long ld, int C, const W* __restrict__ conv_w, const W* __restrict__ bias,
                            int taps, const float* __restrict__ conv_state, const int* __restrict__ seq_of_token,
-                           const int* __restrict__ slot_ids, int add_input, T* __restrict__ out, long ldo, int n_tokens, int act) {
+                           const int* __restrict__ slot_ids, int add_input, T* __restrict__ out, long ldo, int n_tokens) {
   const int c0 = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
   if (c0 >= C) return;
   const int first = blockIdx.x * CONV_TILE, last = min(first + CONV_TILE, n_tokens);
@@ -351,7 +358,7 @@ __global__ void __launch_bounds__(256)
       for (int d = CONV_MAX_TAPS - 1; d > 0; --d) acc = fmaf(back[d][v], hist[d - 1][v], acc);  // the oldest input first
       acc = fmaf(back[0][v], xs[e][v], acc);
       if (add_input) acc += xs[e][v];
-      o[v] = from_f32<T>(fms_activate(acc, act));  // the same sums in the same order as the kernel of short steps
+      o[v] = from_f32<T>(conv_act<SILU>(acc));  // the same sums in the same order as the kernel of short steps
     }
 #pragma unroll
     for (int d = CONV_MAX_TAPS - 2; d > 0; --d) {
@@ -365,12 +372,15 @@ __global__ void __launch_bounds__(256)
 
 extern "C" int fmsamd_short_conv(const float* x, long ld, int channels, const void* conv_w, const void* bias, int weight_dtype,
                                  int taps, float* conv_state, const int* seq_of_token, const int* slot_ids, int add_input,
-                                 void* out, int out_dtype, long ldo, int n_tokens, int single_tokens, int act, hipStream_t stream) {
+                                 void* out, int out_dtype, long ldo, int n_tokens, int single_tokens, int act,
+                                 const int* seq_starts, int n_seqs, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   FMS_REQUIRE(n_tokens > 0 && channels > 0 && ld >= channels && ldo >= channels, "short_conv: bad sizes T=%d C=%d ld=%ld ldo=%ld",
               n_tokens, channels, ld, ldo);
   FMS_REQUIRE(taps >= 1 && taps <= CONV_MAX_TAPS, "short_conv: %d taps (1 to %d)", taps, CONV_MAX_TAPS);
-  FMS_REQUIRE(act >= 0 && act <= FMS_ACT_LAST, "short_conv: unknown activation %d", act);
+  FMS_REQUIRE(act == FMS_ACT_IDENTITY || act == FMS_ACT_SILU, "short_conv: activation %d is neither identity nor silu", act);
+  FMS_REQUIRE(seq_starts == nullptr || n_seqs > 0, "short_conv: no sequences");
+  const bool silu = act == FMS_ACT_SILU;
   FMS_REQUIRE(taps == 1 || conv_state != nullptr, "short_conv: a convolution of %d taps needs the sequences' state", taps);
   const int threads = n_tokens <= 64 ? 1024 : 256;
   // a step in which every sequence brings one token: the kernel that convolves also moves the state on
@@ -381,14 +391,18 @@ extern "C" int fmsamd_short_conv(const float* x, long ld, int channels, const vo
     const int per_block = 256 * (wide ? 4 : 1);
     const dim3 grid(ceil_div(n_tokens, CONV_TILE), ceil_div(channels, per_block));
     FMS_REQUIRE(grid.y <= 65535, "short_conv: %d channels are too many for one launch", channels);
-#define FMS_CONV_TILE(W, T)                                                                                                          \
-  do {                                                                                                                               \
-    if (wide)                                                                                                                        \
-      short_conv_tile_kernel<W, T, 4><<<grid, 256, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps, conv_state, \
-                                                                seq_of_token, slot_ids, add_input, (T*)out, ldo, n_tokens, act);     \
-    else                                                                                                                             \
-      short_conv_tile_kernel<W, T, 1><<<grid, 256, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps, conv_state, \
-                                                                seq_of_token, slot_ids, add_input, (T*)out, ldo, n_tokens, act);     \
+#define FMS_CONV_TILE2(W, T, V, S)                                                                                                   \
+  short_conv_tile_kernel<W, T, V, S><<<grid, 256, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps, conv_state,   \
+                                                               seq_of_token, slot_ids, add_input, (T*)out, ldo, n_tokens)
+#define FMS_CONV_TILE(W, T)                    \
+  do {                                         \
+    if (wide) {                                \
+      if (silu) FMS_CONV_TILE2(W, T, 4, true); \
+      else FMS_CONV_TILE2(W, T, 4, false);     \
+    } else {                                   \
+      if (silu) FMS_CONV_TILE2(W, T, 1, true); \
+      else FMS_CONV_TILE2(W, T, 1, false);     \
+    }                                          \
   } while (0)
     if (weight_dtype == FMS_F32 && out_dtype == FMS_F32) FMS_CONV_TILE(float, float);
     else if (weight_dtype == FMS_F32 && out_dtype == FMS_BF16) FMS_CONV_TILE(float, bf16);
@@ -396,16 +410,25 @@ extern "C" int fmsamd_short_conv(const float* x, long ld, int channels, const vo
     else if (weight_dtype == FMS_BF16 && out_dtype == FMS_BF16) FMS_CONV_TILE(bf16, bf16);
     else FMS_REQUIRE(false, "short_conv: unknown dtypes %d %d", weight_dtype, out_dtype);
 #undef FMS_CONV_TILE
+#undef FMS_CONV_TILE2
     FMS_LAUNCH_CHECK("short_conv_tile");
     if (taps > 1) {
-      conv_state_kernel<<<n_tokens, threads, 0, stream>>>(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, channels);
+      move_conv_state(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, channels, threads, seq_starts, n_seqs, stream);
       FMS_LAUNCH_CHECK("conv_state");
     }
     return 0;
   }
-#define FMS_CONV(W, T)                                                                                                     \
-  short_conv_kernel<W, T><<<n_tokens, threads, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps, conv_state, \
-                                                            seq_of_token, slot_ids, add_input, (T*)out, ldo, move_state, act)
+#define FMS_CONV(W, T)                                                                                                              \
+  do {                                                                                                                              \
+    if (silu)                                                                                                                       \
+      short_conv_kernel<W, T, true><<<n_tokens, threads, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps,      \
+                                                                      conv_state, seq_of_token, slot_ids, add_input, (T*)out, ldo,  \
+                                                                      move_state);                                                  \
+    else                                                                                                                            \
+      short_conv_kernel<W, T, false><<<n_tokens, threads, 0, stream>>>(x, ld, channels, (const W*)conv_w, (const W*)bias, taps,     \
+                                                                       conv_state, seq_of_token, slot_ids, add_input, (T*)out, ldo, \
+                                                                       move_state);                                                 \
+  } while (0)
   if (weight_dtype == FMS_F32 && out_dtype == FMS_F32) FMS_CONV(float, float);
   else if (weight_dtype == FMS_F32 && out_dtype == FMS_BF16) FMS_CONV(float, bf16);
   else if (weight_dtype == FMS_BF16 && out_dtype == FMS_F32) FMS_CONV(bf16, float);
@@ -414,7 +437,7 @@ extern "C" int fmsamd_short_conv(const float* x, long ld, int channels, const vo
 #undef FMS_CONV
   FMS_LAUNCH_CHECK("short_conv");
   if (taps > 1 && !move_state) {
-    conv_state_kernel<<<n_tokens, threads, 0, stream>>>(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, channels);
+    move_conv_state(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, channels, threads, seq_starts, n_seqs, stream);
     FMS_LAUNCH_CHECK("conv_state");
   }
   return 0;

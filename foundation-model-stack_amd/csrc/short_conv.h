@@ -22,18 +22,20 @@ __device__ __forceinline__ int tokens_before(const int* __restrict__ seq_of_toke
 }
 
 // Runs after the kernel that convolves the same step (which reads the old state).  The block of a sequence's last
-// token of the step writes; new entry s is either a row of the step or an old entry above s.  x: float32 rows ld
+// token of the step writes (with seq_starts a block in x is a sequence, else a token row; blocks in y deal the channels); new entry s is either a row of the step or an old entry above s.  x: float32 rows ld
 // apart, already offset to the first convolved channel.
 static __global__ void __launch_bounds__(1024)
     conv_state_kernel(const float* __restrict__ x, long ld, int taps, float* __restrict__ conv_state,
-                      const int* __restrict__ seq_of_token, const int* __restrict__ slot_ids, int n_tokens, int C) {
-  const int t = blockIdx.x;
+                      const int* __restrict__ seq_of_token, const int* __restrict__ slot_ids, int n_tokens, int C,
+                      const int* __restrict__ seq_starts = nullptr) {
+  const int t = seq_starts ? seq_starts[blockIdx.x + 1] - 1 : blockIdx.x;
+  if (seq_starts && t < seq_starts[blockIdx.x]) return;
   const int seq = seq_of_token[t];
   if (seq < 0) return;
   if (t + 1 < n_tokens && seq_of_token[t + 1] == seq) return;  // not the sequence's last token of the step
   const int have = tokens_before(seq_of_token, t, seq, taps);
   float* state = conv_state + (size_t)slot_ids[seq] * (taps - 1) * C;
-  for (int c = threadIdx.x; c < C; c += blockDim.x) {
+  for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < C; c += gridDim.y * blockDim.x) {
     float fresh[CONV_MAX_TAPS - 1];  // all of a channel's new entries are read before any is written
 #pragma unroll
     for (int s = 0; s < CONV_MAX_TAPS - 1; ++s) {
@@ -45,4 +47,13 @@ static __global__ void __launch_bounds__(1024)
     for (int s = 0; s < CONV_MAX_TAPS - 1; ++s)
       if (s < taps - 1) state[(size_t)s * C + c] = fresh[s];
   }
+}
+
+// The launch: blocks for the sequences' last tokens where the caller says where sequences start, else one for every token.
+static inline void move_conv_state(const float* x, long ld, int taps, float* conv_state, const int* seq_of_token, const int* slot_ids,
+                                   int n_tokens, int C, int threads, const int* seq_starts, int n_seqs, hipStream_t stream) {
+  if (seq_starts != nullptr)
+    conv_state_kernel<<<dim3(n_seqs, ceil_div(C, 256)), 256, 0, stream>>>(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, C, seq_starts);
+  else
+    conv_state_kernel<<<n_tokens, threads, 0, stream>>>(x, ld, taps, conv_state, seq_of_token, slot_ids, n_tokens, C);
 }

@@ -4,7 +4,8 @@
 //
 // with x of P channels per head, B and C of N channels per group of heads; everything in float32.
 //
-//   ssd_scan:         token by token (decode steps, short portions).  The rows of S never mix, so 16 lanes share a value
+//   ssd_step:         one token a sequence (decode steps), with the short convolution in front of it in the same kernel.
+//   ssd_scan:         token by token (short portions).  The rows of S never mix, so 16 lanes share a value
 //                     channel, each with a run of its N entries in registers.
 //   ssd_chunk_scores, ssd_chunk_walk: long steps, in chunks of 64 tokens as matrix products (float32 matrix instructions:
 //                     true 32-bit products and sums).  With l_t the sum of the chunk's log decays up to and with token t,
@@ -14,11 +15,13 @@
 //                     a sequence's chunks with the state in accumulators, 16 value channels of a head a block.  The sums
 //                     l are kept in float64 until their differences are taken: a chunk may decay by hundreds of e-folds,
 //                     and neighbours' differences are small.
-//   gated_group_norm: y * silu(z), each of `parts` equal parts of the row over its own root mean square, times a weight.
+//   gated_group_norm: y * silu(z), each of `parts` equal parts of the row over its own root mean square, times a weight; in a
+//                     decode step further blocks of the same launch move the convolution's state on.
 //
 // The state is kept [slot][head][value channel][state row], so that a lane's entries are contiguous.
 #include "common.h"
 #include "fmsamd.h"
+#include "short_conv.h"
 
 #define SSD_MAX_STATE 256
 #define SSD_COLS 16  // value channels of a block of the token-by-token kernel
@@ -370,32 +373,252 @@ extern "C" int fmsamd_ssd_chunked(const float* xbc, long ld, const float* dt, lo
   return 0;
 }
 
+// ---- decode steps: one token a sequence ------------------------------------------------------------------------------------
+// The short convolution, its silu, the step sizes and the recurrence of a (sequence, head) in one kernel: a block forms its
+// own 64 value channels and its group's B and C from the projection and the convolution's state (which it only reads: the
+// other heads of the group read it too; conv_move, which runs with the next kernel, moves it on), while its rows of S are on
+// their way.  A row of S is shared by 16 lanes, four neighbouring entries a load.
+struct SsdStep {
+  const float* proj;  // [T, ld]: convolved channels at col_x, step sizes at col_dt
+  long ld;
+  int col_x, col_dt;
+  const void *conv_w, *conv_b;  // [C, taps], [C]
+  int taps;
+  const float* conv_state;  // [slots][taps - 1][C]
+  const float *a_log, *dt_bias, *skip;
+  float *state, *y;
+  const int *seq_starts, *seq_of_token, *slot_ids;
+  int H, P, G, N;
+};
+#define SSD_STEP_ROWS 64  // value channels of a block
+
+template <int K4, bool VEC, typename W>
+__global__ void __launch_bounds__(256) ssd_step_kernel(SsdStep a) {
+  constexpr int TILES = SSD_STEP_ROWS / 16;
+  __shared__ __attribute__((aligned(16))) float u[SSD_STEP_ROWS + 2 * 64 * K4];  // x | B | C, each of B and C padded to 64 K4 entries
+  const int h = blockIdx.x, b = blockIdx.y;
+  const int t = uniform_load(a.seq_starts + b);
+  if (uniform_load(a.seq_of_token + t) < 0) return;
+  const int slot = uniform_load(a.slot_ids + b);
+  const int H = a.H, P = a.P, N = a.N, group = h / (H / a.G), p0 = blockIdx.z * SSD_STEP_ROWS;
+  const int C = H * P + 2 * a.G * N;
+  const int part = threadIdx.x & 15, row = threadIdx.x >> 4;
+  float* const st = a.state + (((size_t)slot * H + h) * P + p0) * N;
+  f32x4 S[TILES][K4];
+#pragma unroll
+  for (int i = 0; i < TILES; ++i) {
+    const int p = i * 16 + row;
+#pragma unroll
+    for (int k = 0; k < K4; ++k) S[i][k] = ssd_row4<VEC>(st + (size_t)(p0 + p < P ? p : 0) * N, 64 * k + 4 * part, p0 + p < P ? N : 0);
+  }
+  const float dt = a.proj[(size_t)t * a.ld + a.col_dt + h] + a.dt_bias[h];
+  const float rate = -expf(a.a_log[h]), skip = a.skip[h];
+  // the convolved channels: 64 of x, then B, then C
+  const float* now = a.proj + (size_t)t * a.ld + a.col_x;
+  const float* old = a.conv_state + (size_t)slot * (a.taps - 1) * C;
+  const W* cw = (const W*)a.conv_w;
+  const W* cbias = (const W*)a.conv_b;
+  for (int i = threadIdx.x; i < SSD_STEP_ROWS + 2 * 64 * K4; i += 256) {
+    int c = -1;
+    if (i < SSD_STEP_ROWS) {
+      if (p0 + i < P) c = h * P + p0 + i;
+    } else {
+      const int j = (i - SSD_STEP_ROWS) % (64 * K4), which = (i - SSD_STEP_ROWS) / (64 * K4);
+      if (j < N) c = H * P + (which * a.G + group) * N + j;
+    }
+    float v = 0.f;
+    if (c >= 0) {
+      float x[CONV_MAX_TAPS], w[CONV_MAX_TAPS];
+#pragma unroll
+      for (int j = 0; j < CONV_MAX_TAPS; ++j) {
+        x[j] = w[j] = 0.f;
+        if (j < a.taps) {
+          x[j] = j == a.taps - 1 ? now[c] : old[(size_t)j * C + c];
+          w[j] = to_f32(cw[(size_t)c * a.taps + j]);
+        }
+      }
+      float acc = to_f32(cbias[c]);
+#pragma unroll
+      for (int j = 0; j < CONV_MAX_TAPS; ++j) acc = fmaf(w[j], x[j], acc);
+      v = acc / (1.f + expf(-acc));
+    }
+    u[i] = v;
+  }
+  __syncthreads();
+  const float d = softplus_f32(dt), decay = expf(rate * d);
+  f32x4 Bv[K4], Cv[K4];
+#pragma unroll
+  for (int k = 0; k < K4; ++k) {
+    Bv[k] = *reinterpret_cast<const f32x4*>(u + SSD_STEP_ROWS + 64 * k + 4 * part);
+    Cv[k] = *reinterpret_cast<const f32x4*>(u + SSD_STEP_ROWS + 64 * K4 + 64 * k + 4 * part);
+  }
+#pragma unroll
+  for (int i = 0; i < TILES; ++i) {
+    const int p = i * 16 + row;
+    const float x = u[p], dx = d * x;
+    float y = 0.f;
+#pragma unroll
+    for (int k = 0; k < K4; ++k) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][k][e] = fmaf(dx, Bv[k][e], decay * S[i][k][e]);
+        y = fmaf(S[i][k][e], Cv[k][e], y);
+      }
+    }
+    y = row16_sum(y);
+    if (p0 + p < P) {
+      if (part == 0) a.y[(size_t)t * H * P + (size_t)h * P + p0 + p] = fmaf(skip, x, y);
+#pragma unroll
+      for (int k = 0; k < K4; ++k) {
+        const int n = 64 * k + 4 * part;
+        float* dst = st + (size_t)p * N + n;
+        if (VEC) {
+          if (n < N) *reinterpret_cast<f32x4*>(dst) = S[i][k];
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (n + e < N) dst[e] = S[i][k][e];
+        }
+      }
+    }
+  }
+}
+
+extern "C" int fmsamd_ssd_step(const float* proj, long ld, int col_x, int col_dt, const void* conv_w, const void* conv_b, int weight_dtype,
+                               int taps, const float* conv_state, const float* a_log, const float* dt_bias, const float* skip, float* state,
+                               float* y, const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
+                               int vdim, int groups, int n_state, hipStream_t stream) {
+  if (n_seqs == 0) return 0;
+  SsdStep a{proj, ld, col_x, col_dt, conv_w, conv_b, taps, conv_state, a_log, dt_bias, skip, state, y, seq_starts, seq_of_token, slot_ids,
+            heads, vdim, groups, n_state};
+  FMS_REQUIRE(n_seqs > 0 && n_seqs <= 65535 && heads > 0 && vdim > 0 && groups > 0 && heads % groups == 0 && n_state > 0 && n_state <= SSD_MAX_STATE,
+              "ssd_step: bad sizes heads=%d vdim=%d groups=%d state=%d", heads, vdim, groups, n_state);
+  const long C = (long)heads * vdim + 2L * groups * n_state;
+  FMS_REQUIRE(col_x >= 0 && col_x + C <= ld && col_dt >= 0 && col_dt + heads <= ld, "ssd_step: the rows do not hold the columns asked for");
+  FMS_REQUIRE(taps >= 1 && taps <= CONV_MAX_TAPS && (taps == 1 || conv_state != nullptr), "ssd_step: %d taps (1 to %d, with a state)", taps, CONV_MAX_TAPS);
+  FMS_REQUIRE(ceil_div(vdim, SSD_STEP_ROWS) <= 65535, "ssd_step: too many value channels");
+  const bool vec = n_state % 4 == 0 && (uintptr_t)state % 16 == 0;
+  const dim3 grid(heads, n_seqs, ceil_div(vdim, SSD_STEP_ROWS));
+#define FMS_STEP(K4)                                                                      \
+  do {                                                                                    \
+    if (weight_dtype == FMS_F32) {                                                        \
+      if (vec) ssd_step_kernel<K4, true, float><<<grid, 256, 0, stream>>>(a);             \
+      else ssd_step_kernel<K4, false, float><<<grid, 256, 0, stream>>>(a);                \
+    } else {                                                                              \
+      if (vec) ssd_step_kernel<K4, true, bf16><<<grid, 256, 0, stream>>>(a);              \
+      else ssd_step_kernel<K4, false, bf16><<<grid, 256, 0, stream>>>(a);                 \
+    }                                                                                     \
+  } while (0)
+  FMS_REQUIRE(weight_dtype == FMS_F32 || weight_dtype == FMS_BF16, "ssd_step: unknown dtype %d", weight_dtype);
+  if (n_state <= 64) FMS_STEP(1);
+  else if (n_state <= 128) FMS_STEP(2);
+  else FMS_STEP(4);
+#undef FMS_STEP
+  FMS_LAUNCH_CHECK("ssd_step");
+  return 0;
+}
+
+// ---- the gated norm --------------------------------------------------------------------------------------------------------
+// A convolution's state to be moved on by one token a sequence (a decode step), by blocks of their own beside the norm's.
+struct ConvMove {
+  const float* x;  // float32 rows ld apart, at the first convolved channel
+  long ld;
+  int channels, taps;
+  float* state;  // [slots][taps - 1][channels]
+  const int* slot_ids;
+};
+__device__ __forceinline__ void conv_move(const ConvMove& m, const int* seq_of_token, int t, int c) {
+  const int seq = seq_of_token[t];
+  if (seq < 0 || c >= m.channels) return;
+  float* st = m.state + (size_t)m.slot_ids[seq] * (m.taps - 1) * m.channels + c;
+  float v[CONV_MAX_TAPS];
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+    if (j < m.taps - 1) v[j] = j + 1 < m.taps - 1 ? st[(size_t)(j + 1) * m.channels] : m.x[(size_t)t * m.ld + c];
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+    if (j < m.taps - 1) st[(size_t)j * m.channels] = v[j];
+}
+
+__device__ __forceinline__ float gated(float y, float z) { return y * (z / (1.f + expf(-z))); }
+
+// A wave per (token, part), for parts of at most 1024 channels: the part's gated values wait in registers, four neighbours a
+// load, and no wave waits for another.  Blocks from norm_blocks on move the convolution's state.
+template <typename T, typename W>
+__global__ void __launch_bounds__(256)
+    gated_group_norm_wave_kernel(const float* __restrict__ y, const float* __restrict__ z, long ldz, const W* __restrict__ weight, float eps,
+                                 T* __restrict__ out, const int* __restrict__ seq_of_token, int n_tokens, int cols, int size, int norm_blocks,
+                                 ConvMove move, int move_blocks) {
+  if ((int)blockIdx.x >= norm_blocks) {
+    const int i = blockIdx.x - norm_blocks;
+    conv_move(move, seq_of_token, i / move_blocks, (i % move_blocks) * 256 + threadIdx.x);
+    return;
+  }
+  const int parts = cols / size;
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63;
+  const int t = (int)(item / parts), part = (int)(item % parts);
+  if (t >= n_tokens || seq_of_token[t] < 0) return;
+  const float* yr = y + (size_t)t * cols + (size_t)part * size;
+  const float* zr = z + (size_t)t * ldz + (size_t)part * size;
+  const W* wr = weight + (size_t)part * size;
+  T* o = out + (size_t)t * cols + (size_t)part * size;
+  f32x4 v[4];
+  float s = 0.f;
+#pragma unroll
+  for (int n = 0; n < 4; ++n) {
+    const int i = (n * 64 + lane) * 4;
+    v[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (i < size) {
+      const f32x4 yv = *reinterpret_cast<const f32x4*>(yr + i), zv = *reinterpret_cast<const f32x4*>(zr + i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[n][e] = gated(yv[e], zv[e]), s = fmaf(v[n][e], v[n][e], s);
+    }
+  }
+  const float inv = 1.f / sqrtf(wave_sum(s) / (float)size + eps);
+#pragma unroll
+  for (int n = 0; n < 4; ++n) {
+    const int i = (n * 64 + lane) * 4;
+    if (i < size) {
+      T r[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r[e] = from_f32<T>(v[n][e] * inv * to_f32(wr[i + e]));
+      if constexpr (sizeof(T) == 2) *reinterpret_cast<bf16x4*>(o + i) = bf16x4{r[0], r[1], r[2], r[3]};
+      else *reinterpret_cast<f32x4*>(o + i) = f32x4{r[0], r[1], r[2], r[3]};
+    }
+  }
+}
+
 // A block per (token, part); the part's gated values wait in registers (up to 16 a thread, the rest is formed again).
 template <typename T, typename W>
 __global__ void __launch_bounds__(1024)
     gated_group_norm_kernel(const float* __restrict__ y, const float* __restrict__ z, long ldz, const W* __restrict__ weight, float eps,
-                            T* __restrict__ out, const int* __restrict__ seq_of_token, int cols, int size) {
+                            T* __restrict__ out, const int* __restrict__ seq_of_token, int cols, int size, int norm_blocks, ConvMove move,
+                            int move_blocks) {
   __shared__ float scratch[17];
   constexpr int KEEP = 16;
-  const int t = blockIdx.x, c0 = blockIdx.y * size;
+  if ((int)blockIdx.x >= norm_blocks) {
+    const int i = blockIdx.x - norm_blocks;
+    const int c = (i % move_blocks) * 256;
+    for (int k = threadIdx.x; k < 256; k += blockDim.x) conv_move(move, seq_of_token, i / move_blocks, c + k);
+    return;
+  }
+  const int parts = cols / size;
+  const int t = blockIdx.x / parts, c0 = (blockIdx.x % parts) * size;
   if (seq_of_token[t] < 0) return;
   const float* yr = y + (size_t)t * cols + c0;
   const float* zr = z + (size_t)t * ldz + c0;
   const W* wr = weight + c0;
   T* o = out + (size_t)t * cols + c0;
-  auto gated = [&](int i) {
-    const float g = zr[i];
-    return yr[i] * (g / (1.f + expf(-g)));
-  };
   float keep[KEEP], s = 0.f;
 #pragma unroll
   for (int n = 0; n < KEEP; ++n) {
     const int i = threadIdx.x + n * blockDim.x;
-    keep[n] = i < size ? gated(i) : 0.f;
+    keep[n] = i < size ? gated(yr[i], zr[i]) : 0.f;
     s = fmaf(keep[n], keep[n], s);
   }
   for (int i = threadIdx.x + KEEP * blockDim.x; i < size; i += blockDim.x) {
-    const float v = gated(i);
+    const float v = gated(yr[i], zr[i]);
     s = fmaf(v, v, s);
   }
   const float inv = 1.f / sqrtf(block_sum(s, scratch) / (float)size + eps);
@@ -404,19 +627,36 @@ __global__ void __launch_bounds__(1024)
     const int i = threadIdx.x + n * blockDim.x;
     if (i < size) o[i] = from_f32<T>(keep[n] * inv * to_f32(wr[i]));
   }
-  for (int i = threadIdx.x + KEEP * blockDim.x; i < size; i += blockDim.x) o[i] = from_f32<T>(gated(i) * inv * to_f32(wr[i]));
+  for (int i = threadIdx.x + KEEP * blockDim.x; i < size; i += blockDim.x) o[i] = from_f32<T>(gated(yr[i], zr[i]) * inv * to_f32(wr[i]));
 }
 
 extern "C" int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void* weight, int weight_dtype, int parts, float eps,
-                                       void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, hipStream_t stream) {
+                                       void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, const float* conv_x,
+                                       long ld_conv, int channels, int taps, float* conv_state, const int* slot_ids, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   FMS_REQUIRE(n_tokens > 0 && cols > 0 && parts > 0 && cols % parts == 0 && ldz >= cols, "gated_group_norm: %d parts of %d channels", parts, cols);
-  FMS_REQUIRE(parts <= 65535, "gated_group_norm: %d parts are too many for one launch", parts);
   const int size = cols / parts;
+  ConvMove move{conv_x, ld_conv, channels, taps, conv_state, slot_ids};
+  int move_blocks = 0;  // a token's
+  if (conv_x != nullptr) {
+    FMS_REQUIRE(taps >= 2 && taps <= CONV_MAX_TAPS && channels > 0 && ld_conv >= channels && conv_state != nullptr && slot_ids != nullptr,
+                "gated_group_norm: a state of %d taps over %d channels", taps, channels);
+    move_blocks = ceil_div(channels, 256);
+  }
+  const bool by_waves = size <= 1024 && size % 4 == 0 && ldz % 4 == 0 && (((uintptr_t)y | (uintptr_t)z | (uintptr_t)out) & 15) == 0;
+  const long norm_blocks = by_waves ? ceil_div((long)n_tokens * parts, 4) : (long)n_tokens * parts;
+  const long blocks = norm_blocks + (long)n_tokens * move_blocks;
+  FMS_REQUIRE(blocks < (1L << 31), "gated_group_norm: too many blocks");
   const int threads = size >= 2048 ? 512 : (size >= 512 ? 256 : 64);
-  const dim3 grid(n_tokens, parts);
-#define FMS_GGN(T, W)                                                                                                             \
-  gated_group_norm_kernel<T, W><<<grid, threads, 0, stream>>>(y, z, ldz, (const W*)weight, eps, (T*)out, seq_of_token, cols, size)
+#define FMS_GGN(T, W)                                                                                                                   \
+  do {                                                                                                                                  \
+    if (by_waves)                                                                                                                       \
+      gated_group_norm_wave_kernel<T, W><<<(unsigned)blocks, 256, 0, stream>>>(y, z, ldz, (const W*)weight, eps, (T*)out, seq_of_token, \
+                                                                               n_tokens, cols, size, (int)norm_blocks, move, move_blocks); \
+    else                                                                                                                                \
+      gated_group_norm_kernel<T, W><<<(unsigned)blocks, threads, 0, stream>>>(y, z, ldz, (const W*)weight, eps, (T*)out, seq_of_token,  \
+                                                                              cols, size, (int)norm_blocks, move, move_blocks);         \
+  } while (0)
   if (out_dtype == FMS_F32 && weight_dtype == FMS_F32) FMS_GGN(float, float);
   else if (out_dtype == FMS_BF16 && weight_dtype == FMS_F32) FMS_GGN(bf16, float);
   else if (out_dtype == FMS_BF16 && weight_dtype == FMS_BF16) FMS_GGN(bf16, bf16);

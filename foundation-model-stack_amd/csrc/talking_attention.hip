@@ -143,24 +143,42 @@ __device__ __forceinline__ bf16x8 talk_mixed_query(const bf16* qrow, const TalkA
   return bf16x8{(bf16)s[0], (bf16)s[1], (bf16)s[2], (bf16)s[3], (bf16)s[4], (bf16)s[5], (bf16)s[6], (bf16)s[7]};
 }
 
-// Prompts.  A block is four waves: `hb` heads of one kv head times 4 / hb runs of 32 consecutive query tokens of one
-// sequence; a wave owns one head and 32 queries (one tile column of the 32x32x16 product).  Tiles of 32 keys (all kv heads'
-// keys, and the values of the block's kv head) go through LDS, two at a time: one is multiplied while the next is written
-// and the one after it is on its way from memory.
+// Prompts.  A block has four units: `hb` heads of one kv head times 4 / hb runs of 32 consecutive query tokens of one
+// sequence.  A unit is one head and 32 queries (one tile column of the 32x32x16 product) and has two waves, which split the
+// entries of the mixed queries (a wave multiplies its half of every key row, and the halves of the scores meet in LDS) and
+// the value channels: a query's mixed row is as long as all kv heads' keys together, and half of it leaves a wave room to be
+// one of two on its SIMD.  Tiles of 32 keys (all kv heads' keys, and the values of the block's kv head) go through LDS: the
+// keys are free as soon as the scores are formed, so the next tile's are written while this one's softmax and second product
+// run, and the tile after that is on its way from memory.
 //
 // Which key sits in which row of the score tile is free: rows are dealt so that a lane's 16 scores are the keys 8 half ..
 // 8 half + 7 and 16 + 8 half .. 16 + 8 half + 7, each eight the operand of one step of the second product.
+#define TALK_UNITS 4
+#define TALK_NOWHERE 0xffff0000u
+#define TALK_PREFILL_THREADS (TALK_UNITS * 2 * WAVE)
+
 template <int KC, int DT>
-__global__ void __launch_bounds__(256)
+struct TalkPrefillLds {
+  static constexpr int KS = KC * 16 + TALK_PAD;     // row stride of the keys [32][KS]
+  static constexpr int VS = TALK_KEYS + TALK_PAD;   // row stride of the transposed values [DT * 32][VS]
+  static constexpr int K_ELEMS = TALK_KEYS * KS, V_ELEMS = DT * 32 * VS;
+  static constexpr int EXCHANGE = TALK_UNITS * 2 * WAVE * 16;  // float32: a score tile's half of every wave
+  static constexpr int BYTES = (K_ELEMS + 2 * V_ELEMS) * 2 + EXCHANGE * 4;
+};
+
+template <int KC, int DT>
+__global__ void __launch_bounds__(TALK_PREFILL_THREADS) __attribute__((amdgpu_waves_per_eu(2, 2)))
     talking_prefill_kernel(TalkArgs a, const int* __restrict__ qblock_start, const int* __restrict__ qblock_len, int n_qblocks, int hb) {
-  constexpr int KW = KC * 16;                   // entries of a key row, padded
-  constexpr int KS = KW + TALK_PAD;             // LDS row stride of the keys [32][KS]
-  constexpr int VS = TALK_KEYS + TALK_PAD;      // LDS row stride of the transposed values [DT * 32][VS]
-  constexpr int K_ELEMS = TALK_KEYS * KS, V_ELEMS = DT * 32 * VS, TILE_ELEMS = K_ELEMS + V_ELEMS;
-  constexpr int KCH = TALK_KEYS * KW / 8 / 256;            // 16-byte pieces a thread moves per key tile
-  constexpr int VCH = (DT * 32 * TALK_KEYS / 8 + 255) / 256;  // ... and per value tile
+  typedef TalkPrefillLds<KC, DT> L;
+  constexpr int KH = KC / 2, DH = (DT + 1) / 2;  // a wave's share of the key entries (steps of 16) and value tiles
+  constexpr bool LATE = KC > 32;  // the longest rows leave the softmax no room for a tile on its way: it is asked for behind it
+  constexpr int KW = KC * 16, KS = L::KS, VS = L::VS;
+  constexpr int KCH = TALK_KEYS * KW / 8 / TALK_PREFILL_THREADS;                                          // 16-byte pieces a thread
+  constexpr int VCH = (DT * 32 * TALK_KEYS / 8 + TALK_PREFILL_THREADS - 1) / TALK_PREFILL_THREADS;  // moves per tile
   extern __shared__ __attribute__((aligned(16))) unsigned char talk_lds[];
-  bf16* const lds = reinterpret_cast<bf16*>(talk_lds);
+  bf16* const ks = reinterpret_cast<bf16*>(talk_lds);
+  bf16* const vs = ks + L::K_ELEMS;  // two of them, in turn
+  f32x4* const exchange = reinterpret_cast<f32x4*>(vs + 2 * L::V_ELEMS);  // [wave][4][lane]
 
   // blocks with the most keys (a causal step's last) are handed out first
   const int per = a.nheads / a.kvheads, tiles = per / hb, per_qb = a.kvheads * tiles;
@@ -168,31 +186,42 @@ __global__ void __launch_bounds__(256)
   const int y = blockIdx.x % per_qb;
   const int kh = y / tiles;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int unit = wave >> 1, side = wave & 1;
   const int j = lane & 31, half = lane >> 5;
-  const int h = kh * per + (y % tiles) * hb + wave % hb;
+  const int h = kh * per + (y % tiles) * hb + unit % hb;
   const int t_begin = qblock_start[qb], t_end = t_begin + qblock_len[qb];
   const int seq = a.seq_of_token[t_begin];
   if (seq < 0) return;  // whole block: uniform
   const int* bt = a.block_table + (size_t)seq * a.table_stride;
   const size_t page_elems = (size_t)a.kvheads * PAGE_TOKENS * a.dim, vpage_elems = (size_t)a.kvheads * PAGE_TOKENS * a.vdim;
 
-  // this wave's queries
-  const int t0 = t_begin + (wave / hb) * 32;
+  // this unit's queries
+  const int t0 = t_begin + (unit / hb) * 32;
   const bool has_work = t0 < t_end;
   const int t = t0 + j;
   const bool valid = t < t_end;
   const int row = a.kvheads * a.dim;  // entries of a key row
-  bf16x8 qreg[KC];
+  // the mixed queries of one unit after the other pass through the keys' place in LDS: all threads form them, the unit's
+  // waves take their halves.  (Their padding leaves zeros behind the keys' entries, which are multiplied by zeros later.)
+  bf16x8 qreg[KH];
+  for (int u = 0; u < TALK_UNITS; ++u) {
+    const int uh = kh * per + (y % tiles) * hb + u % hb, ut = t_begin + (u / hb) * 32;
+    for (int i = threadIdx.x; i < 32 * (KW / 8); i += TALK_PREFILL_THREADS) {
+      const int tok = i / (KW / 8), k = (i % (KW / 8)) * 8;
+      bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (ut + tok < t_end && k < row) v = talk_mixed_query(a.q + (size_t)(ut + tok) * a.q_stride, a, uh, k);
+      *reinterpret_cast<bf16x8*>(ks + tok * KS + k) = v;
+    }
+    __syncthreads();
+    if (u == unit) {
 #pragma unroll
-  for (int c = 0; c < KC; ++c) {
-    const int k = c * 16 + half * 8;
-    bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (valid && k < row) v = talk_mixed_query(a.q + (size_t)t * a.q_stride, a, h, k);
-    qreg[c] = v;
+      for (int c = 0; c < KH; ++c) qreg[c] = talk_load8(ks + j * KS + (side * KH + c) * 16 + half * 8);
+    }
+    __syncthreads();
   }
   const int qpos = valid ? a.positions[t] : -1;
   const int qlo = valid ? talk_first_key(qpos, a.window) : 0;
-  int wave_hi = -1, wave_lo = 0, full_hi = -1, full_lo = 0;  // keys some / every column of the wave sees
+  int wave_hi = -1, wave_lo = 0, full_hi = -1, full_lo = 0;  // keys some / every column of the unit sees
   if (has_work) {
     const int t_last = (t0 + 32 < t_end ? t0 + 32 : t_end) - 1;
     wave_hi = a.positions[t_last];
@@ -203,17 +232,17 @@ __global__ void __launch_bounds__(256)
   const int tile_first = talk_first_key(a.positions[t_begin], a.window) / TALK_KEYS;
   const int tile_last = a.positions[t_end - 1] / TALK_KEYS;
 
-  // where a thread's pieces of a tile lie in the page and in LDS (the same for every tile)
-  int k_src[KCH], k_dst[KCH];
+  // where a thread's pieces of a tile lie in the page and in LDS (the same for every tile), in pieces of eight entries: the
+  // place in LDS in the upper 16 bits (TALK_NOWHERE: the padding has no piece), the one in the page in the lower
+  unsigned k_at[KCH];
   const int d8 = a.dim / 8;
 #pragma unroll
   for (int n = 0; n < KCH; ++n) {
-    const int id = threadIdx.x + n * 256;
+    const int id = threadIdx.x + n * TALK_PREFILL_THREADS;
     const int c = id / (TALK_KEYS * d8), rest = id - c * (TALK_KEYS * d8);
     const int tok = rest / d8, d = rest - tok * d8;
     const bool there = c < a.kvheads;
-    k_src[n] = there ? (c * PAGE_TOKENS + tok) * a.dim + d * 8 : 0;
-    k_dst[n] = there ? tok * KS + c * a.dim + d * 8 : -1;
+    k_at[n] = there ? (unsigned)(tok * (KS / 8) + c * d8 + d) << 16 | (unsigned)((c * PAGE_TOKENS + tok) * d8 + d) : TALK_NOWHERE;
   }
   const int v_pieces = a.vdim * (TALK_KEYS / 8);
   bf16x8 kbuf[KCH], vbuf[VCH];
@@ -224,40 +253,34 @@ __global__ void __launch_bounds__(256)
     const bf16* kp = a.k_cache + phys * page_elems + (size_t)in_page * a.dim;
     const bf16* vp = a.v_cache + phys * vpage_elems + (size_t)kh * a.vdim * PAGE_TOKENS + in_page;
 #pragma unroll
-    for (int n = 0; n < KCH; ++n) kbuf[n] = talk_load8(kp + k_src[n]);
+    for (int n = 0; n < KCH; ++n) kbuf[n] = talk_load8(kp + (size_t)(k_at[n] & 0xffffu) * 8);
 #pragma unroll
     for (int n = 0; n < VCH; ++n) {
-      const int id = threadIdx.x + n * 256;
+      const int id = threadIdx.x + n * TALK_PREFILL_THREADS;
       vbuf[n] = talk_load8(vp + (id < v_pieces ? (size_t)(id / (TALK_KEYS / 8)) * PAGE_TOKENS + (id % (TALK_KEYS / 8)) * 8 : 0));
     }
   };
-  auto stash = [&](int which) {
-    bf16* ks = lds + which * TILE_ELEMS;
-    bf16* vs = ks + K_ELEMS;
+  auto stash = [&](int which) {  // keys into their one place, values into place `which`
 #pragma unroll
     for (int n = 0; n < KCH; ++n)
-      if (k_dst[n] >= 0) *reinterpret_cast<bf16x8*>(ks + k_dst[n]) = kbuf[n];
+      if (k_at[n] != TALK_NOWHERE) *reinterpret_cast<bf16x8*>(ks + (k_at[n] >> 16) * 8) = kbuf[n];
 #pragma unroll
     for (int n = 0; n < VCH; ++n) {
-      const int id = threadIdx.x + n * 256;
-      if (id < v_pieces) *reinterpret_cast<bf16x8*>(vs + (id / (TALK_KEYS / 8)) * VS + (id % (TALK_KEYS / 8)) * 8) = vbuf[n];
+      const int id = threadIdx.x + n * TALK_PREFILL_THREADS;
+      if (id < v_pieces) *reinterpret_cast<bf16x8*>(vs + which * L::V_ELEMS + (id / (TALK_KEYS / 8)) * VS + (id % (TALK_KEYS / 8)) * 8) = vbuf[n];
     }
   };
-  if (row < KW) {  // the padded entries of the key rows are multiplied by zeros: they must be numbers
-    for (int i = threadIdx.x; i < 2 * TALK_KEYS * (KW - row); i += 256) {
-      const int which = i / (TALK_KEYS * (KW - row)), rest = i % (TALK_KEYS * (KW - row));
-      lds[which * TILE_ELEMS + (rest / (KW - row)) * KS + row + rest % (KW - row)] = (bf16)0.f;
-    }
-  }
-
-  f32x16 acc[DT];
+  f32x16 acc[DH];
 #pragma unroll
-  for (int dt = 0; dt < DT; ++dt)
+  for (int dt = 0; dt < DH; ++dt)
 #pragma unroll
     for (int v = 0; v < 16; ++v) acc[dt][v] = 0.f;
   float m = TALK_EMPTY, l = 0.f;
   const float scale2 = a.scale * TALK_LOG2E;
   const int key_row = 16 * (j >> 4) + 8 * ((j >> 2) & 1) + 4 * ((j >> 3) & 1) + (j & 3);
+  const bf16* const kbase = ks + (size_t)key_row * KS + side * KH * 16 + half * 8;
+  f32x4* const give = exchange + (size_t)wave * 4 * WAVE + lane;
+  const f32x4* const take = exchange + (size_t)(wave ^ 1) * 4 * WAVE + lane;
 
   fetch(tile_first);
   stash(0);
@@ -265,21 +288,28 @@ __global__ void __launch_bounds__(256)
   block_sync_lds();
   for (int tile = tile_first; tile <= tile_last; ++tile) {
     const int cur = (tile - tile_first) & 1;
-    if (tile < tile_last) stash(cur ^ 1);
-    fetch(tile + 2 <= tile_last ? tile + 2 : tile_last);  // past the end the last tile again: cheaper than a branch around loads
     const int key0 = tile * TALK_KEYS;
-    if (has_work && key0 <= wave_hi && key0 + TALK_KEYS - 1 >= wave_lo) {  // uniform over the wave
-      const bf16* kbase = lds + cur * TILE_ELEMS + (size_t)key_row * KS + half * 8;
-      const bf16* vbase = lds + cur * TILE_ELEMS + K_ELEMS;
-      f32x16 sc, sd;  // two sums, so that neighbouring products do not wait for one another
+    const bool active = has_work && key0 <= wave_hi && key0 + TALK_KEYS - 1 >= wave_lo;  // uniform over the unit
+    f32x16 sc;
+    if (active) {
 #pragma unroll
-      for (int v = 0; v < 16; ++v) sc[v] = 0.f, sd[v] = 0.f;
+      for (int v = 0; v < 16; ++v) sc[v] = 0.f;
 #pragma unroll
-      for (int c = 0; c < KC; c += 2) {
-        sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(kbase + c * 16), qreg[c], sc, 0, 0, 0);
-        sd = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(kbase + c * 16 + 16), qreg[c + 1], sd, 0, 0, 0);
+      for (int c = 0; c < KH; ++c) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(kbase + c * 16), qreg[c], sc, 0, 0, 0);
+#pragma unroll
+      for (int q = 0; q < 4; ++q) give[q * WAVE] = f32x4{sc[4 * q], sc[4 * q + 1], sc[4 * q + 2], sc[4 * q + 3]};
+    }
+    block_sync_lds();  // the scores' halves are there; nobody reads this tile's keys any more
+    if (tile < tile_last) stash(cur ^ 1);
+    // (past the end the last tile again: cheaper than a branch around loads)
+    if (!LATE) fetch(tile + 2 <= tile_last ? tile + 2 : tile_last);
+    if (active) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const f32x4 o = take[q * WAVE];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sc[4 * q + e] += o[e];  // the same two numbers in both waves, and so the same sum
       }
-      sc += sd;
       if (!(key0 + TALK_KEYS - 1 <= full_hi && key0 >= full_lo)) {
 #pragma unroll
         for (int v = 0; v < 16; ++v) {
@@ -311,17 +341,19 @@ __global__ void __launch_bounds__(256)
                          (bf16)p[8 * e + 4], (bf16)p[8 * e + 5], (bf16)p[8 * e + 6], (bf16)p[8 * e + 7]};
       if (__any(alpha != 1.f)) {  // the running maximum seldom moves after the first keys
 #pragma unroll
-        for (int dt = 0; dt < DT; ++dt) acc[dt] *= alpha;
+        for (int dt = 0; dt < DH; ++dt) acc[dt] *= alpha;
       }
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt) {
+      for (int dt = 0; dt < DH; ++dt) {
+        if (side * DH + dt < DT) {  // uniform over the wave
+          const bf16* vbase = vs + cur * L::V_ELEMS + (size_t)((side * DH + dt) * 32 + j) * VS + 8 * half;
 #pragma unroll
-        for (int e = 0; e < 2; ++e)
-          acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(vbase + (size_t)(dt * 32 + j) * VS + 16 * e + 8 * half), pmat[e],
-                                                            acc[dt], 0, 0, 0);
+          for (int e = 0; e < 2; ++e) acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(vbase + 16 * e), pmat[e], acc[dt], 0, 0, 0);
+        }
       }
     }
-    block_sync_lds();  // the tile just multiplied is overwritten after the next one
+    if (LATE) fetch(tile + 2 <= tile_last ? tile + 2 : tile_last);
+    block_sync_lds();  // the next tile's keys are there; this tile's values and the scores' halves are read
   }
   if (!valid) return;
   l += __shfl_xor(l, 32, WAVE);
@@ -329,10 +361,10 @@ __global__ void __launch_bounds__(256)
   const float inv = l > 0.f ? 1.f / l : 0.f;
   bf16* orow = a.out + (size_t)t * a.out_stride + (size_t)h * a.vdim;
 #pragma unroll
-  for (int dt = 0; dt < DT; ++dt) {
+  for (int dt = 0; dt < DH; ++dt) {
 #pragma unroll
     for (int v = 0; v < 16; v += 4) {
-      const int d = dt * 32 + 2 * v + 4 * half;
+      const int d = (side * DH + dt) * 32 + 2 * v + 4 * half;
       if (d < a.vdim)
         *reinterpret_cast<bf16x4*>(orow + d) =
             bf16x4{(bf16)(acc[dt][v] * inv), (bf16)(acc[dt][v + 1] * inv), (bf16)(acc[dt][v + 2] * inv), (bf16)(acc[dt][v + 3] * inv)};
@@ -565,19 +597,13 @@ extern "C" int fmsamd_talking_attn_mfma_fits(int kvheads, int head_dim, int valu
   return head_dim % 8 == 0 && value_dim % 8 == 0 && value_dim <= 128 && talking_padded_row(kvheads, head_dim) > 0;
 }
 
-// The prompt kernel keeps a wave's 32 mixed queries in registers beside its accumulators: rows above 512 entries leave no
-// room for values above 64.  (The decode kernel, a block per token, takes prompts of such sizes.)
-extern "C" int fmsamd_talking_attn_prefill_fits(int kvheads, int head_dim, int value_dim) {
-  return fmsamd_talking_attn_mfma_fits(kvheads, head_dim, value_dim) && (talking_padded_row(kvheads, head_dim) <= 512 || value_dim <= 64);
-}
-
 // heads of a kv head that share a prompt block: the largest of 4, 2, 1 that divides them
 static int talking_heads_of_block(int nheads, int kvheads) {
   const int per = nheads / kvheads;
   return per % 4 == 0 ? 4 : (per % 2 == 0 ? 2 : 1);
 }
 
-extern "C" int fmsamd_talking_attn_qblock(int nheads, int kvheads) { return 32 * 4 / talking_heads_of_block(nheads, kvheads); }
+extern "C" int fmsamd_talking_attn_qblock(int nheads, int kvheads) { return 32 * TALK_UNITS / talking_heads_of_block(nheads, kvheads); }
 
 static int talking_mfma_common(const char* name, const TalkArgs& a) {
   if (talking_common(name, a.n_tokens, a.nheads, a.kvheads, a.dim, a.vdim, a.q_stride, a.out_stride, a.talk)) return -1;
@@ -617,22 +643,19 @@ extern "C" int fmsamd_talking_attn_prefill(const void* q, long q_stride, void* o
   TalkArgs a{(const bf16*)q, q_stride, (bf16*)out, out_stride, positions, seq_of_token, block_table, table_stride, (const bf16*)k_cache,
              (const bf16*)v_cache, talk, sink, n_tokens, nheads, kvheads, head_dim, value_dim, scale, window};
   if (talking_mfma_common("talking_attn_prefill", a)) return -1;
-  FMS_REQUIRE(fmsamd_talking_attn_prefill_fits(kvheads, head_dim, value_dim), "talking_attn_prefill: %d kv heads of %d with values of %d do not fit",
-              kvheads, head_dim, value_dim);
   FMS_REQUIRE(qblock_tokens == fmsamd_talking_attn_qblock(nheads, kvheads), "talking_attn_prefill: query blocks of %d tokens, the kernel takes %d",
               qblock_tokens, fmsamd_talking_attn_qblock(nheads, kvheads));
   const int hb = talking_heads_of_block(nheads, kvheads);
   const long blocks = (long)n_qblocks * kvheads * (nheads / kvheads / hb);
   FMS_REQUIRE(blocks < (1L << 31), "talking_attn_prefill: too many blocks");
   const int kw = talking_padded_row(kvheads, head_dim), dt = ceil_div(value_dim, 32);
-#define FMS_TP(KC, DT)                                                                                                        \
-  do {                                                                                                                        \
-    constexpr int DTF = KC <= 32 || DT <= 2 ? DT : 2; /* the host has checked: no larger values with the longest rows */       \
-    constexpr int bytes = 2 * (TALK_KEYS * (KC * 16 + TALK_PAD) + DTF * 32 * (TALK_KEYS + TALK_PAD)) * 2;                       \
-    static const hipError_t sized = hipFuncSetAttribute(reinterpret_cast<const void*>(talking_prefill_kernel<KC, DTF>),         \
-                                                        hipFuncAttributeMaxDynamicSharedMemorySize, bytes);                    \
-    FMS_REQUIRE(sized == hipSuccess, "talking_attn_prefill: %d bytes of LDS refused: %s", bytes, hipGetErrorString(sized));    \
-    talking_prefill_kernel<KC, DTF><<<(unsigned)blocks, 256, bytes, stream>>>(a, qblock_start, qblock_len, n_qblocks, hb);      \
+#define FMS_TP(KC, DT)                                                                                                                \
+  do {                                                                                                                                \
+    constexpr int bytes = TalkPrefillLds<KC, DT>::BYTES;                                                                              \
+    static const hipError_t sized = hipFuncSetAttribute(reinterpret_cast<const void*>(talking_prefill_kernel<KC, DT>),                \
+                                                        hipFuncAttributeMaxDynamicSharedMemorySize, bytes);                           \
+    FMS_REQUIRE(sized == hipSuccess, "talking_attn_prefill: %d bytes of LDS refused: %s", bytes, hipGetErrorString(sized));           \
+    talking_prefill_kernel<KC, DT><<<(unsigned)blocks, TALK_PREFILL_THREADS, bytes, stream>>>(a, qblock_start, qblock_len, n_qblocks, hb); \
   } while (0)
   FMS_TALK_SIZES(kw, dt, FMS_TP);
 #undef FMS_TP

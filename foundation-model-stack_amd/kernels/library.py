@@ -42,7 +42,7 @@ _SIGNATURES = {
     "fmsamd_gemm_bf16": [P, L, P, P, I, P, I, L, I, I, I, P],
     "fmsamd_gemm_bf16_any": [P, L, P, P, I, P, I, L, I, I, I, P],
     "fmsamd_gemm_skinny_workspace": [I, I, I],
-    "fmsamd_gemm_skinny_bf16": [P, L, P, P, I, P, I, L, I, I, I, P, P, L, P],
+    "fmsamd_gemm_skinny_bf16": [P, L, P, P, I, P, I, L, I, I, I, I, P, P, L, P],
     "fmsamd_gemm_skinny_gated_bf16": [P, L, P, P, I, P, I, L, I, I, I, I, P, P, L, P],
     "fmsamd_gemm_skinny_residual_partials": [I, I, I],
     "fmsamd_gemm_skinny_residual_bf16": [P, L, P, P, I, P, L, P, I, P, L, P, I, I, I, I, P, P, L, P],
@@ -64,7 +64,7 @@ _SIGNATURES = {
     "fmsamd_moe_route_grouped": [P, L, I, I, I, P, I, I, F, P, P, P],
     "fmsamd_poly_norm": [P, L, I, F, F, F, F, F, P, I, L, I, P],
     "fmsamd_group_norm_chain": [P, P, I, P, I, I, F, P, I, I, F, P, I, P, I, I, P],
-    "fmsamd_short_conv": [P, L, I, P, P, I, I, P, P, P, I, P, I, L, I, I, I, P],
+    "fmsamd_short_conv": [P, L, I, P, P, I, I, P, P, P, I, P, I, L, I, I, I, P, I, P],
     "fmsamd_rglru_gates": [P, L, P, P, P, P, I, P, F, P, P, P, I, I, I, P],
     "fmsamd_rglru_scan": [P, P, P, L, I, P, P, P, P, P, I, L, I, I, P],
     "fmsamd_rglru_scan_chunk": [I, I],
@@ -74,19 +74,19 @@ _SIGNATURES = {
     "fmsamd_value_head_norm": [P, L, I, I, I, F, P, I, L, P, I, P],
     "fmsamd_scale_f32": [P, L, F, P],
     "fmsamd_cast_cols": [P, L, P, I, L, I, I, P],
-    "fmsamd_delta_prepare": [P, L, I, P, L, I, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P],
+    "fmsamd_delta_prepare": [P, L, I, P, L, I, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, P, I, P],
     "fmsamd_delta_rule": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
     "fmsamd_gated_head_norm": [P, P, L, P, I, F, I, F, P, I, L, P, I, I, I, P],
     "fmsamd_moe_combine": [P, P, I, P, P, L, P, I, I, I, P, I, P, L, P],
     "fmsamd_talking_attn_generic": [P, L, P, L, I, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
     "fmsamd_talking_attn_mfma_fits": [I, I, I],
-    "fmsamd_talking_attn_prefill_fits": [I, I, I],
     "fmsamd_talking_attn_qblock": [I, I],
     "fmsamd_talking_attn_prefill": [P, L, P, L, P, P, P, P, I, I, P, I, P, P, P, P, I, I, I, I, I, F, I, P],
     "fmsamd_talking_attn_decode": [P, L, P, L, P, L, P, P, P, I, P, P, P, P, I, I, I, I, I, F, I, I, P],
     "fmsamd_ssd_scan": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
     "fmsamd_ssd_chunked": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, L, P],
-    "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P],
+    "fmsamd_ssd_step": [P, L, I, I, P, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P, L, I, I, P, P, P],
     "fmsamd_probe_read": [P, L, I, I, P, P],
     "fmsamd_probe_mfma": [I, I, I, P, P, P],
 }

@@ -514,6 +514,7 @@ def prefill_qblock(nheads: int, kvheads: int, head_dim: int, n_tokens: int) -> i
 # matrix products
 # --------------------------------------------------------------------------
 SKINNY_MAX_ROWS = 192
+_PLAIN_ACTIVATIONS = ("identity", "relu", "relu2")  # what the skinny kernels finish a plain product with
 # Up to this many rows the skinny kernel, with the norms, rotation and activation fused into it, beats the
 # vendor library followed by those as kernels of their own.
 SKINNY_FAST_ROWS = 192
@@ -526,8 +527,10 @@ def linear(
     out_dtype: Optional[torch.dtype] = None,
     allow_library: bool = True,
     row_norm: Optional[RowNorm] = None,
+    activation: str = "identity",
 ) -> torch.Tensor:
-    """x [M, K] @ weight[N, K]^T (+ bias) -> [M, N].
+    """act(x [M, K] @ weight[N, K]^T (+ bias)) -> [M, N].  The skinny kernels finish with relu and its square themselves; every
+    other activation and kernel is followed by the activation kernel.
 
     float32 x float32: the FMA kernel (true 32-bit).  bfloat16 x bfloat16: the weight-streaming
     skinny kernels up to 192 rows; above that the vendor library (hipBLASLt through torch.matmul,
@@ -548,6 +551,9 @@ def linear(
         raise ValueError(f"bias must be a contiguous [{N}] tensor")
     out_dtype = out_dtype or x.dtype
     lib = load()
+    if activation != "identity" and not (activation in _PLAIN_ACTIVATIONS and x.dtype == weight.dtype == torch.bfloat16
+                                         and M <= SKINNY_FAST_ROWS and K % 8 == 0 and x.stride(0) % 8 == 0):
+        return activate(linear(x, weight, bias, out_dtype, allow_library, row_norm), activation)
     if row_norm is not None and not (weight.dtype == x.dtype == torch.bfloat16 and M <= SKINNY_FAST_ROWS):
         raise ValueError(f"a deferred row norm goes with the bfloat16 product of at most {SKINNY_FAST_ROWS} rows")
     if weight.dtype == torch.float32:
@@ -578,12 +584,14 @@ def linear(
         out = torch.empty(M, N, dtype=out_dtype, device=x.device)
         ws, ws_bytes = _skinny_workspace(M, N, K, x.device)
         check(lib.fmsamd_gemm_skinny_bf16(x.data_ptr(), x.stride(0), weight.data_ptr(), _ptr(bias), bcode, out.data_ptr(),
-                                          _code(out_dtype), out.stride(0), M, N, K, _row_scale(row_norm, M), _ptr(ws),
+                                          _code(out_dtype), out.stride(0), M, N, K, ACTIVATIONS[activation], _row_scale(row_norm, M), _ptr(ws),
                                           ws_bytes, _stream()))
         return out
     if allow_library and out_dtype in (torch.bfloat16, torch.float32):
         # vendor library GEMM, float32 accumulation; float32 results (the logits of many rows) come straight from the
         # accumulators, without a rounding to bfloat16 in between
+        if out_dtype == torch.bfloat16 and bias is not None and bias.dtype == torch.bfloat16:
+            return torch.addmm(bias, x, weight.t())  # the bias joins the float32 sums: one rounding, no pass of its own
         if out_dtype == torch.bfloat16:
             out = torch.matmul(x, weight.t())
         else:
@@ -828,13 +836,20 @@ CONV_MAX_TAPS = 8
 
 def short_conv(x: torch.Tensor, col0: int, channels: int, conv_w: torch.Tensor, bias: Optional[torch.Tensor], conv_state: Optional[torch.Tensor],
                seq_of_token: torch.Tensor, slot_ids: torch.Tensor, out_dtype: torch.dtype, add_input: bool = False,
-               single_tokens: bool = False, activation: str = "identity") -> torch.Tensor:
+               single_tokens: bool = False, activation: str = "identity", seq_starts: Optional[torch.Tensor] = None,
+               n_seqs: int = 0) -> torch.Tensor:
     """A causal convolution over time on the channels col0 .. col0 + channels of float32 rows: out[t, c] = act((x[t, c] if
     add_input) + bias[c] + sum_j conv_w[c, j] x[t - taps + 1 + j, c]) over the sequence's own tokens -> [T, channels] in
     out_dtype.  The inputs before the step come from conv_state [slots, taps - 1, channels] (float32; zeros before a
     sequence's start), which is then moved on to the step's last inputs.  single_tokens: every sequence of the step
-    brings exactly one token (a decode step); the kernel that convolves then moves the state on as well."""
-    _need_cuda(x, conv_w, bias, conv_state, seq_of_token, slot_ids)
+    brings exactly one token (a decode step); the kernel that convolves then moves the state on as well.  activation:
+    "identity" or "silu".  seq_starts [n_seqs + 1]: where the sequences' rows start (the state is then moved on by their last
+    tokens' blocks only)."""
+    _need_cuda(x, conv_w, bias, conv_state, seq_of_token, slot_ids, seq_starts)
+    if seq_starts is not None:
+        _need_i32("seq_starts", seq_starts)
+        if n_seqs < 1 or seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs:
+            raise ValueError("short_conv: the step's index arrays are shorter than its sequences")
     _rows2d("x", x)
     _need_i32("seq_of_token", seq_of_token)
     _need_i32("slot_ids", slot_ids)
@@ -853,7 +868,8 @@ def short_conv(x: torch.Tensor, col0: int, channels: int, conv_w: torch.Tensor, 
     view = x[:, col0 : col0 + channels]
     check(load().fmsamd_short_conv(view.data_ptr(), x.stride(0), channels, conv_w.data_ptr(), _ptr(bias), _code(conv_w.dtype), taps,
                                    _ptr(conv_state), seq_of_token.data_ptr(), slot_ids.data_ptr(), int(bool(add_input)), out.data_ptr(),
-                                   _code(out_dtype), out.stride(0), T, int(bool(single_tokens)), ACTIVATIONS[activation], _stream()))
+                                   _code(out_dtype), out.stride(0), T, int(bool(single_tokens)), ACTIVATIONS[activation],
+                                   _ptr(seq_starts), int(n_seqs), _stream()))
     return out
 
 
@@ -918,7 +934,7 @@ def rglru_scan(a: torch.Tensor, b: torch.Tensor, y: torch.Tensor, activation: st
     return out
 
 
-def activation(x: torch.Tensor, kind: str) -> torch.Tensor:
+def activate(x: torch.Tensor, kind: str) -> torch.Tensor:
     """act(x), elementwise, for the activations of ACTIVATIONS."""
     _need_cuda(x)
     if not x.is_contiguous():
@@ -926,6 +942,9 @@ def activation(x: torch.Tensor, kind: str) -> torch.Tensor:
     out = torch.empty_like(x)
     check(load().fmsamd_activate(x.data_ptr(), out.data_ptr(), _code(x.dtype), x.numel(), ACTIVATIONS[kind], _stream()))
     return out
+
+
+activation = activate
 
 
 def clamped_gated_act(gu: torch.Tensor, limit: float, alpha: float, shift: float) -> torch.Tensor:
@@ -1334,7 +1353,7 @@ def talking_qblock(nheads: int, kvheads: int, head_dim: int, value_dim: int) -> 
     """The number of consecutive query tokens of one sequence that a block of the bfloat16 prompt kernel takes; 0: sizes that
     it does not take."""
     lib = load()
-    return lib.fmsamd_talking_attn_qblock(nheads, kvheads) if lib.fmsamd_talking_attn_prefill_fits(kvheads, head_dim, value_dim) else 0
+    return lib.fmsamd_talking_attn_qblock(nheads, kvheads) if lib.fmsamd_talking_attn_mfma_fits(kvheads, head_dim, value_dim) else 0
 
 
 def gate_mul(x: torch.Tensor, gate: Optional[torch.Tensor], activation: str = "sigmoid", scale: float = 1.0,
@@ -1392,13 +1411,19 @@ DELTA_MAX_DIM = 256
 
 def delta_prepare(proj: torch.Tensor, col_b: int, a: torch.Tensor, col_a: int, conv_w: torch.Tensor, a_log: torch.Tensor,
                   dt_bias: torch.Tensor, conv_state: torch.Tensor, seq_of_token: torch.Tensor, slot_ids: torch.Tensor, heads: int,
-                  kv_heads: int, dim: int, vdim: int, per_channel: bool, q_scale: float):
+                  kv_heads: int, dim: int, vdim: int, per_channel: bool, q_scale: float, seq_starts: Optional[torch.Tensor] = None,
+                  n_seqs: int = 0):
     """What the recurrence of a step reads, from the float32 projections of its tokens: (qkv [T, C], beta [T, heads],
     decay [T, heads] or [T, heads*dim], kq [T, kv_heads] = k . q), all float32.  The first C = 2*kv_heads*dim + heads*vdim columns of `proj` pass the
     short causal convolution (conv_w [C, taps]; the inputs before the step come from conv_state [slots, taps-1, C], which
     is then moved on), silu, and q and k become unit vectors per head (q times q_scale); beta = sigmoid(proj[:, col_b:]);
-    decay = exp(-exp(a_log) * softplus(a[:, col_a:] + dt_bias))."""
-    _need_cuda(proj, a, conv_w, a_log, dt_bias, conv_state, seq_of_token, slot_ids)
+    decay = exp(-exp(a_log) * softplus(a[:, col_a:] + dt_bias)).  seq_starts [n_seqs + 1]: where the sequences' rows start
+    (the convolution's state is then moved on by their last tokens' blocks only)."""
+    _need_cuda(proj, a, conv_w, a_log, dt_bias, conv_state, seq_of_token, slot_ids, seq_starts)
+    if seq_starts is not None:
+        _need_i32("seq_starts", seq_starts)
+        if n_seqs < 1 or seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs:
+            raise ValueError("delta_prepare: the step's index arrays are shorter than its sequences")
     _rows2d("proj", proj)
     _rows2d("a", a)
     _need_i32("seq_of_token", seq_of_token)
@@ -1428,7 +1453,8 @@ def delta_prepare(proj: torch.Tensor, col_b: int, a: torch.Tensor, col_a: int, c
     check(load().fmsamd_delta_prepare(proj.data_ptr(), proj.stride(0), col_b, a.data_ptr(), a.stride(0), col_a, conv_w.data_ptr(),
                                       _code(conv_w.dtype), taps, a_log.data_ptr(), dt_bias.data_ptr(), conv_state.data_ptr(),
                                       seq_of_token.data_ptr(), slot_ids.data_ptr(), qkv.data_ptr(), beta.data_ptr(), decay.data_ptr(),
-                                      kq.data_ptr(), T, heads, kv_heads, dim, vdim, int(bool(per_channel)), float(q_scale), _stream()))
+                                      kq.data_ptr(), T, heads, kv_heads, dim, vdim, int(bool(per_channel)), float(q_scale),
+                                      _ptr(seq_starts), int(n_seqs), _stream()))
     return qkv, beta, decay, kq
 
 
@@ -1536,11 +1562,64 @@ def ssd(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, dt_bias: torch
     return y
 
 
+def ssd_step(proj: torch.Tensor, col_x: int, col_dt: int, conv_w: torch.Tensor, conv_b: torch.Tensor, conv_state: Optional[torch.Tensor],
+             a_log: torch.Tensor, dt_bias: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, seq_starts: torch.Tensor,
+             seq_of_token: torch.Tensor, slot_ids: torch.Tensor, n_seqs: int, heads: int, vdim: int, groups: int, n_state: int) -> torch.Tensor:
+    """`short_conv` with silu followed by `ssd`, for a step in which every sequence brings one token: proj holds the channels
+    before the convolution at col_x and the step sizes at col_dt.  The convolution's state [slots, taps - 1, channels] is
+    read and left as it is: whoever runs next moves it on (gated_group_norm)."""
+    _need_cuda(proj, conv_w, conv_b, conv_state, a_log, dt_bias, skip, state, seq_starts, seq_of_token, slot_ids)
+    _rows2d("proj", proj)
+    for name, t in (("seq_starts", seq_starts), ("seq_of_token", seq_of_token), ("slot_ids", slot_ids)):
+        _need_i32(name, t)
+    T = proj.shape[0]
+    C = heads * vdim + 2 * groups * n_state
+    if proj.dtype != torch.float32 or min(col_x, col_dt) < 0 or proj.shape[1] < max(col_x + C, col_dt + heads):
+        raise ValueError("ssd_step takes float32 rows that hold the columns asked for")
+    if conv_w.dim() != 2 or conv_w.shape[0] != C or not conv_w.is_contiguous() or not 1 <= conv_w.shape[1] <= CONV_MAX_TAPS:
+        raise ValueError(f"the convolution's weights are contiguous [{C}, taps], taps at most {CONV_MAX_TAPS}")
+    taps = conv_w.shape[1]
+    if tuple(conv_b.shape) != (C,) or not conv_b.is_contiguous() or conv_b.dtype != conv_w.dtype:
+        raise ValueError(f"the convolution's bias is a contiguous [{C}] tensor of the weights' type")
+    if taps > 1:
+        _check_conv_state(conv_state, taps, C)
+    for name, t in (("a_log", a_log), ("dt_bias", dt_bias), ("skip", skip)):
+        if t.dtype != torch.float32 or tuple(t.shape) != (heads,) or not t.is_contiguous():
+            raise ValueError(f"{name} is a contiguous float32 [{heads}] tensor")
+    if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, vdim, n_state) or not state.is_contiguous():
+        raise ValueError(f"the state is contiguous float32 [slots, {heads}, {vdim}, {n_state}]")
+    if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs or seq_of_token.numel() < T:
+        raise ValueError("the step's index arrays are shorter than its sequences or tokens")
+    y = torch.empty(T, heads * vdim, dtype=torch.float32, device=proj.device)
+    check(load().fmsamd_ssd_step(proj.data_ptr(), proj.stride(0), col_x, col_dt, conv_w.data_ptr(), conv_b.data_ptr(), _code(conv_w.dtype), taps,
+                                 _ptr(conv_state) if taps > 1 else None, a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(), state.data_ptr(),
+                                 y.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(), int(n_seqs), heads, vdim,
+                                 groups, n_state, _stream()))
+    return y
+
+
+def _check_conv_state(conv_state: Optional[torch.Tensor], taps: int, channels: int) -> None:
+    if (conv_state is None or conv_state.dtype != torch.float32 or conv_state.dim() != 3
+            or tuple(conv_state.shape[1:]) != (taps - 1, channels) or not conv_state.is_contiguous()):
+        raise ValueError(f"the convolution's state is contiguous float32 [slots, {taps - 1}, {channels}]")
+
+
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, parts: int, eps: float, out_dtype: torch.dtype,
-                     seq_of_token: torch.Tensor) -> torch.Tensor:
+                     seq_of_token: torch.Tensor, conv_x: Optional[torch.Tensor] = None, taps: int = 0,
+                     conv_state: Optional[torch.Tensor] = None, slot_ids: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y * silu(z), each of `parts` equal consecutive parts of a row divided by its own root mean square, times weight:
-    y float32 [T, cols] contiguous, z float32 rows [T, cols] of any stride -> [T, cols] in out_dtype."""
-    _need_cuda(y, z, weight, seq_of_token)
+    y float32 [T, cols] contiguous, z float32 rows [T, cols] of any stride -> [T, cols] in out_dtype.
+    conv_x (float32 rows [T, channels], with taps, conv_state and slot_ids): the same launch moves the state of a convolution
+    over those rows on, in a step in which every sequence brings one token."""
+    _need_cuda(y, z, weight, seq_of_token, conv_x, conv_state, slot_ids)
+    channels = 0
+    if conv_x is not None:
+        _rows2d("conv_x", conv_x)
+        _need_i32("slot_ids", slot_ids)
+        channels = conv_x.shape[1]
+        if conv_x.dtype != torch.float32 or conv_x.shape[0] != y.shape[0] or not 2 <= taps <= CONV_MAX_TAPS:
+            raise ValueError(f"a state is moved on by float32 rows, one a token, and has 1 to {CONV_MAX_TAPS - 1} inputs")
+        _check_conv_state(conv_state, taps, channels)
     _rows2d("z", z)
     _need_i32("seq_of_token", seq_of_token)
     T, cols = y.shape
@@ -1550,7 +1629,9 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, par
         raise ValueError(f"gated_group_norm: a contiguous weight [{cols}], {parts} equal parts, a sequence index per token")
     out = torch.empty(T, cols, dtype=out_dtype, device=y.device)
     check(load().fmsamd_gated_group_norm(y.data_ptr(), z.data_ptr(), z.stride(0), weight.data_ptr(), _code(weight.dtype), int(parts), float(eps),
-                                         out.data_ptr(), _code(out_dtype), seq_of_token.data_ptr(), T, cols, _stream()))
+                                         out.data_ptr(), _code(out_dtype), seq_of_token.data_ptr(), T, cols, _ptr(conv_x),
+                                         conv_x.stride(0) if conv_x is not None else 0, channels, int(taps), _ptr(conv_state), _ptr(slot_ids),
+                                         _stream()))
     return out
 
 

@@ -52,7 +52,7 @@ class MLP(FeedForward):
             # the three norms are formed from the float32 sums of the product
             hidden = ops.poly_norm(self.up.forward(x, out_dtype=torch.float32), self._coefficients, self.eps, x.dtype)
             return BranchOutput(hidden, self.down)
-        return BranchOutput(ops.activation(self.up.forward(x), self.activation), self.down)
+        return BranchOutput(self.up.forward(x, activation=self.activation), self.down)
 
 
 class ExpertsFeedForward(FeedForward):

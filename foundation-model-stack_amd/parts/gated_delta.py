@@ -113,7 +113,8 @@ class GatedDeltaRule(Mixer):
         else:
             gate = proj[:, self.col_g : self.col_g + H * V]
         qkv, beta, decay, kq = ops.delta_prepare(proj, self.col_b, a, col_a, self.w["conv.weight"], self._a_log, self._dt_bias,
-                                             state["conv"], batch.seq_of_token, batch.slot_ids, H, G, D, V, self.per_channel, D ** -0.5)
+                                             state["conv"], batch.seq_of_token, batch.slot_ids, H, G, D, V, self.per_channel, D ** -0.5,
+                                             seq_starts=batch.seq_starts, n_seqs=batch.n_seqs)
         o = ops.delta_rule(qkv, beta, decay, kq, state["S"], batch.seq_starts, batch.seq_of_token, batch.slot_ids, batch.n_seqs, H, G, D, V,
                            self.per_channel, single_tokens=batch.is_decode)
         normed = ops.gated_head_norm(o, gate, self.w["norm.weight"], self.eps, self.gate_activation, H, V, x.dtype, batch.seq_of_token,

@@ -20,9 +20,10 @@ class Linear(Part):
             self.declare("bias", (out_features,), init="zeros")
 
     def forward(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None, row_norm=None,
-                bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                bias: Optional[torch.Tensor] = None, activation: str = "identity") -> torch.Tensor:
         """bias: a vector to add in the place of the layer's own (a layer without one takes one that changes from call to call)."""
-        return ops.linear(x, self.w["weight"], self.w.get("bias") if bias is None else bias, out_dtype=out_dtype, row_norm=row_norm)
+        return ops.linear(x, self.w["weight"], self.w.get("bias") if bias is None else bias, out_dtype=out_dtype, row_norm=row_norm,
+                          activation=activation)
 
     def streams(self, rows: int, dtype: torch.dtype) -> bool:
         """True if a product of this shape runs in the weight-streaming kernel, which can take a deferred

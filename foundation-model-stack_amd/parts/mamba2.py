@@ -77,11 +77,20 @@ class Mamba2(Mixer):
         state = cache.state
         # step sizes, decays, the gate and the recurrence are formed from the float32 sums of this product
         proj = self.in_proj.forward(x, out_dtype=torch.float32)
+        z = proj[:, : self.inner]
+        if batch.is_decode:
+            # the convolution and the recurrence as one kernel; the convolution's state moves on beside the norm
+            y = ops.ssd_step(proj, self.col_x, self.col_dt, self.w["conv.weight"], self.w["conv.bias"], state.get("conv"), self._a_log,
+                             self._dt_bias, self._skip, state["S"], batch.seq_starts, batch.seq_of_token, batch.slot_ids, batch.n_seqs,
+                             self.heads, self.vdim, self.groups, self.state)
+            move = dict(conv_x=proj[:, self.col_x : self.col_dt], taps=self.taps, conv_state=state["conv"], slot_ids=batch.slot_ids) if self.taps > 1 else {}
+            return BranchOutput(ops.gated_group_norm(y, z, self.w["norm.weight"], self.norm_groups, self.eps, x.dtype, batch.seq_of_token, **move),
+                                self.out)
         xbc = ops.short_conv(proj, self.col_x, self.channels, self.w["conv.weight"], self.w["conv.bias"], state.get("conv"), batch.seq_of_token,
-                             batch.slot_ids, torch.float32, single_tokens=batch.is_decode, activation="silu")
+                             batch.slot_ids, torch.float32, activation="silu", seq_starts=batch.seq_starts, n_seqs=batch.n_seqs)
         y = ops.ssd(xbc, proj[:, self.col_dt :], self._a_log, self._dt_bias, self._skip, state["S"], batch.seq_starts, batch.seq_of_token,
                     batch.slot_ids, batch.n_seqs, self.heads, self.vdim, self.groups, self.state, longest=max(batch.q_lens))
-        normed = ops.gated_group_norm(y, proj[:, : self.inner], self.w["norm.weight"], self.norm_groups, self.eps, x.dtype, batch.seq_of_token)
+        normed = ops.gated_group_norm(y, z, self.w["norm.weight"], self.norm_groups, self.eps, x.dtype, batch.seq_of_token)
         return BranchOutput(normed, self.out)
 
 
