@@ -109,6 +109,9 @@ def _to_model_names(sd, model_config=None, **kw):
             out[p + "in_proj.qkv_fused.weight"] = torch.cat(list(weights.values()), dim=0)
             out[p + "in_proj.qkv_fused.bias"] = torch.cat(list(biases.values()), dim=0)
             out[p + "dense.weight"] = out.pop(p + "o")
+        if layer.get("mlp") is None:  # a layer without a feed-forward has no use for that branch's norm and scale
+            for n in ("norm2", "ls2"):
+                out.pop(name[: -len("mix.o")] + n, None)
     renamed = {}
     for name, t in out.items():
         if re.search(r"\.mlp\.(up|down)\.b$", name):
