@@ -125,29 +125,34 @@ struct TalkArgs {
 
 __device__ __forceinline__ int talk_first_key(int pos, int window) { return (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0; }
 
-// Eight entries k .. k + 7 of the mixed query of head h of the token whose queries start at qrow: kv head k / dim, entry
-// k % dim, summed over that kv head's query heads.  dim is a multiple of 8, so the eight share a kv head.
-__device__ __forceinline__ bf16x8 talk_mixed_query(const bf16* qrow, const TalkArgs& a, int h, int k) {
-  const int per = a.nheads / a.kvheads;
-  const int c = k / a.dim, d = k - c * a.dim;
+// Eight entries of the mixed query of a head: kv head c, entries d .. d + 7 of its query heads summed with the head's row of the
+// mixing matrix.  The heads' pieces are asked for four at a time.
+__device__ __forceinline__ bf16x8 talk_mixed_query(const bf16* qrow, const float* mix, int c, int d, int per, int dim) {
   float s[8];
 #pragma unroll
   for (int e = 0; e < 8; ++e) s[e] = 0.f;
-  for (int i = 0; i < per; ++i) {
-    const int g = c * per + i;
-    const float w = a.talk[(size_t)h * a.nheads + g];
-    const bf16x8 v = talk_load8(qrow + (size_t)g * a.dim + d);
+  const bf16* src = qrow + (size_t)c * per * dim + d;
+  for (int i0 = 0; i0 < per; i0 += 4) {
+    bf16x8 v[4];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) s[e] = fmaf(w, (float)v[e], s[e]);
+    for (int i = 0; i < 4; ++i) v[i] = talk_load8(src + (size_t)(i0 + i < per ? i0 + i : 0) * dim);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float w = i0 + i < per ? mix[c * per + i0 + i] : 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s[e] = fmaf(w, (float)v[i][e], s[e]);
+    }
   }
   return bf16x8{(bf16)s[0], (bf16)s[1], (bf16)s[2], (bf16)s[3], (bf16)s[4], (bf16)s[5], (bf16)s[6], (bf16)s[7]};
 }
 
 // Prompts.  A block has four units: `hb` heads of one kv head times 4 / hb runs of 32 consecutive query tokens of one
 // sequence.  A unit is one head and 32 queries (one tile column of the 32x32x16 product) and has two waves, which split the
-// entries of the mixed queries (a wave multiplies its half of every key row, and the halves of the scores meet in LDS) and
-// the value channels: a query's mixed row is as long as all kv heads' keys together, and half of it leaves a wave room to be
-// one of two on its SIMD.  Tiles of 32 keys (all kv heads' keys, and the values of the block's kv head) go through LDS: the
+// entries of the mixed queries (a query's mixed row is as long as all kv heads' keys together, and half of it leaves a wave
+// room to be one of two on its SIMD) and the keys behind them: a wave multiplies its half of every key row, hands its sums for
+// the other's 16 keys of the tile over through LDS, and runs softmax and second product over its own 16; at the end the
+// two waves' results are joined.  (Where the rows are longest, a wave's registers do not hold the accumulators of all value
+// channels: there both waves take all 32 keys, and the value channels are split.)  Tiles of 32 keys (all kv heads' keys, and the values of the block's kv head) go through LDS: the
 // keys are free as soon as the scores are formed, so the next tile's are written while this one's softmax and second product
 // run, and the tile after that is on its way from memory.
 //
@@ -162,7 +167,9 @@ struct TalkPrefillLds {
   static constexpr int KS = KC * 16 + TALK_PAD;     // row stride of the keys [32][KS]
   static constexpr int VS = TALK_KEYS + TALK_PAD;   // row stride of the transposed values [DT * 32][VS]
   static constexpr int K_ELEMS = TALK_KEYS * KS, V_ELEMS = DT * 32 * VS;
-  static constexpr int EXCHANGE = TALK_UNITS * 2 * WAVE * 16;  // float32: a score tile's half of every wave
+  static constexpr bool SPLIT_VALUES = KC > 32 && DT > 2;
+  static constexpr int OWN = SPLIT_VALUES ? 16 : 8;  // scores of a tile that a lane runs the softmax over
+  static constexpr int EXCHANGE = TALK_UNITS * 2 * WAVE * OWN;  // float32: what every wave hands over
   static constexpr int BYTES = (K_ELEMS + 2 * V_ELEMS) * 2 + EXCHANGE * 4;
 };
 
@@ -170,20 +177,28 @@ template <int KC, int DT>
 __global__ void __launch_bounds__(TALK_PREFILL_THREADS) __attribute__((amdgpu_waves_per_eu(2, 2)))
     talking_prefill_kernel(TalkArgs a, const int* __restrict__ qblock_start, const int* __restrict__ qblock_len, int n_qblocks, int hb) {
   typedef TalkPrefillLds<KC, DT> L;
-  constexpr int KH = KC / 2, DH = (DT + 1) / 2;  // a wave's share of the key entries (steps of 16) and value tiles
-  constexpr bool LATE = KC > 32;  // the longest rows leave the softmax no room for a tile on its way: it is asked for behind it
+  constexpr int KH = KC / 2;  // a wave's share of the key entries, in steps of 16
+  constexpr bool SPLIT_VALUES = L::SPLIT_VALUES;
+  constexpr int OWN = L::OWN, DA = SPLIT_VALUES ? (DT + 1) / 2 : DT;  // DA: tiles of 32 value channels of a wave
+  // The longest rows leave registers for half a tile of keys on its way: one half is under way while the scores are formed,
+  // the other while softmax and second product run.
+  constexpr bool HALVES = KC > 32;
   constexpr int KW = KC * 16, KS = L::KS, VS = L::VS;
   constexpr int KCH = TALK_KEYS * KW / 8 / TALK_PREFILL_THREADS;                                          // 16-byte pieces a thread
   constexpr int VCH = (DT * 32 * TALK_KEYS / 8 + TALK_PREFILL_THREADS - 1) / TALK_PREFILL_THREADS;  // moves per tile
   extern __shared__ __attribute__((aligned(16))) unsigned char talk_lds[];
   bf16* const ks = reinterpret_cast<bf16*>(talk_lds);
   bf16* const vs = ks + L::K_ELEMS;  // two of them, in turn
-  f32x4* const exchange = reinterpret_cast<f32x4*>(vs + 2 * L::V_ELEMS);  // [wave][4][lane]
+  f32x4* const exchange = reinterpret_cast<f32x4*>(vs + 2 * L::V_ELEMS);  // [wave][OWN / 4][lane]
 
-  // blocks with the most keys (a causal step's last) are handed out first
+  // Blocks with the most keys (a causal step's last) are handed out first.  Workgroups go to the chip's eight dies in turn,
+  // each with a cache of its own: runs of four query blocks, whose windows overlap, with all their heads go to one die.
   const int per = a.nheads / a.kvheads, tiles = per / hb, per_qb = a.kvheads * tiles;
-  const int qb = n_qblocks - 1 - (int)(blockIdx.x / per_qb);
-  const int y = blockIdx.x % per_qb;
+  int id = blockIdx.x;
+  const int run = 4 * per_qb, whole = n_qblocks / 32 * 8 * run;  // blocks of whole rounds over the dies
+  if (id < whole) id = ((id / 8 / run) * 8 + id % 8) * run + (id / 8) % run;
+  const int qb = n_qblocks - 1 - id / per_qb;
+  const int y = id % per_qb;
   const int kh = y / tiles;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   const int unit = wave >> 1, side = wave & 1;
@@ -204,13 +219,20 @@ __global__ void __launch_bounds__(TALK_PREFILL_THREADS) __attribute__((amdgpu_wa
   // the mixed queries of one unit after the other pass through the keys' place in LDS: all threads form them, the unit's
   // waves take their halves.  (Their padding leaves zeros behind the keys' entries, which are multiplied by zeros later.)
   bf16x8 qreg[KH];
+  float* const mix = reinterpret_cast<float*>(exchange);  // the heads' rows of the mixing matrix
+  for (int i = threadIdx.x; i < hb * a.nheads; i += TALK_PREFILL_THREADS)
+    mix[i] = a.talk[(size_t)(kh * per + (y % tiles) * hb) * a.nheads + i];
+  // a thread's pieces share their entries k: a row has a power of two of pieces, or (384) 48, and tokens are 512 / that apart
+  const int uk = (threadIdx.x % (KW / 8)) * 8, uc = uk < row ? uk / a.dim : 0, ud = uk - uc * a.dim;
+  __syncthreads();
   for (int u = 0; u < TALK_UNITS; ++u) {
-    const int uh = kh * per + (y % tiles) * hb + u % hb, ut = t_begin + (u / hb) * 32;
-    for (int i = threadIdx.x; i < 32 * (KW / 8); i += TALK_PREFILL_THREADS) {
-      const int tok = i / (KW / 8), k = (i % (KW / 8)) * 8;
+    const int ut = t_begin + (u / hb) * 32;
+    for (int tok = threadIdx.x / (KW / 8); tok < 32; tok += TALK_PREFILL_THREADS / (KW / 8)) {
+      if (KW == 384 && threadIdx.x >= TALK_PREFILL_THREADS / (KW / 8) * (KW / 8)) break;  // 480 of the threads have a piece
       bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (ut + tok < t_end && k < row) v = talk_mixed_query(a.q + (size_t)(ut + tok) * a.q_stride, a, uh, k);
-      *reinterpret_cast<bf16x8*>(ks + tok * KS + k) = v;
+      if (ut + tok < t_end && uk < row)
+        v = talk_mixed_query(a.q + (size_t)(ut + tok) * a.q_stride, mix + (u % hb) * a.nheads, uc, ud, per, a.dim);
+      *reinterpret_cast<bf16x8*>(ks + tok * KS + uk) = v;
     }
     __syncthreads();
     if (u == unit) {
@@ -245,80 +267,107 @@ __global__ void __launch_bounds__(TALK_PREFILL_THREADS) __attribute__((amdgpu_wa
     k_at[n] = there ? (unsigned)(tok * (KS / 8) + c * d8 + d) << 16 | (unsigned)((c * PAGE_TOKENS + tok) * d8 + d) : TALK_NOWHERE;
   }
   const int v_pieces = a.vdim * (TALK_KEYS / 8);
-  bf16x8 kbuf[KCH], vbuf[VCH];
-  auto fetch = [&](int tile) {
+  constexpr int KP = HALVES ? KCH / 2 : KCH;
+  bf16x8 kbuf[KP], vbuf[VCH];
+  // the pieces of a tile's keys from n0 on (and, with the first of them, its values) into registers, and on into LDS
+  auto fetch = [&](int tile, int n0) {
     const int key0 = tile * TALK_KEYS;
-    const size_t phys = readable_page(bt[key0 / PAGE_TOKENS]);
+    const size_t phys = readable_page(uniform_load(bt + key0 / PAGE_TOKENS));
     const int in_page = key0 % PAGE_TOKENS;
     const bf16* kp = a.k_cache + phys * page_elems + (size_t)in_page * a.dim;
     const bf16* vp = a.v_cache + phys * vpage_elems + (size_t)kh * a.vdim * PAGE_TOKENS + in_page;
 #pragma unroll
-    for (int n = 0; n < KCH; ++n) kbuf[n] = talk_load8(kp + (size_t)(k_at[n] & 0xffffu) * 8);
+    for (int n = 0; n < KP; ++n) kbuf[n] = talk_load8(kp + (size_t)(k_at[HALVES && n0 ? n + KCH - KP : n] & 0xffffu) * 8);
+    if (n0) return;
 #pragma unroll
     for (int n = 0; n < VCH; ++n) {
       const int id = threadIdx.x + n * TALK_PREFILL_THREADS;
       vbuf[n] = talk_load8(vp + (id < v_pieces ? (size_t)(id / (TALK_KEYS / 8)) * PAGE_TOKENS + (id % (TALK_KEYS / 8)) * 8 : 0));
     }
   };
-  auto stash = [&](int which) {  // keys into their one place, values into place `which`
+  auto stash = [&](int which, int n0) {  // keys into their one place, values into place `which`
 #pragma unroll
-    for (int n = 0; n < KCH; ++n)
-      if (k_at[n] != TALK_NOWHERE) *reinterpret_cast<bf16x8*>(ks + (k_at[n] >> 16) * 8) = kbuf[n];
+    for (int n = 0; n < KP; ++n) {
+      const unsigned at = k_at[HALVES && n0 ? n + KCH - KP : n];
+      if (at != TALK_NOWHERE) *reinterpret_cast<bf16x8*>(ks + (at >> 16) * 8) = kbuf[n];
+    }
+    if (n0) return;
 #pragma unroll
     for (int n = 0; n < VCH; ++n) {
       const int id = threadIdx.x + n * TALK_PREFILL_THREADS;
       if (id < v_pieces) *reinterpret_cast<bf16x8*>(vs + which * L::V_ELEMS + (id / (TALK_KEYS / 8)) * VS + (id % (TALK_KEYS / 8)) * 8) = vbuf[n];
     }
   };
-  f32x16 acc[DH];
+  f32x16 acc[DA];
 #pragma unroll
-  for (int dt = 0; dt < DH; ++dt)
+  for (int dt = 0; dt < DA; ++dt)
 #pragma unroll
     for (int v = 0; v < 16; ++v) acc[dt][v] = 0.f;
   float m = TALK_EMPTY, l = 0.f;
   const float scale2 = a.scale * TALK_LOG2E;
   const int key_row = 16 * (j >> 4) + 8 * ((j >> 2) & 1) + 4 * ((j >> 3) & 1) + (j & 3);
   const bf16* const kbase = ks + (size_t)key_row * KS + side * KH * 16 + half * 8;
-  f32x4* const give = exchange + (size_t)wave * 4 * WAVE + lane;
-  const f32x4* const take = exchange + (size_t)(wave ^ 1) * 4 * WAVE + lane;
+  f32x4* const give = exchange + (size_t)wave * (OWN / 4) * WAVE + lane;
+  const f32x4* const take = exchange + (size_t)(wave ^ 1) * (OWN / 4) * WAVE + lane;
 
-  fetch(tile_first);
-  stash(0);
-  fetch(tile_first < tile_last ? tile_first + 1 : tile_last);
+  fetch(tile_first, 0);
+  stash(0, 0);
+  if (HALVES) {
+    fetch(tile_first, KP);
+    stash(0, KP);
+  }
+  fetch(tile_first < tile_last ? tile_first + 1 : tile_last, 0);
   block_sync_lds();
   for (int tile = tile_first; tile <= tile_last; ++tile) {
     const int cur = (tile - tile_first) & 1;
     const int key0 = tile * TALK_KEYS;
     const bool active = has_work && key0 <= wave_hi && key0 + TALK_KEYS - 1 >= wave_lo;  // uniform over the unit
-    f32x16 sc;
+    float own[OWN];  // scores of the tile's keys 8 half .. + 7 of 0 .. 15, of 16 .. 31, or both
     if (active) {
+      f32x16 sc;
 #pragma unroll
       for (int v = 0; v < 16; ++v) sc[v] = 0.f;
 #pragma unroll
       for (int c = 0; c < KH; ++c) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(kbase + c * 16), qreg[c], sc, 0, 0, 0);
+      if (SPLIT_VALUES) {
 #pragma unroll
-      for (int q = 0; q < 4; ++q) give[q * WAVE] = f32x4{sc[4 * q], sc[4 * q + 1], sc[4 * q + 2], sc[4 * q + 3]};
+        for (int q = 0; q < OWN / 4; ++q) give[q * WAVE] = f32x4{sc[4 * q], sc[4 * q + 1], sc[4 * q + 2], sc[4 * q + 3]};
+#pragma unroll
+        for (int v = 0; v < OWN; ++v) own[v] = sc[v];
+      } else if (side == 0) {  // uniform over the wave
+        give[0] = f32x4{sc[8], sc[9], sc[10], sc[11]}, give[WAVE] = f32x4{sc[12], sc[13], sc[14], sc[15]};
+#pragma unroll
+        for (int v = 0; v < 8; ++v) own[v] = sc[v];
+      } else {
+        give[0] = f32x4{sc[0], sc[1], sc[2], sc[3]}, give[WAVE] = f32x4{sc[4], sc[5], sc[6], sc[7]};
+#pragma unroll
+        for (int v = 0; v < 8; ++v) own[v] = sc[8 + v];
+      }
     }
-    block_sync_lds();  // the scores' halves are there; nobody reads this tile's keys any more
-    if (tile < tile_last) stash(cur ^ 1);
+    block_sync_lds();  // the handed-over sums are there; nobody reads this tile's keys any more
+    if (tile < tile_last) stash(cur ^ 1, 0);
     // (past the end the last tile again: cheaper than a branch around loads)
-    if (!LATE) fetch(tile + 2 <= tile_last ? tile + 2 : tile_last);
+    if (HALVES) fetch(tile < tile_last ? tile + 1 : tile_last, KP);
+    else fetch(tile + 2 <= tile_last ? tile + 2 : tile_last, 0);
     if (active) {
+      const int first = key0 + (SPLIT_VALUES ? 0 : 16 * side);
 #pragma unroll
-      for (int q = 0; q < 4; ++q) {
+      for (int q = 0; q < OWN / 4; ++q) {
         const f32x4 o = take[q * WAVE];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) sc[4 * q + e] += o[e];  // the same two numbers in both waves, and so the same sum
+        for (int e = 0; e < 4; ++e) own[4 * q + e] += o[e];
       }
-      if (!(key0 + TALK_KEYS - 1 <= full_hi && key0 >= full_lo)) {
+      if (!(first + 2 * OWN - 1 <= full_hi && first >= full_lo)) {
 #pragma unroll
-        for (int v = 0; v < 16; ++v) {
-          const int key = key0 + 16 * (v >> 3) + 8 * half + (v & 7);
-          sc[v] = (key <= qpos && key >= qlo) ? sc[v] : -INFINITY;
+        for (int v = 0; v < OWN; ++v) {
+          const int key = first + 16 * (v >> 3) + 8 * half + (v & 7);
+          own[v] = (key <= qpos && key >= qlo) ? own[v] : -INFINITY;
         }
       }
-      float mx = talk_max3(talk_max3(sc[0], sc[1], sc[2]), talk_max3(sc[3], sc[4], sc[5]), talk_max3(sc[6], sc[7], sc[8]));
-      mx = talk_max3(mx, talk_max3(sc[9], sc[10], sc[11]), talk_max3(sc[12], sc[13], talk_max2(sc[14], sc[15])));
+      float mx = own[0];
+#pragma unroll
+      for (int v = 1; v + 1 < OWN; v += 2) mx = talk_max3(mx, own[v], own[v + 1]);
+      mx = talk_max2(mx, own[OWN - 1]);
       {
         const unsigned u = __float_as_uint(mx);
         const auto halves = __builtin_amdgcn_permlane32_swap(u, u, false, false);  // the column's other lane
@@ -327,48 +376,87 @@ __global__ void __launch_bounds__(TALK_PREFILL_THREADS) __attribute__((amdgpu_wa
       const float m_new = talk_max2(m, mx * scale2);
       const float alpha = __builtin_amdgcn_exp2f(m - m_new);
       m = m_new;
-      float p[16], psum = 0.f;
+      float psum = 0.f;
 #pragma unroll
-      for (int v = 0; v < 16; ++v) {
-        p[v] = __builtin_amdgcn_exp2f(fmaf(sc[v], scale2, -m_new));
-        psum += p[v];
+      for (int v = 0; v < OWN; ++v) {
+        own[v] = __builtin_amdgcn_exp2f(fmaf(own[v], scale2, -m_new));
+        psum += own[v];
       }
       l = l * alpha + psum;
-      bf16x8 pmat[2];
-#pragma unroll
-      for (int e = 0; e < 2; ++e)
-        pmat[e] = bf16x8{(bf16)p[8 * e], (bf16)p[8 * e + 1], (bf16)p[8 * e + 2], (bf16)p[8 * e + 3],
-                         (bf16)p[8 * e + 4], (bf16)p[8 * e + 5], (bf16)p[8 * e + 6], (bf16)p[8 * e + 7]};
       if (__any(alpha != 1.f)) {  // the running maximum seldom moves after the first keys
 #pragma unroll
-        for (int dt = 0; dt < DH; ++dt) acc[dt] *= alpha;
+        for (int dt = 0; dt < DA; ++dt) acc[dt] *= alpha;
       }
 #pragma unroll
-      for (int dt = 0; dt < DH; ++dt) {
-        if (side * DH + dt < DT) {  // uniform over the wave
-          const bf16* vbase = vs + cur * L::V_ELEMS + (size_t)((side * DH + dt) * 32 + j) * VS + 8 * half;
+      for (int e = 0; e < OWN / 8; ++e) {
+        const bf16x8 pmat = {(bf16)own[8 * e], (bf16)own[8 * e + 1], (bf16)own[8 * e + 2], (bf16)own[8 * e + 3],
+                             (bf16)own[8 * e + 4], (bf16)own[8 * e + 5], (bf16)own[8 * e + 6], (bf16)own[8 * e + 7]};
+        const bf16* vbase = vs + cur * L::V_ELEMS + (size_t)((SPLIT_VALUES ? side * DA * 32 : 0) + j) * VS + (SPLIT_VALUES ? 16 * e : 16 * side) + 8 * half;
 #pragma unroll
-          for (int e = 0; e < 2; ++e) acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(vbase + 16 * e), pmat[e], acc[dt], 0, 0, 0);
-        }
+        for (int dt = 0; dt < DA; ++dt)
+          if (!SPLIT_VALUES || side * DA + dt < DT)  // uniform over the wave
+            acc[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(talk_load8(vbase + dt * 32 * VS), pmat, acc[dt], 0, 0, 0);
       }
     }
-    if (LATE) fetch(tile + 2 <= tile_last ? tile + 2 : tile_last);
-    block_sync_lds();  // the next tile's keys are there; this tile's values and the scores' halves are read
+    if (HALVES) {
+      if (tile < tile_last) stash(cur ^ 1, KP);
+      fetch(tile + 2 <= tile_last ? tile + 2 : tile_last, 0);
+    }
+    block_sync_lds();  // the next tile's keys are there; this tile's values and the handed-over sums are read
   }
-  if (!valid) return;
+  // ---- the two waves of a unit meet: the second hands its result over, one run of 32 value channels after the other ----
+  __syncthreads();  // the loads still under way, before the memory changes its use
   l += __shfl_xor(l, 32, WAVE);
-  if (a.sink != nullptr) l += __builtin_amdgcn_exp2f(a.sink[h] * TALK_LOG2E - m);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-  bf16* orow = a.out + (size_t)t * a.out_stride + (size_t)h * a.vdim;
+  if constexpr (SPLIT_VALUES) {  // both waves have the whole sums, and channels of their own
+    if (!valid) return;
+    if (a.sink != nullptr) l += __builtin_amdgcn_exp2f(a.sink[h] * TALK_LOG2E - m);
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    bf16* orow = a.out + (size_t)t * a.out_stride + (size_t)h * a.vdim;
 #pragma unroll
-  for (int dt = 0; dt < DH; ++dt) {
+    for (int dt = 0; dt < DA; ++dt) {
 #pragma unroll
-    for (int v = 0; v < 16; v += 4) {
-      const int d = (side * DH + dt) * 32 + 2 * v + 4 * half;
-      if (d < a.vdim)
-        *reinterpret_cast<bf16x4*>(orow + d) =
-            bf16x4{(bf16)(acc[dt][v] * inv), (bf16)(acc[dt][v + 1] * inv), (bf16)(acc[dt][v + 2] * inv), (bf16)(acc[dt][v + 3] * inv)};
+      for (int q = 0; q < 4; ++q) {
+        const int d = (side * DA + dt) * 32 + 8 * q + 4 * half;
+        if (d < a.vdim)
+          *reinterpret_cast<bf16x4*>(orow + d) = bf16x4{(bf16)(acc[dt][4 * q] * inv), (bf16)(acc[dt][4 * q + 1] * inv),
+                                                        (bf16)(acc[dt][4 * q + 2] * inv), (bf16)(acc[dt][4 * q + 3] * inv)};
+      }
     }
+    return;
+  }
+  f32x4* const hand = reinterpret_cast<f32x4*>(talk_lds) + (size_t)unit * 5 * WAVE + lane;  // [unit][4 + 1][lane]
+  float f0 = 0.f, f1 = 0.f;  // what the two results are multiplied by
+#pragma unroll
+  for (int dt = 0; dt < DA; ++dt) {
+    if (side == 1) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) hand[q * WAVE] = f32x4{acc[dt][4 * q], acc[dt][4 * q + 1], acc[dt][4 * q + 2], acc[dt][4 * q + 3]};
+      if (dt == 0) hand[4 * WAVE] = f32x4{m, l, 0.f, 0.f};
+    }
+    __syncthreads();
+    if (side == 0 && valid) {
+      if (dt == 0) {
+        const f32x4 other = hand[4 * WAVE];
+        float top = fmaxf(m, other[0]);
+        if (a.sink != nullptr) top = fmaxf(top, a.sink[h] * TALK_LOG2E);
+        f0 = __builtin_amdgcn_exp2f(m - top), f1 = __builtin_amdgcn_exp2f(other[0] - top);
+        float sum = l * f0 + other[1] * f1;
+        if (a.sink != nullptr) sum += __builtin_amdgcn_exp2f(a.sink[h] * TALK_LOG2E - top);
+        const float inv = sum > 0.f ? 1.f / sum : 0.f;
+        f0 *= inv, f1 *= inv;
+      }
+      bf16* orow = a.out + (size_t)t * a.out_stride + (size_t)h * a.vdim;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int d = dt * 32 + 8 * q + 4 * half;
+        const f32x4 o = hand[q * WAVE];
+        if (d < a.vdim)
+          *reinterpret_cast<bf16x4*>(orow + d) =
+              bf16x4{(bf16)(acc[dt][4 * q] * f0 + o[0] * f1), (bf16)(acc[dt][4 * q + 1] * f0 + o[1] * f1),
+                     (bf16)(acc[dt][4 * q + 2] * f0 + o[2] * f1), (bf16)(acc[dt][4 * q + 3] * f0 + o[3] * f1)};
+      }
+    }
+    __syncthreads();  // the memory carries the next run
   }
 }
 
@@ -405,7 +493,10 @@ __global__ void __launch_bounds__(TALK_DECODE_WAVES* WAVE)
   for (int i = threadIdx.x; i < 16 * (KW / 8); i += THREADS) {
     const int hh = i / (KW / 8), k = (i % (KW / 8)) * 8;
     bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (h0 + hh < a.nheads && k < row) v = talk_mixed_query(a.q + (size_t)t * a.q_stride, a, h0 + hh, k);
+    if (h0 + hh < a.nheads && k < row) {
+      const int c = k / a.dim;
+      v = talk_mixed_query(a.q + (size_t)t * a.q_stride, a.talk + (size_t)(h0 + hh) * a.nheads, c, k - c * a.dim, per, a.dim);
+    }
     *reinterpret_cast<bf16x8*>(qs + hh * KS + k) = v;
   }
   __syncthreads();
@@ -648,6 +739,7 @@ extern "C" int fmsamd_talking_attn_prefill(const void* q, long q_stride, void* o
   const int hb = talking_heads_of_block(nheads, kvheads);
   const long blocks = (long)n_qblocks * kvheads * (nheads / kvheads / hb);
   FMS_REQUIRE(blocks < (1L << 31), "talking_attn_prefill: too many blocks");
+  FMS_REQUIRE((long)hb * nheads * 4 <= TALK_UNITS * 2 * WAVE * 8 * 4, "talking_attn_prefill: %d heads", nheads);
   const int kw = talking_padded_row(kvheads, head_dim), dt = ceil_div(value_dim, 32);
 #define FMS_TP(KC, DT)                                                                                                                \
   do {                                                                                                                                \
