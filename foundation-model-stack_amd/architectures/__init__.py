@@ -1,4 +1,4 @@
-from . import basopel, defapel, llama, sidalorn, zimorax, zodolorn  # noqa: F401  (register the architectures, their adapters and variants)
+from . import basopel, defapel, kapuvik, llama, sidalorn, zimorax, zodolorn  # noqa: F401  (register the architectures, their adapters and variants)
 from .registry import (
     Architecture,
     architecture_for_hf,

@@ -8,6 +8,7 @@
 //                       into rows of any stride.
 //   cast_cols:          a run of columns of float32 rows as rows of their own, in the activation type.
 //   scale_f32:          x *= s in place.
+//   soft_cap_f32:       x = cap * tanh(x / cap) in place.
 #include "common.h"
 #include "fmsamd.h"
 
@@ -194,6 +195,19 @@ extern "C" int fmsamd_cast_cols(const float* x, long ldx, void* out, int out_dty
 
 __global__ void __launch_bounds__(256) scale_f32_kernel(float* __restrict__ x, size_t n, float s) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) x[i] *= s;
+}
+
+__global__ void __launch_bounds__(256) soft_cap_f32_kernel(float* __restrict__ x, size_t n, float cap) {
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int fmsamd_soft_cap_f32(float* x, long n, float cap, hipStream_t stream) {
+  if (n == 0) return 0;
+  FMS_REQUIRE(n > 0 && cap > 0.f, "soft_cap_f32: count %ld, cap %g", n, (double)cap);
+  const int blocks = ceil_div(n, 256) > 4096 ? 4096 : ceil_div(n, 256);
+  soft_cap_f32_kernel<<<blocks, 256, 0, stream>>>(x, (size_t)n, cap);
+  FMS_LAUNCH_CHECK("soft_cap_f32");
+  return 0;
 }
 
 extern "C" int fmsamd_scale_f32(float* x, long n, float s, hipStream_t stream) {

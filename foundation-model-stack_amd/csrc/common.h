@@ -89,6 +89,12 @@ __device__ __forceinline__ float fms_activate(float x, int kind) {
   }
 }
 
+// g sigmoid(alpha g) (u + shift) with g = min(gate, limit) and u = clamp(up, -limit, limit)
+__device__ __forceinline__ float clamped_gate(float gate, float up, float limit, float alpha, float shift) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + shift);
+}
+
 // --------------------------------------------------------------------------
 // reductions
 // --------------------------------------------------------------------------

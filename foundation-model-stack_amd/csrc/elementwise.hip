@@ -306,14 +306,65 @@ extern "C" int fmsamd_stream_rows(const float* resid, const void* branch, const 
 // --------------------------------------------------------------------------
 __device__ __forceinline__ float activate(float x, int kind) { return fms_activate(x, kind); }
 
+// --------------------------------------------------------------------------
+// a new stream from the old one, what is still to be added to it, another stream and a vector
+// --------------------------------------------------------------------------
+template <int VEC, typename T>
+__global__ void __launch_bounds__(256)
+    stream_enter_kernel(const float* __restrict__ resid, const T* __restrict__ branch, const float* __restrict__ branch_scale,
+                        const float* __restrict__ base, const float* __restrict__ shift, float* __restrict__ out, int width) {
+  const size_t at = (size_t)blockIdx.x * width;
+  for (int i = threadIdx.x * VEC; i < width; i += blockDim.x * VEC) {
+    float v[VEC], w[VEC];
+    load_vec<VEC>(resid + at + i, v);
+    if (branch != nullptr) {
+      load_branch<VEC>(branch + at + i, branch_scale ? branch_scale + i : nullptr, w);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += w[e];
+    }
+    if (base != nullptr) {
+      load_vec<VEC>(base + at + i, w);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += w[e];
+    }
+    if (shift != nullptr) {
+      load_vec<VEC>(shift + i, w);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += w[e];
+    }
+    store_vec<VEC>(out + at + i, v);
+  }
+}
+
+extern "C" int fmsamd_stream_enter(const float* resid, const void* branch, int act_dtype, const float* branch_scale, const float* base,
+                                   const float* shift, float* out, int n_tokens, int width, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  FMS_REQUIRE(n_tokens > 0 && width > 0, "stream_enter: bad sizes T=%d width=%d", n_tokens, width);
+  const bool by_fours = width % 4 == 0 && (((size_t)resid | (size_t)branch | (size_t)branch_scale | (size_t)base | (size_t)shift | (size_t)out) & 15) == 0;
+  const int threads = width >= 1024 ? 256 : 64;
+#define FMS_SE(V, T) stream_enter_kernel<V, T><<<n_tokens, threads, 0, stream>>>(resid, (const T*)branch, branch_scale, base, shift, out, width)
+  if (act_dtype == FMS_F32) {
+    if (by_fours) FMS_SE(4, float);
+    else FMS_SE(1, float);
+  } else if (act_dtype == FMS_BF16) {
+    if (by_fours) FMS_SE(4, bf16);
+    else FMS_SE(1, bf16);
+  } else {
+    FMS_REQUIRE(false, "stream_enter: unknown dtype %d", act_dtype);
+  }
+#undef FMS_SE
+  FMS_LAUNCH_CHECK("stream_enter");
+  return 0;
+}
+
 // VEC elements per thread and step: 16 bytes of the activation type when the row length allows it
 template <int VEC, typename T, typename BiasT>
 __global__ void gated_act_kernel(const T* __restrict__ gu, const BiasT* __restrict__ bias, T* __restrict__ out,
-                                 int hidden, int act) {
+                                 long ldo, int hidden, int act, fmsamd_gate_clamp clamp) {
   const size_t t = blockIdx.y;
   const T* g = gu + t * 2 * hidden;
   const T* u = g + hidden;
-  T* o = out + t * hidden;
+  T* o = out + t * ldo;
   for (int j = (blockIdx.x * blockDim.x + threadIdx.x) * VEC; j < hidden; j += gridDim.x * blockDim.x * VEC) {
     __attribute__((aligned(16))) T gv[VEC], uv[VEC], ov[VEC];
     if constexpr (VEC * sizeof(T) == 16) {
@@ -330,7 +381,7 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const BiasT* __restri
         a += to_f32(bias[j + e]);
         b += to_f32(bias[hidden + j + e]);
       }
-      ov[e] = from_f32<T>(activate(a, act) * b);
+      ov[e] = from_f32<T>(act == FMS_ACT_CLAMPED_GATE ? clamped_gate(a, b, clamp.limit, clamp.alpha, clamp.shift) : activate(a, act) * b);
     }
     if constexpr (VEC * sizeof(T) == 16) {
       *reinterpret_cast<f32x4*>(o + j) = *reinterpret_cast<const f32x4*>(ov);
@@ -342,33 +393,36 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const BiasT* __restri
 }
 
 template <typename T, typename BiasT>
-static void launch_gated_act(const void* gu, const void* bias, void* out, int n_tokens, int hidden, int act,
-                             hipStream_t stream) {
+static void launch_gated_act(const void* gu, const void* bias, void* out, long ldo, int n_tokens, int hidden, int act,
+                             fmsamd_gate_clamp clamp, hipStream_t stream) {
   constexpr int VEC = 16 / sizeof(T);
-  const bool wide = hidden % VEC == 0 && (((size_t)gu | (size_t)out) & 15) == 0;
+  const bool wide = hidden % VEC == 0 && ldo % VEC == 0 && (((size_t)gu | (size_t)out) & 15) == 0;
   const int per_thread = wide ? VEC : 1;
   const int blocks = ceil_div(hidden, 256 * per_thread);
   dim3 grid(blocks > 64 ? 64 : blocks, n_tokens);
   if (wide)
-    gated_act_kernel<VEC, T, BiasT><<<grid, 256, 0, stream>>>((const T*)gu, (const BiasT*)bias, (T*)out, hidden, act);
+    gated_act_kernel<VEC, T, BiasT><<<grid, 256, 0, stream>>>((const T*)gu, (const BiasT*)bias, (T*)out, ldo, hidden, act, clamp);
   else
-    gated_act_kernel<1, T, BiasT><<<grid, 256, 0, stream>>>((const T*)gu, (const BiasT*)bias, (T*)out, hidden, act);
+    gated_act_kernel<1, T, BiasT><<<grid, 256, 0, stream>>>((const T*)gu, (const BiasT*)bias, (T*)out, ldo, hidden, act, clamp);
 }
 
-extern "C" int fmsamd_gated_act(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, int n_tokens,
-                                int hidden, int act, hipStream_t stream) {
+extern "C" int fmsamd_gated_act(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, long ldo, int n_tokens,
+                                int hidden, int act, const fmsamd_gate_clamp* clamp_in, hipStream_t stream) {
   if (n_tokens == 0) return 0;
-  FMS_REQUIRE(n_tokens > 0 && hidden > 0, "gated_act: bad sizes T=%d hidden=%d", n_tokens, hidden);
+  FMS_REQUIRE(n_tokens > 0 && hidden > 0 && ldo >= hidden, "gated_act: bad sizes T=%d hidden=%d", n_tokens, hidden);
   FMS_REQUIRE(act >= FMS_ACT_SILU && act <= FMS_ACT_LAST, "gated_act: unknown activation %d", act);
   FMS_REQUIRE(n_tokens <= 65535, "gated_act: %d tokens exceed one launch (65535)", n_tokens);
+  FMS_REQUIRE(clamp_in == nullptr || clamp_in->limit > 0.f, "gated_act: a limit of %g", (double)clamp_in->limit);
+  const fmsamd_gate_clamp clamp = clamp_in ? *clamp_in : fmsamd_gate_clamp{0.f, 0.f, 0.f};
+  if (clamp_in) act = FMS_ACT_CLAMPED_GATE;
   if (dtype == FMS_F32 && (bias == nullptr || bias_dtype == FMS_F32))
-    launch_gated_act<float, float>(gu, bias, out, n_tokens, hidden, act, stream);
+    launch_gated_act<float, float>(gu, bias, out, ldo, n_tokens, hidden, act, clamp, stream);
   else if (dtype == FMS_BF16 && (bias == nullptr || bias_dtype == FMS_BF16))
-    launch_gated_act<bf16, bf16>(gu, bias, out, n_tokens, hidden, act, stream);
+    launch_gated_act<bf16, bf16>(gu, bias, out, ldo, n_tokens, hidden, act, clamp, stream);
   else if (dtype == FMS_BF16 && bias_dtype == FMS_F32)
-    launch_gated_act<bf16, float>(gu, bias, out, n_tokens, hidden, act, stream);
+    launch_gated_act<bf16, float>(gu, bias, out, ldo, n_tokens, hidden, act, clamp, stream);
   else if (dtype == FMS_F32 && bias_dtype == FMS_BF16)
-    launch_gated_act<float, bf16>(gu, bias, out, n_tokens, hidden, act, stream);
+    launch_gated_act<float, bf16>(gu, bias, out, ldo, n_tokens, hidden, act, clamp, stream);
   else
     FMS_REQUIRE(false, "gated_act: unknown dtypes %d/%d", dtype, bias_dtype);
   FMS_LAUNCH_CHECK("gated_act");

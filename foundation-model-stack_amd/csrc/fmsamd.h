@@ -6,7 +6,7 @@
 
 #include <hip/hip_runtime.h>
 
-#define FMSAMD_ABI_VERSION 11
+#define FMSAMD_ABI_VERSION 12
 
 // element types
 #define FMS_F32 0
@@ -23,6 +23,7 @@
 #define FMS_ACT_GELU_TANH 7  // the tanh approximation
 #define FMS_ACT_RELU2 8      // the square of relu
 #define FMS_ACT_LAST FMS_ACT_RELU2
+#define FMS_ACT_CLAMPED_GATE 100  // inside the kernels: a gated unit with an fmsamd_gate_clamp
 
 #ifdef __cplusplus
 extern "C" {
@@ -46,9 +47,15 @@ int fmsamd_add_norm(float* resid, const void* branch, int act_dtype, const void*
 int fmsamd_stream_rows(const float* resid, const void* branch, const float* branch_scale, void* out, int act_dtype, long ldo,
                        int n_tokens, int width, hipStream_t stream);
 
-// out[t, j] = act(gu[t, j] + b[j]) * (gu[t, hidden + j] + b[hidden + j])
-int fmsamd_gated_act(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, int n_tokens, int hidden,
-                     int act, hipStream_t stream);
+// The clamped gated unit: g sigmoid(alpha g) (u + shift) with g = min(gate, limit) and u = clamp(up, -limit, limit)
+typedef struct fmsamd_gate_clamp {
+  float limit, alpha, shift;
+} fmsamd_gate_clamp;
+
+// out[t, j] = act(gu[t, j] + b[j]) * (gu[t, hidden + j] + b[hidden + j]), or the clamped unit of the two sums (clamp, may be
+// null: act is then not used); rows of out ldo apart
+int fmsamd_gated_act(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, long ldo, int n_tokens, int hidden,
+                     int act, const fmsamd_gate_clamp* clamp, hipStream_t stream);
 
 // positions[i] += 1 where seq_of_token[i] >= 0
 int fmsamd_advance_positions(int* positions, const int* seq_of_token, int n, hipStream_t stream);
@@ -135,7 +142,7 @@ int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, const void* 
                             void* workspace, long workspace_bytes, hipStream_t stream);
 int fmsamd_gemm_skinny_gated_bf16(const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
                                   int out_dtype, long ldo, int M, int hidden, int K, int act,
-                                  const fmsamd_row_scale* row_scale, void* workspace, long workspace_bytes,
+                                  const fmsamd_gate_clamp* clamp, const fmsamd_row_scale* row_scale, void* workspace, long workspace_bytes,
                                   hipStream_t stream);
 // resid += x W^T (+ bias) in float32; scaled = resid * norm_w in bfloat16; partials[M, partial_count] = sums
 // of squares of resid by groups of columns (partial_count as fmsamd_gemm_skinny_residual_partials(M, N, K) says;
@@ -315,7 +322,7 @@ int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const float* a, 
 int fmsamd_delta_rule(const float* qkv, const float* beta, const float* decay, const float* kq, float* state, float* out,
                       const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
                       int kv_heads, int dim, int vdim, int per_channel, int single_tokens, hipStream_t stream);
-// out[t, h, :] = o[t, h, :] / rms * weight * act(gate[t, h, :]) * out_scale
+// out[t, h, :] = o[t, h, :] / rms * weight (null: no weight) * act(gate[t, h, :]) * out_scale
 int fmsamd_gated_head_norm(const float* o, const float* gate, long ldg, const void* weight, int weight_dtype, float eps,
                            int act, float out_scale, void* out, int out_dtype, long ldo, const int* seq_of_token,
                            int n_tokens, int heads, int vdim, hipStream_t stream);
@@ -409,6 +416,46 @@ int fmsamd_ssd_step(const float* proj, long ld, int col_x, int col_dt, const voi
 int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void* weight, int weight_dtype, int parts, float eps,
                             void* out, int out_dtype, const int* seq_of_token, int n_tokens, int cols, const float* conv_x, long ld_conv,
                             int channels, int taps, float* conv_state, const int* slot_ids, hipStream_t stream);
+
+// Linear attention with a decay (linear_recurrence.hip): S <- S diag(a) + v k^T, o = S q per head, over the tokens of every
+// sequence, from and into state [slots][heads][vdim][dim] (float32).  Every token's row of proj (float32, ld apart) holds q and
+// k (heads * dim entries from col_q, col_k on), v and gate logits (heads * vdim from col_v, col_g on).  Decays: a = exp(log_decay)
+// per head, or (up_t) sigmoid(z)^inv_tau per head and key channel, z = up (the rank numbers from col_low on) + up_bias with
+// up_t [rank][heads * dim].  rot_dim > 0: the first rot_dim channels of q and k are rotated in neighbouring pairs by the
+// token's position.  q is multiplied by q_scale.  The walk writes o / rms(o) * norm_w (or no weight) * act(gate) * out_scale to
+// rows of out (ldo apart, zeros for padding rows); the chunked form (long steps) writes o itself.
+typedef struct fmsamd_linear_recurrence {
+  const float* proj;
+  long ld;
+  int col_q, col_k, col_v, col_g, col_low;
+  int heads, dim, vdim, rank;
+  const float *log_decay, *up_t, *up_bias;
+  float inv_tau;
+  int rot_dim, max_pos;
+  const float *cos_t, *sin_t;
+  const int* positions;
+  float q_scale;
+  float* state;
+  const int *seq_starts, *seq_of_token, *slot_ids;
+  int n_seqs, n_tokens;
+  const float* norm_w;
+  float eps, out_scale;
+  int act;
+  void* out;
+  int out_dtype;
+  long ldo;
+} fmsamd_linear_recurrence;
+int fmsamd_linear_recurrence_walk(const fmsamd_linear_recurrence* args, hipStream_t stream);
+long fmsamd_linear_recurrence_workspace(int n_tokens, int n_seqs, int heads, int dim);
+int fmsamd_linear_recurrence_chunked(const fmsamd_linear_recurrence* args, float* y, int longest, float* workspace,
+                                     long workspace_bytes, hipStream_t stream);
+
+// out[t] = resid[t] + branch[t] * branch_scale + base[t] + shift, float32 rows (branch in the activation type; branch,
+// branch_scale, base and shift (width entries) may be null)
+int fmsamd_stream_enter(const float* resid, const void* branch, int act_dtype, const float* branch_scale, const float* base,
+                        const float* shift, float* out, int n_tokens, int width, hipStream_t stream);
+// x = cap * tanh(x / cap) in place
+int fmsamd_soft_cap_f32(float* x, long n, float cap, hipStream_t stream);
 
 #ifdef __cplusplus
 }

@@ -226,7 +226,7 @@ template <int SK_WAVES, int UNR, int NTB, int MT, int EPI, typename OutT, typena
 __global__ void __launch_bounds__(SK_WAVES* WAVE)
     __attribute__((amdgpu_waves_per_eu(MT > 1 ? 2 : 4)))  // two blocks a compute unit; one with several tiles of x
     skinny_bf16_kernel(const bf16* __restrict__ x, long ldx, const bf16* __restrict__ w, const BiasT* __restrict__ bias,
-                       OutT* __restrict__ out, long ldo, int M, int N, int K, int tile2_offset, int act,
+                       OutT* __restrict__ out, long ldo, int M, int N, int K, int tile2_offset, OutAct act,
                        int rows_per_block, RowScale scale, RopeEpilogue rope, ResidEpilogue res) {
   constexpr bool GATED = EPI == EPI_GATED;
   // per wave: one tile of 16 rows x 128 k (4 KB) of W and one of x between load and MFMA layout; after
@@ -468,7 +468,7 @@ __global__ void __launch_bounds__(SK_WAVES* WAVE)
         v += to_f32(bias[n]);
         u += to_f32(bias[tile2_offset + n]);
       }
-      out[(size_t)m * ldo + n] = from_f32<OutT>(sk_activate(v, act) * u);
+      out[(size_t)m * ldo + n] = from_f32<OutT>(sk_gated(v, u, act));
     } else if (EPI == EPI_ROPE) {
       if (bias && live) v += to_f32(bias[n]);
       const float partner = __shfl_xor(v, 1, WAVE);  // the other element of the rotary pair: N is a multiple of 16
@@ -510,14 +510,14 @@ __global__ void __launch_bounds__(SK_WAVES* WAVE)
     } else {
       if (!live) continue;
       if (bias) v += to_f32(bias[n]);
-      out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v, act));
+      out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v, act.kind));
     }
   }
 }
 
 template <int NTB, int MT, int EPI>
 static void launch_skinny(const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
-                          int out_dtype, long ldo, int M, int N, int K, int tile2_offset, int act, int rows_per_block,
+                          int out_dtype, long ldo, int M, int N, int K, int tile2_offset, OutAct act, int rows_per_block,
                           hipStream_t stream, RowScale scale, RopeEpilogue rope = RopeEpilogue{},
                           ResidEpilogue res = ResidEpilogue{}) {
   const int blocks = ceil_div(N, rows_per_block);
@@ -602,11 +602,11 @@ extern "C" int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, c
   FMS_REQUIRE(ldx >= K && ldo >= N, "gemm_skinny_bf16: leading dimensions too small");
   FMS_REQUIRE(out_dtype == FMS_BF16 || out_dtype == FMS_F32, "gemm_skinny_bf16: unknown output dtype %d", out_dtype);
   if (M > 16 && !skinny_takes_many_rows(M, N, K))
-    return wide_product(EPI_PLAIN, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, act, scale, RopeEpilogue{},
+    return wide_product(EPI_PLAIN, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, plain_act(act), scale, RopeEpilogue{},
                         ResidEpilogue{}, workspace, workspace_bytes, stream);
   const int rows = skinny_rows_per_block(N, M);
 #define FMS_LS(NTB, MT) \
-  launch_skinny<NTB, MT, EPI_PLAIN>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, act, rows, stream, scale)
+  launch_skinny<NTB, MT, EPI_PLAIN>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, N, K, 0, plain_act(act), rows, stream, scale)
 #define FMS_LS_MT(NTB)  \
   do {                  \
     if (M <= 16)        \
@@ -624,11 +624,11 @@ extern "C" int fmsamd_gemm_skinny_bf16(const void* x, long ldx, const void* w, c
   return 0;
 }
 
-// out[M, hidden] = act(x Wg^T + bg) * (x Wu^T + bu) with w = [Wg; Wu] stacked, [2*hidden, K].  M <= 192.
+// out[M, hidden] = act(x Wg^T + bg) * (x Wu^T + bu), or the clamped unit of both, with w = [Wg; Wu] stacked, [2*hidden, K].  M <= 192.
 extern "C" int fmsamd_gemm_skinny_gated_bf16(const void* x, long ldx, const void* w, const void* bias,
                                              int bias_dtype, void* out, int out_dtype, long ldo, int M, int hidden,
-                                             int K, int act, const fmsamd_row_scale* row_scale, void* workspace,
-                                             long workspace_bytes, hipStream_t stream) {
+                                             int K, int act, const fmsamd_gate_clamp* clamp, const fmsamd_row_scale* row_scale,
+                                             void* workspace, long workspace_bytes, hipStream_t stream) {
   if (M == 0 || hidden == 0) return 0;
   RowScale scale;
   if (row_scale_of(row_scale, K, &scale)) return -1;
@@ -639,11 +639,13 @@ extern "C" int fmsamd_gemm_skinny_gated_bf16(const void* x, long ldx, const void
   FMS_REQUIRE(ldx >= K && ldo >= hidden, "gemm_skinny_gated_bf16: leading dimensions too small");
   FMS_REQUIRE(out_dtype == FMS_BF16 || out_dtype == FMS_F32, "gemm_skinny_gated_bf16: unknown output dtype %d", out_dtype);
   FMS_REQUIRE(act >= FMS_ACT_SILU && act <= FMS_ACT_LAST, "gemm_skinny_gated_bf16: unknown activation %d", act);
+  FMS_REQUIRE(clamp == nullptr || clamp->limit > 0.f, "gemm_skinny_gated_bf16: a limit of %g", (double)clamp->limit);
+  const OutAct unit = clamp ? OutAct{FMS_ACT_CLAMPED_GATE, clamp->limit, clamp->alpha, clamp->shift} : plain_act(act);
   if (M > 16)
-    return wide_product(EPI_GATED, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, hidden, K, hidden, act, scale,
+    return wide_product(EPI_GATED, x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, hidden, K, hidden, unit, scale,
                         RopeEpilogue{}, ResidEpilogue{}, workspace, workspace_bytes, stream);
 #define FMS_LG(MT) \
-  launch_skinny<2, MT, EPI_GATED>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, hidden, K, hidden, act,     \
+  launch_skinny<2, MT, EPI_GATED>(x, ldx, w, bias, bias_dtype, out, out_dtype, ldo, M, hidden, K, hidden, unit,    \
                                   skinny_gated_rows_per_block(hidden, M), stream, scale)
   FMS_LG(1);
 #undef FMS_LG
@@ -678,11 +680,11 @@ extern "C" int fmsamd_qkv_rope_skinny_bf16(const void* x, long ldx, const void* 
   RopeEpilogue rope{positions, seq_of_token, block_table, table_stride, rot_dim > 0 ? cos_t : nullptr, sin_t, rot_dim,
                     max_pos, (bf16*)k_cache, (bf16*)v_cache, nheads, kvheads, head_dim};
   if (M > 16 && !skinny_takes_many_rows(M, N, K))
-    return wide_product(EPI_ROPE, x, ldx, w, bias, bias_dtype, out, FMS_BF16, ldo, M, N, K, 0, 0, scale, rope,
+    return wide_product(EPI_ROPE, x, ldx, w, bias, bias_dtype, out, FMS_BF16, ldo, M, N, K, 0, plain_act(FMS_ACT_IDENTITY), scale, rope,
                         ResidEpilogue{}, workspace, workspace_bytes, stream);
   const int rows = skinny_rows_per_block(N, M);
 #define FMS_LR(NTB, MT) \
-  launch_skinny<NTB, MT, EPI_ROPE>(x, ldx, w, bias, bias_dtype, out, FMS_BF16, ldo, M, N, K, 0, 0, rows, stream, scale, rope)
+  launch_skinny<NTB, MT, EPI_ROPE>(x, ldx, w, bias, bias_dtype, out, FMS_BF16, ldo, M, N, K, 0, plain_act(FMS_ACT_IDENTITY), rows, stream, scale, rope)
 #define FMS_LR_MT(NTB)  \
   do {                  \
     if (M <= 16)        \
@@ -744,11 +746,11 @@ extern "C" int fmsamd_gemm_skinny_residual_bf16(const void* x, long ldx, const v
     res.tiles = tiles;  // the finish kernel writes exactly these
     FMS_REQUIRE(partial_count == tiles, "gemm_skinny_residual_bf16: %d partial sums per row, %d expected", partial_count,
                 tiles);
-    return wide_product(EPI_RESID, x, ldx, w, bias, bias_dtype, scaled, FMS_BF16, ldo, M, N, K, 0, 0, scale,
+    return wide_product(EPI_RESID, x, ldx, w, bias, bias_dtype, scaled, FMS_BF16, ldo, M, N, K, 0, plain_act(FMS_ACT_IDENTITY), scale,
                         RopeEpilogue{}, res, workspace, workspace_bytes, stream);
   }
 #define FMS_LX(NTB, MT)                                                                                              \
-  launch_skinny<NTB, MT, EPI_RESID>(x, ldx, w, bias, bias_dtype, scaled, FMS_BF16, ldo, M, N, K, 0, 0, rows, stream, \
+  launch_skinny<NTB, MT, EPI_RESID>(x, ldx, w, bias, bias_dtype, scaled, FMS_BF16, ldo, M, N, K, 0, plain_act(FMS_ACT_IDENTITY), rows, stream, \
                                     scale, RopeEpilogue{}, res)
 #define FMS_LX_MT(NTB)  \
   do {                  \

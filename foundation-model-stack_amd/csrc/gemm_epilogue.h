@@ -18,9 +18,23 @@ __device__ __forceinline__ float sk_plain(float x, int act) {
   return act == FMS_ACT_RELU2 ? r * r : r;
 }
 
+// What a product finishes an element with: an activation, and for the clamped gated unit (FMS_ACT_CLAMPED_GATE, gated
+// products only) its constants.
+struct OutAct {
+  int kind;
+  float limit, alpha, shift;
+};
+static inline OutAct plain_act(int kind) { return OutAct{kind, 0.f, 0.f, 0.f}; }
+
+// The gated unit: act(gate) * up, or g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit).
+__device__ __forceinline__ float sk_gated(float gate, float up, const OutAct& a) {
+  if (a.kind == FMS_ACT_CLAMPED_GATE) return clamped_gate(gate, up, a.limit, a.alpha, a.shift);
+  return sk_activate(gate, a.kind) * up;
+}
+
 // What the skinny kernel does with a finished output element.
 #define EPI_PLAIN 0  // store act(product + bias), act one of identity, relu and its square
-#define EPI_GATED 1  // the block's second tile is the "up" half: out = act(first) * second, N is the hidden size
+#define EPI_GATED 1  // the block's second tile is the "up" half: out = act(first) * second (or the clamped unit), N is the hidden size
 #define EPI_ROPE 2   // the output row is [queries | keys | values] of attention: rotate q and k, store q, and
                      // write k and v into their cache pages (layout: see rope.hip)
 #define EPI_RESID 3  // add the product to the float32 residual stream in place, store the new stream times the
@@ -66,5 +80,5 @@ struct RopeEpilogue {
 // `rows` counts all rows of W (for the gated product both halves).
 long wide_workspace_bytes(int M, int rows, int K);
 int wide_product(int epi, const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
-                 int out_dtype, long ldo, int M, int N, int K, int tile2_offset, int act, RowScale scale,
+                 int out_dtype, long ldo, int M, int N, int K, int tile2_offset, OutAct act, RowScale scale,
                  RopeEpilogue rope, ResidEpilogue res, void* workspace, long workspace_bytes, hipStream_t stream);

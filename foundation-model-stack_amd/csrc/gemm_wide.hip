@@ -35,7 +35,8 @@ struct WideOut {
   long ldo;
   const void* bias;
   int bias_f32;
-  int N, tile2_offset, act;
+  int N, tile2_offset;
+  OutAct act;
   int gate_rows;  // WD_GATED: gate rows (and up rows) a block owns, a multiple of 4, at most 64
   int vec;  // rows of the destination start 16-byte aligned: four elements at a time
   RowScale scale;
@@ -306,7 +307,7 @@ __global__ void __launch_bounds__(512)
           v += wide_bias(o, n + e);
           u += wide_bias(o, o.tile2_offset + n + e);
         }
-        res[e] = sk_activate(v, o.act) * u;
+        res[e] = sk_gated(v, u, o.act);
       }
       if (o.vec && n + 3 < n_hi) {
         store4(out + (size_t)m * o.ldo + n, res);
@@ -332,7 +333,7 @@ __global__ void __launch_bounds__(512)
         for (int e = 0; e < 4; ++e) {
           v[e] *= rs;
           if (o.bias != nullptr && n + e < n_lim) v[e] += wide_bias(o, n + e);
-          v[e] = sk_plain(v[e], o.act);
+          v[e] = sk_plain(v[e], o.act.kind);
         }
         OutT* const out = (OutT*)o.out;
         if (o.vec && n + 3 < n_lim) {
@@ -360,7 +361,7 @@ __global__ void __launch_bounds__(512)
 template <int EPI, typename OutT, typename BiasT>
 __global__ void __launch_bounds__(256)
     wide_finish_kernel(const float* __restrict__ part, int slices, int rows, const BiasT* __restrict__ bias,
-                       OutT* __restrict__ out, long ldo, int M, int N, int tile2_offset, int act, RowScale scale,
+                       OutT* __restrict__ out, long ldo, int M, int N, int tile2_offset, OutAct act, RowScale scale,
                        RopeEpilogue rope, ResidEpilogue res) {
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   const int m = blockIdx.y * 4 + wave;
@@ -433,7 +434,7 @@ __global__ void __launch_bounds__(256)
 
   if (EPI == EPI_GATED) {
     if (!live) return;
-    out[(size_t)m * ldo + n] = from_f32<OutT>(sk_activate(v + bias_v, act) * (u + bias_u));
+    out[(size_t)m * ldo + n] = from_f32<OutT>(sk_gated(v + bias_v, u + bias_u, act));
   } else if (EPI == EPI_ROPE) {
     v += bias_v;
     const float partner = __shfl_xor(v, 1, WAVE);  // the other element of the rotary pair (N is even)
@@ -476,7 +477,7 @@ __global__ void __launch_bounds__(256)
     if ((lane & 15) == 0 && n / 16 < res.tiles) res.partials[(size_t)m * res.tiles + n / 16] = sq;
   } else {
     if (!live) return;
-    out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v + bias_v, act));
+    out[(size_t)m * ldo + n] = from_f32<OutT>(sk_plain(v + bias_v, act.kind));
   }
 }
 
@@ -510,7 +511,7 @@ long wide_workspace_bytes(int M, int rows, int K) {
 
 template <int EPI>
 static void launch_finish(const float* part, int slices, int rows, const void* bias, int bias_dtype, void* out,
-                          int out_dtype, long ldo, int M, int N, int tile2_offset, int act, RowScale scale,
+                          int out_dtype, long ldo, int M, int N, int tile2_offset, OutAct act, RowScale scale,
                           RopeEpilogue rope, ResidEpilogue res, hipStream_t stream) {
   dim3 grid(ceil_div(N, WAVE), ceil_div(M, 4));
   const bool fb = bias != nullptr && bias_dtype == FMS_F32;
@@ -576,7 +577,7 @@ static bool aligned16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 
 // N: columns of the output (for the gated product the hidden size; W then has tile2_offset + N rows).
 int wide_product(int epi, const void* x, long ldx, const void* w, const void* bias, int bias_dtype, void* out,
-                 int out_dtype, long ldo, int M, int N, int K, int tile2_offset, int act, RowScale scale,
+                 int out_dtype, long ldo, int M, int N, int K, int tile2_offset, OutAct act, RowScale scale,
                  RopeEpilogue rope, ResidEpilogue res, void* workspace, long workspace_bytes, hipStream_t stream) {
   const int rows = epi == EPI_GATED ? tile2_offset + N : N;
   FMS_REQUIRE(M > 16 && M <= WD_MAX_ROWS, "wide product: %d rows (17..%d)", M, WD_MAX_ROWS);
@@ -625,10 +626,10 @@ int wide_product(int epi, const void* x, long ldx, const void* w, const void* bi
                                rope, res, stream);
       break;
     case EPI_ROPE:
-      launch_finish<EPI_ROPE>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, 0, scale, rope, res, stream);
+      launch_finish<EPI_ROPE>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, act, scale, rope, res, stream);
       break;
     default:
-      launch_finish<EPI_RESID>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, 0, scale, rope, res, stream);
+      launch_finish<EPI_RESID>(part, slices, rows, bias, bias_dtype, out, out_dtype, ldo, M, N, 0, act, scale, rope, res, stream);
   }
   FMS_LAUNCH_CHECK("wide product finish");
   return 0;

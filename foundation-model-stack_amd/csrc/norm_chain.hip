@@ -335,12 +335,6 @@ extern "C" int fmsamd_activate(const void* x, void* out, int dtype, long n, int 
   return 0;
 }
 
-__device__ __forceinline__ float clamped_gate(float g, float u, float limit, float alpha, float shift) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + shift);
-}
-
 // gu [T, 2 * hidden] (gate first), out [T, hidden]; hidden a multiple of 4: four elements a thread and step
 template <typename T>
 __global__ void clamped_gated_act4_kernel(const T* __restrict__ gu, T* __restrict__ out, int hidden, float limit, float alpha,

@@ -24,7 +24,11 @@ class DecoderModel(Part):
         self.embedding = self.add_child(spec.embedding_name, make_part("embedding", spec.embedding.kind, vocab=spec.vocab, width=spec.width, **spec.embedding.args))
         self.layers: List[Part] = []
         for i, layer in enumerate(spec.layers):
-            pos = self.positions[layer.position] if layer.position is not None else None
+            pos = None
+            if isinstance(layer.position, dict):
+                pos = {side: self.positions[key] for side, key in layer.position.items()}
+            elif layer.position is not None:
+                pos = self.positions[layer.position]
             mixer = make_part("mixer", layer.mixer.kind, width=spec.width, position_encoder=pos, **layer.mixer.args)
             ff = None  # a layer may have no feed-forward, if its block takes None
             if layer.feed_forward is not None:

@@ -17,7 +17,7 @@ import torch  # noqa: F401  (loads libamdhip64 before our library asks for it)
 
 from . import build as _build
 
-ABI_VERSION = 11
+ABI_VERSION = 12
 
 _lib: Optional[ctypes.CDLL] = None
 _lock = threading.Lock()
@@ -28,7 +28,7 @@ _SIGNATURES = {
     "fmsamd_embed": [P, P, I, P, I, I, I, F, P],
     "fmsamd_add_norm": [P, P, I, P, P, I, P, P, I, I, F, I, P, P],
     "fmsamd_stream_rows": [P, P, P, P, I, L, I, I, P],
-    "fmsamd_gated_act": [P, P, I, P, I, I, I, I, P],
+    "fmsamd_gated_act": [P, P, I, P, I, L, I, I, I, P, P],
     "fmsamd_cast": [P, I, P, I, L, P],
     "fmsamd_advance_positions": [P, P, I, P],
     "fmsamd_bias_add": [P, I, P, I, I, I, P],
@@ -43,7 +43,7 @@ _SIGNATURES = {
     "fmsamd_gemm_bf16_any": [P, L, P, P, I, P, I, L, I, I, I, P],
     "fmsamd_gemm_skinny_workspace": [I, I, I],
     "fmsamd_gemm_skinny_bf16": [P, L, P, P, I, P, I, L, I, I, I, I, P, P, L, P],
-    "fmsamd_gemm_skinny_gated_bf16": [P, L, P, P, I, P, I, L, I, I, I, I, P, P, L, P],
+    "fmsamd_gemm_skinny_gated_bf16": [P, L, P, P, I, P, I, L, I, I, I, I, P, P, P, L, P],
     "fmsamd_gemm_skinny_residual_partials": [I, I, I],
     "fmsamd_gemm_skinny_residual_bf16": [P, L, P, P, I, P, L, P, I, P, L, P, I, I, I, I, P, P, L, P],
     "fmsamd_sample": [P, L, I, I, I, F, I, P, P, P],
@@ -87,6 +87,10 @@ _SIGNATURES = {
     "fmsamd_ssd_chunked": [P, L, P, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, L, P],
     "fmsamd_ssd_step": [P, L, I, I, P, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
     "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P, L, I, I, P, P, P],
+    "fmsamd_linear_recurrence_walk": [P, P],
+    "fmsamd_linear_recurrence_chunked": [P, P, I, P, L, P],
+    "fmsamd_stream_enter": [P, P, I, P, P, P, P, I, I, P],
+    "fmsamd_soft_cap_f32": [P, L, F, P],
     "fmsamd_probe_read": [P, L, I, I, P, P],
     "fmsamd_probe_mfma": [I, I, I, P, P, P],
 }
@@ -132,6 +136,8 @@ def load(verbose: bool = True) -> ctypes.CDLL:
         lib.fmsamd_latent_attn_mfma_fits.argtypes = [I, I]
         lib.fmsamd_ssd_chunk_workspace.restype = c_long
         lib.fmsamd_ssd_chunk_workspace.argtypes = [I, I, I]
+        lib.fmsamd_linear_recurrence_workspace.restype = c_long
+        lib.fmsamd_linear_recurrence_workspace.argtypes = [I, I, I, I]
         lib.fmsamd_talking_attn_workspace.restype = c_long
         lib.fmsamd_talking_attn_workspace.argtypes = [I, I, I, I]
         lib.fmsamd_moe_max_tiles.restype = c_int

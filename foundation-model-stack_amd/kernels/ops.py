@@ -130,19 +130,63 @@ def stream_rows(resid: torch.Tensor, branch: Optional[torch.Tensor], branch_scal
                                     resid.shape[0], resid.shape[1], _stream()))
 
 
-def gated_act(gu: torch.Tensor, bias: Optional[torch.Tensor], activation: str) -> torch.Tensor:
-    """[T, 2*hidden] (gate first) -> act(gate + b) * (up + b) [T, hidden]."""
+class GateClamp(ctypes.Structure):
+    """The clamped gated unit of a gated product: g sigmoid(alpha g) (u + shift) with g = min(gate, limit) and
+    u = clamp(up, -limit, limit), in the place of act(gate) * up."""
+
+    _fields_ = [("limit", ctypes.c_float), ("alpha", ctypes.c_float), ("shift", ctypes.c_float)]
+
+
+def _clamp(clamp: Optional[GateClamp]):
+    return None if clamp is None else ctypes.byref(clamp)
+
+
+def _rows_out(out: Optional[torch.Tensor], rows: int, cols: int, dtype: torch.dtype, device) -> torch.Tensor:
+    """`out` checked to be rows [rows, cols] of any stride, or a new tensor."""
+    if out is None:
+        return torch.empty(rows, cols, dtype=dtype, device=device)
+    _need_cuda(out)
+    _rows2d("out", out)
+    if out.dtype != dtype or tuple(out.shape) != (rows, cols):
+        raise ValueError(f"out is [{rows}, {cols}] of {dtype}, got {tuple(out.shape)} of {out.dtype}")
+    return out
+
+
+def gated_act(gu: torch.Tensor, bias: Optional[torch.Tensor], activation: str, clamp: Optional[GateClamp] = None,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """[T, 2*hidden] (gate first) -> act(gate + b) * (up + b) [T, hidden], or the clamped unit of the two sums.  out: rows of
+    any stride to write into (default: a new tensor)."""
     _need_cuda(gu, bias)
     if gu.dim() != 2 or not gu.is_contiguous() or gu.shape[1] % 2:
         raise ValueError("gated_act takes a contiguous [T, 2*hidden] tensor")
     T, hidden = gu.shape[0], gu.shape[1] // 2
     if bias is not None and (bias.shape != (2 * hidden,) or not bias.is_contiguous()):
         raise ValueError(f"bias must be a contiguous [{2 * hidden}] tensor")
-    out = torch.empty(T, hidden, dtype=gu.dtype, device=gu.device)
+    out = _rows_out(out, T, hidden, gu.dtype, gu.device)
     for t0 in range(0, T, 65535):
         n = min(65535, T - t0)
         check(load().fmsamd_gated_act(gu[t0:].data_ptr(), _ptr(bias), _code(bias.dtype) if bias is not None else 0,
-                                      out[t0:].data_ptr(), _code(gu.dtype), n, hidden, ACTIVATIONS[activation], _stream()))
+                                      out[t0:].data_ptr(), _code(gu.dtype), out.stride(0), n, hidden, ACTIVATIONS[activation],
+                                      _clamp(clamp), _stream()))
+    return out
+
+
+def stream_enter(resid: torch.Tensor, branch: Optional[torch.Tensor] = None, branch_scale: Optional[torch.Tensor] = None,
+                 base: Optional[torch.Tensor] = None, shift: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A new stream, resid + branch (* branch_scale) + base + shift in float32: base another stream, shift a vector
+    (float32 [width]); resid stays as it is."""
+    _need_cuda(resid, branch, branch_scale, base, shift)
+    if resid.dtype != torch.float32 or resid.dim() != 2 or not resid.is_contiguous():
+        raise ValueError("the residual stream must be a contiguous float32 [T, width] tensor")
+    _check_branch_scale(branch_scale, resid)
+    _check_branch_scale(shift, resid)
+    if branch is not None and (branch.shape != resid.shape or not branch.is_contiguous()):
+        raise ValueError(f"the branch is contiguous {tuple(resid.shape)}")
+    if base is not None and (base.shape != resid.shape or not base.is_contiguous() or base.dtype != torch.float32):
+        raise ValueError(f"base is contiguous float32 {tuple(resid.shape)}")
+    out = torch.empty_like(resid)
+    check(load().fmsamd_stream_enter(resid.data_ptr(), _ptr(branch), _code(branch.dtype) if branch is not None else F32, _ptr(branch_scale),
+                                     _ptr(base), _ptr(shift), out.data_ptr(), resid.shape[0], resid.shape[1], _stream()))
     return out
 
 
@@ -648,9 +692,10 @@ def linear_into_stream(
 
 def gated_linear(
     x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], activation: str, allow_library: bool = True,
-    row_norm: Optional[RowNorm] = None,
+    row_norm: Optional[RowNorm] = None, clamp: Optional[GateClamp] = None, out: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
-    """act(x Wg^T + bg) * (x Wu^T + bu) for weight = [Wg; Wu] stacked [2*hidden, K] -> [M, hidden]."""
+    """act(x Wg^T + bg) * (x Wu^T + bu), or the clamped unit of the two sums, for weight = [Wg; Wu] stacked [2*hidden, K]
+    -> [M, hidden] (into `out`, rows of any stride)."""
     M = x.shape[0]
     if weight.shape[0] % 2:
         raise ValueError("the stacked gate/up weight needs an even number of rows")
@@ -664,17 +709,17 @@ def gated_linear(
             raise ValueError("weight must be contiguous [2*hidden, K] with K the width of x")
         if bias is not None and (bias.shape != (2 * hidden,) or not bias.is_contiguous()):
             raise ValueError(f"bias must be a contiguous [{2 * hidden}] tensor")
-        out = torch.empty(M, hidden, dtype=torch.bfloat16, device=x.device)
+        out = _rows_out(out, M, hidden, torch.bfloat16, x.device)
         ws, ws_bytes = _skinny_workspace(M, 2 * hidden, K, x.device)
         check(load().fmsamd_gemm_skinny_gated_bf16(x.data_ptr(), x.stride(0), weight.data_ptr(), _ptr(bias),
                                                    _code(bias.dtype) if bias is not None else 0, out.data_ptr(), BF16,
-                                                   out.stride(0), M, hidden, K, ACTIVATIONS[activation],
+                                                   out.stride(0), M, hidden, K, ACTIVATIONS[activation], _clamp(clamp),
                                                    _row_scale(row_norm, M), _ptr(ws), ws_bytes, _stream()))
         return out
     if row_norm is not None:
         raise ValueError(f"a deferred row norm goes with the bfloat16 product of at most {SKINNY_FAST_ROWS} rows")
     gu = linear(x, weight, None, allow_library=allow_library)
-    return gated_act(gu, bias, activation)
+    return gated_act(gu, bias, activation, clamp, out)
 
 
 # --------------------------------------------------------------------------
@@ -1402,6 +1447,15 @@ def scale_(x: torch.Tensor, s: float) -> torch.Tensor:
     return x
 
 
+def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """x = cap * tanh(x / cap) in place (contiguous float32)."""
+    _need_cuda(x)
+    if x.dtype != torch.float32 or not x.is_contiguous() or cap <= 0:
+        raise ValueError("soft_cap_ takes a contiguous float32 tensor and a positive cap")
+    check(load().fmsamd_soft_cap_f32(x.data_ptr(), x.numel(), float(cap), _stream()))
+    return x
+
+
 # --------------------------------------------------------------------------
 # the gated delta rule
 # --------------------------------------------------------------------------
@@ -1487,9 +1541,9 @@ def delta_rule(qkv: torch.Tensor, beta: torch.Tensor, decay: torch.Tensor, kq: t
     return out
 
 
-def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, activation: str, heads: int, vdim: int,
+def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], eps: float, activation: str, heads: int, vdim: int,
                     out_dtype: torch.dtype, seq_of_token: torch.Tensor, scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """o float32 [T, heads*vdim]: every head divided by its root mean square, times weight [vdim], times act(gate)
+    """o float32 [T, heads*vdim]: every head divided by its root mean square, times weight [vdim] (None: no weight), times act(gate)
     (float32 logits [T, heads*vdim], rows of any stride), times scale -> out_dtype (into `out`, rows of any stride)."""
     _need_cuda(o, gate, weight, seq_of_token, out)
     _rows2d("gate", gate)
@@ -1499,14 +1553,14 @@ def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, e
         raise ValueError(f"o is contiguous float32 [T, {heads * vdim}]")
     if gate.dtype != torch.float32 or tuple(gate.shape) != (T, heads * vdim):
         raise ValueError(f"the gate is float32 [{T}, {heads * vdim}]")
-    if tuple(weight.shape) != (vdim,) or not weight.is_contiguous():
+    if weight is not None and (tuple(weight.shape) != (vdim,) or not weight.is_contiguous()):
         raise ValueError(f"the norm weight is a contiguous [{vdim}] tensor")
     if out is None:
         out = torch.empty(T, heads * vdim, dtype=out_dtype, device=o.device)
     _rows2d("out", out)
     if out.dtype != out_dtype or tuple(out.shape) != (T, heads * vdim):
         raise ValueError(f"out is [{T}, {heads * vdim}] of {out_dtype}")
-    check(load().fmsamd_gated_head_norm(o.data_ptr(), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight.dtype), float(eps),
+    check(load().fmsamd_gated_head_norm(o.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(weight), _code(weight.dtype) if weight is not None else F32, float(eps),
                                         ACTIVATIONS[activation], float(scale), out.data_ptr(), _code(out_dtype), out.stride(0),
                                         seq_of_token.data_ptr(), T, heads, vdim, _stream()))
     return out
@@ -1632,6 +1686,95 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, par
                                          out.data_ptr(), _code(out_dtype), seq_of_token.data_ptr(), T, cols, _ptr(conv_x),
                                          conv_x.stride(0) if conv_x is not None else 0, channels, int(taps), _ptr(conv_state), _ptr(slot_ids),
                                          _stream()))
+    return out
+
+
+# --------------------------------------------------------------------------
+# linear attention with a decay
+# --------------------------------------------------------------------------
+LINEAR_MAX_DIM = 256
+LINEAR_CHUNK_FROM = 32  # tokens a sequence: from there on a step runs the recurrence in chunks
+
+
+class _LinearRecurrenceArg(ctypes.Structure):
+    _P, _I, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
+    _fields_ = [("proj", _P), ("ld", ctypes.c_long), ("col_q", _I), ("col_k", _I), ("col_v", _I), ("col_g", _I), ("col_low", _I),
+                ("heads", _I), ("dim", _I), ("vdim", _I), ("rank", _I), ("log_decay", _P), ("up_t", _P), ("up_bias", _P), ("inv_tau", _F),
+                ("rot_dim", _I), ("max_pos", _I), ("cos_t", _P), ("sin_t", _P), ("positions", _P), ("q_scale", _F), ("state", _P),
+                ("seq_starts", _P), ("seq_of_token", _P), ("slot_ids", _P), ("n_seqs", _I), ("n_tokens", _I), ("norm_w", _P), ("eps", _F),
+                ("out_scale", _F), ("act", _I), ("out", _P), ("out_dtype", _I), ("ldo", ctypes.c_long)]
+
+
+def linear_recurrence(proj: torch.Tensor, cols, heads: int, dim: int, vdim: int, state: torch.Tensor, seq_starts: torch.Tensor,
+                      seq_of_token: torch.Tensor, slot_ids: torch.Tensor, n_seqs: int, longest: int, out_dtype: torch.dtype, *,
+                      log_decay: Optional[torch.Tensor] = None, up_t: Optional[torch.Tensor] = None, up_bias: Optional[torch.Tensor] = None,
+                      inv_tau: float = 1.0, rotation=None, positions: Optional[torch.Tensor] = None, q_scale: float = 1.0,
+                      norm_weight: Optional[torch.Tensor] = None, eps: float = 1e-6, activation: str = "silu", scale: float = 1.0,
+                      out: Optional[torch.Tensor] = None, chunked: Optional[bool] = None) -> torch.Tensor:
+    """S <- S diag(a) + v k^T, o = S q per head, over the tokens of every sequence of the step, from and into state
+    [slots, heads, vdim, dim] (float32); every head's o divided by its root mean square, times norm_weight (float32 [vdim] or
+    None), times act(gate), times scale -> [T, heads*vdim] in out_dtype (into `out`, rows of any stride; padding rows: zeros).
+
+    proj: float32 rows; cols = (q, k, v, gate, low): where q and k (heads*dim columns), v and the gate's logits (heads*vdim)
+    and the numbers of a projected decay start.  Decays: exp(log_decay[head]) (float32 [heads]), or sigmoid(z)^inv_tau per head
+    and key channel with z = low @ up_t + up_bias (float32 [rank, heads*dim] and [heads*dim]).  rotation: (cos, sin, size),
+    tables for neighbouring pairs of the first `size` channels of q and k, or None.  q is multiplied by q_scale.  Sequence b
+    owns the token rows seq_starts[b] .. seq_starts[b + 1] and the state of slot_ids[b]; longest: the most tokens a sequence
+    brings.  chunked: in chunks of 64 tokens as matrix products (default: from LINEAR_CHUNK_FROM tokens a sequence on), else
+    token by token; the two differ by rounding."""
+    _need_cuda(proj, state, seq_starts, seq_of_token, slot_ids, log_decay, up_t, up_bias, norm_weight)
+    _rows2d("proj", proj)
+    for name, t in (("seq_starts", seq_starts), ("seq_of_token", seq_of_token), ("slot_ids", slot_ids)):
+        _need_i32(name, t)
+    T = proj.shape[0]
+    HD, HV = heads * dim, heads * vdim
+    if proj.dtype != torch.float32:
+        raise TypeError("the recurrence reads float32 rows")
+    if not 0 < dim <= LINEAR_MAX_DIM:
+        raise ValueError(f"the recurrence takes at most {LINEAR_MAX_DIM} key channels a head, not {dim}")
+    if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, vdim, dim) or not state.is_contiguous():
+        raise ValueError(f"the state is contiguous float32 [slots, {heads}, {vdim}, {dim}]")
+    if (log_decay is None) == (up_t is None):
+        raise ValueError("decays are given either per head or by a projection")
+    rank = 0
+    if up_t is not None:
+        rank = up_t.shape[0]
+        if up_t.dtype != torch.float32 or tuple(up_t.shape) != (rank, HD) or not up_t.is_contiguous():
+            raise ValueError(f"the decays' projection is contiguous float32 [rank, {HD}]")
+        if up_bias is None or up_bias.dtype != torch.float32 or tuple(up_bias.shape) != (HD,) or not up_bias.is_contiguous():
+            raise ValueError(f"the decays' bias is contiguous float32 [{HD}]")
+    elif log_decay.dtype != torch.float32 or tuple(log_decay.shape) != (heads,) or not log_decay.is_contiguous():
+        raise ValueError(f"the heads' log decays are contiguous float32 [{heads}]")
+    for col, n in zip(cols, (HD, HD, HV, HV, rank)):
+        if n and not 0 <= col <= proj.shape[1] - n:
+            raise ValueError(f"rows of {proj.shape[1]} columns do not hold {n} from column {col} on")
+    if norm_weight is not None and (norm_weight.dtype != torch.float32 or tuple(norm_weight.shape) != (vdim,) or not norm_weight.is_contiguous()):
+        raise ValueError(f"the norm weight is contiguous float32 [{vdim}]")
+    if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs or seq_of_token.numel() < T:
+        raise ValueError("the step's index arrays are shorter than its sequences or tokens")
+    cos = sin = None
+    rot = max_pos = 0
+    if rotation is not None:
+        cos, sin, rot = rotation
+        _need_cuda(cos, sin, positions)
+        _need_i32("positions", positions)
+        max_pos = _check_tables(cos, sin, rot)
+        if positions.numel() < T:
+            raise ValueError("a position per token is needed")
+    out = _rows_out(out, T, HV, out_dtype, proj.device)
+    arg = _LinearRecurrenceArg(
+        proj.data_ptr(), proj.stride(0), cols[0], cols[1], cols[2], cols[3], cols[4] if rank else 0, heads, dim, vdim, rank, _ptr(log_decay),
+        _ptr(up_t), _ptr(up_bias), float(inv_tau), rot, max_pos, _ptr(cos), _ptr(sin), _ptr(positions) if rot else None, float(q_scale),
+        state.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(), int(n_seqs), T, _ptr(norm_weight), float(eps),
+        float(scale), ACTIVATIONS[activation], out.data_ptr(), _code(out_dtype), out.stride(0))
+    lib = load()
+    if longest >= LINEAR_CHUNK_FROM if chunked is None else chunked:
+        ws_bytes = lib.fmsamd_linear_recurrence_workspace(T, int(n_seqs), heads, dim)
+        ws = torch.empty(ws_bytes // 4, dtype=torch.float32, device=proj.device)
+        y = torch.empty(T, HV, dtype=torch.float32, device=proj.device)
+        check(lib.fmsamd_linear_recurrence_chunked(ctypes.byref(arg), y.data_ptr(), int(longest), ws.data_ptr(), ws_bytes, _stream()))
+        return gated_head_norm(y, proj[:, cols[3] : cols[3] + HV], norm_weight, eps, activation, heads, vdim, out_dtype, seq_of_token, scale, out)
+    check(lib.fmsamd_linear_recurrence_walk(ctypes.byref(arg), _stream()))
     return out
 
 

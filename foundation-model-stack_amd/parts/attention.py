@@ -162,6 +162,10 @@ class MultiHeadAttention(Mixer):
             pieces += (("in_proj.gate", self.n_gate),)
         return {"in_proj.qkv_fused": pieces}
 
+    @property
+    def writes_padding_rows(self) -> bool:
+        return not self.talking_heads
+
     def output_projection(self) -> Linear:
         return self.dense
 

@@ -119,6 +119,21 @@ class Mixer(Part):
     def forward(self, x: torch.Tensor, batch, cache) -> torch.Tensor:
         raise NotImplementedError
 
+    # optional, for callers that run the part beside another and project both at once --------
+    # True if rows of padding (sequence -1) of a decode step's output are written too, with any numbers
+    writes_padding_rows = False
+
+    def output_projections(self) -> List["Part"]:
+        """The linear layers at the mixer's end, in the order in which forward_branch lays their inputs next to each other
+        when it is given rows to write them into (out=)."""
+        return [self.output_projection()]
+
+    def output_projection(self) -> "Part":
+        raise NotImplementedError(f"{type(self).__name__} does not run beside another part")
+
+    def leaves_output_to_caller(self) -> None:
+        """Said once, before finalize, by a caller that will always pass out= and run the output projections itself."""
+
     # optional, for kernels that fuse across the boundary of the part --------
     def accepts_normed_rows(self, rows: int, dtype, batch) -> bool:
         """True if forward_branch takes a NormedRows for a step of this shape."""

@@ -16,6 +16,7 @@ import torch
 from ..cache import StateNeed
 from ..kernels import ops
 from .base import BranchOutput, NormedRows, Part, register_part
+from .linear import JointProjection
 
 
 class ResidualStream:
@@ -72,6 +73,12 @@ class ResidualStream:
         if self.pending_norm is not None:
             raise NotImplementedError("a branch with a norm of its own is added by the norm that reads the stream next")
         ops.stream_rows(self.resid, self.pending, self.pending_scale, out)
+
+    def advance(self, base: Optional[torch.Tensor] = None, shift: Optional[torch.Tensor] = None) -> None:
+        """A new stream in the place of this one: what is pending is added, and another stream `base` and a vector `shift`."""
+        if self.pending_norm is not None:
+            raise NotImplementedError("a branch with a norm of its own is added by the norm that reads the stream next")
+        self.replace(ops.stream_enter(self.resid, self.pending, self.pending_scale, base, shift))
 
     def replace(self, resid: torch.Tensor) -> None:
         """Another stream in the place of this one; what was pending goes with the old one."""
@@ -227,6 +234,47 @@ class PostNormBlock(Part):
             stream.add_branch(self.feed_forward.forward(stream.rows(act_dtype)), post_norm=self.norm2)
 
 
+class ParallelBlock(Part):
+    """A block with one norm whose branches run side by side: with h = norm1(x), x + (mixer(h) + ff(h)).  Both branches end in a
+    projection back to the width; the two run as one product over their inputs laid next to each other, so that the sum of
+    the branches costs no kernel and no rounding of its own.  The feed-forward may be absent (None)."""
+
+    fuses_next_norm = True
+    norm_arguments = ("norm1",)
+
+    def __init__(self, mixer: Part, feed_forward: Optional[Part], norm1: Part, names=("norm1", "mix", "mlp")):
+        super().__init__()
+        self.norm1 = self.add_child(names[0], norm1)
+        self.mixer = self.add_child(names[1], mixer)
+        self.feed_forward = feed_forward
+        if feed_forward is not None:
+            self.add_child(names[2], feed_forward)
+        self.joint = JointProjection([*mixer.output_projections(), *(feed_forward.output_projections() if feed_forward is not None else [])])
+        mixer.leaves_output_to_caller()
+
+    def first_norm(self) -> Part:
+        return self.norm1
+
+    def finalize(self, device, dtype) -> None:
+        self.joint.join()
+
+    def forward(self, stream: ResidualStream, batch, cache, act_dtype: torch.dtype, next_norm: Optional[Part] = None) -> None:
+        T, ff = stream.resid.shape[0], self.feed_forward
+        deferred = self.mixer.accepts_normed_rows(T, act_dtype, batch) and (ff is None or ff.accepts_normed_rows(T, act_dtype))
+        h = stream.normed(self.norm1, act_dtype, deferred)
+        both = self.joint.input_rows(T, act_dtype, h_device(h), batch, self.mixer.writes_padding_rows)
+        n = self.joint.in_features - (ff.output_projections()[0].in_features if ff is not None else 0)
+        self.mixer.forward_branch(h, batch, cache, out=both[:, :n])
+        if ff is not None:
+            ff.forward_branch(h, out=both[:, n:])
+        stream.add_branch(BranchOutput(both, self.joint), next_norm)
+
+
+def h_device(h) -> torch.device:
+    return (h.rows if isinstance(h, NormedRows) else h).device
+
+
 register_part("block", "pre_norm", PreNormBlock)
+register_part("block", "parallel", ParallelBlock)
 register_part("block", "post_norm", PostNormBlock)
 register_part("block", "sandwich_norm", SandwichNormBlock)

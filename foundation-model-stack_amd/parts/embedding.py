@@ -25,14 +25,19 @@ class TokenEmbedding(Part):
 
 
 class LinearHead(Part):
-    def __init__(self, width: int, vocab: int, scale: float = 1.0):
+    def __init__(self, width: int, vocab: int, scale: float = 1.0, soft_cap: float = 0.0):
+        """scale: a constant factor on every logit.  soft_cap: logits become soft_cap * tanh(logit / soft_cap) (0: no cap)."""
         super().__init__()
-        self.vocab, self.width, self.scale = vocab, width, float(scale)  # scale: a constant factor on every logit
+        self.vocab, self.width, self.scale, self.soft_cap = vocab, width, float(scale), float(soft_cap)
+        if self.soft_cap < 0:
+            raise ValueError(f"soft_cap {soft_cap} must be zero (none) or positive")
         self.declare("weight", (vocab, width))
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         logits = ops.linear(x, self.w["weight"], None, out_dtype=torch.float32)
-        return logits if self.scale == 1.0 else ops.scale_(logits, self.scale)
+        if self.scale != 1.0:
+            logits = ops.scale_(logits, self.scale)
+        return ops.soft_cap_(logits, self.soft_cap) if self.soft_cap else logits
 
 
 register_part("embedding", "table", TokenEmbedding)

@@ -7,6 +7,8 @@ one fused projection whose first half is the gate and second half the "up" path
 
 from __future__ import annotations
 
+from typing import List, Optional
+
 import torch
 
 from ..kernels import ops
@@ -15,12 +17,18 @@ from .linear import Linear
 
 
 class GatedLinearUnit(FeedForward):
-    def __init__(self, width: int, hidden_dim: int, activation: str = "swish", use_bias: bool = False):
+    def __init__(self, width: int, hidden_dim: int, activation: str = "swish", use_bias: bool = False,
+                 limit: Optional[float] = None, alpha: float = 1.0, shift: float = 0.0):
+        """limit: the clamped unit instead of act(gate) * up: g sigmoid(alpha g) (u + shift) with g = min(gate, limit) and
+        u = clamp(up, -limit, limit)."""
         super().__init__()
         activation = str(activation).lower()  # the reference looks names up without regard to case
         if activation not in ops.ACTIVATIONS:
             raise ValueError(f"activation {activation!r} is not one of {sorted(ops.ACTIVATIONS)}")
         self.width, self.hidden_dim, self.activation = width, int(hidden_dim), activation
+        if limit is not None and limit <= 0:
+            raise ValueError(f"a limit of {limit} must be positive")
+        self.clamp = ops.GateClamp(float(limit), float(alpha), float(shift)) if limit is not None else None
         self.wg1 = self.add_child("wg1_fused", Linear(width, 2 * self.hidden_dim, use_bias))
         self.w2 = self.add_child("w2", Linear(self.hidden_dim, width, use_bias))
 
@@ -34,9 +42,13 @@ class GatedLinearUnit(FeedForward):
     def accepts_normed_rows(self, rows: int, dtype) -> bool:
         return self.wg1.streams(rows, dtype)
 
-    def forward_branch(self, x) -> BranchOutput:
+    def output_projections(self) -> List[Linear]:
+        return [self.w2]
+
+    def forward_branch(self, x, out: Optional[torch.Tensor] = None) -> BranchOutput:
+        """out (rows of any stride): where the input of the last projection is written, for a caller that runs that itself."""
         x, row_norm = split_normed(x)
-        hidden = ops.gated_linear(x, self.wg1.w["weight"], self.wg1.w.get("bias"), self.activation, row_norm=row_norm)
+        hidden = ops.gated_linear(x, self.wg1.w["weight"], self.wg1.w.get("bias"), self.activation, row_norm=row_norm, clamp=self.clamp, out=out)
         return BranchOutput(hidden, self.w2)
 
 

@@ -22,7 +22,7 @@ import torch
 
 from ..cache import KVNeed
 from ..kernels import ops
-from .base import BranchOutput, Mixer, register_part
+from .base import BranchOutput, Mixer, register_part, split_normed
 from .linear import Linear
 from .position import PositionEncoding
 
@@ -111,10 +111,21 @@ class LatentAttention(Mixer):
             if tables is None or tables[2] != self.rot_dim:
                 raise ValueError("latent attention rotates by a table of exactly its rotated size")
 
+    writes_padding_rows = True
+
+    def output_projection(self) -> Linear:
+        return self.o
+
+    def accepts_normed_rows(self, rows: int, dtype, batch) -> bool:
+        return self.down.streams(rows, dtype)
+
     def forward(self, x: torch.Tensor, batch, cache) -> torch.Tensor:
         return self.forward_branch(x, batch, cache).value()
 
-    def forward_branch(self, x: torch.Tensor, batch, cache) -> BranchOutput:
+    def forward_branch(self, x, batch, cache, out: Optional[torch.Tensor] = None) -> BranchOutput:
+        """out (rows [T, heads * vdim] of any stride): where the input of the output projection is written, for a caller that
+        runs that itself."""
+        x, row_norm = split_normed(x)
         H, D, P, R, V = self.nheads, self.dim, self.rot_dim, self.kv_rank, self.vdim
         T = x.shape[0]
         table = batch.block_tables[cache.group]
@@ -122,7 +133,7 @@ class LatentAttention(Mixer):
         if P:
             cos, sin, _ = self.position_encoder.tables_for_step(batch)
         # norms, gates and everything that enters the cache are formed from the float32 sums of this product
-        down = self.down.forward(x, out_dtype=torch.float32)
+        down = self.down.forward(x, out_dtype=torch.float32, row_norm=row_norm)
         if cache.owns:
             if not self.owns_kv:
                 raise RuntimeError("this layer has no down-projection for keys and values: it must read another layer's cache")
@@ -140,11 +151,11 @@ class LatentAttention(Mixer):
         mixed_latent = ops.latent_attention(qa, batch.positions, batch.seq_of_token, table, cache.keys, self._sink, H, R, P,
                                             self.scale, self.window, decode=batch.is_decode, max_context=batch.context_bound,
                                             vt_cache=cache.values)
-        mixed = torch.empty(T, H * V, dtype=x.dtype, device=x.device)
+        mixed = torch.empty(T, H * V, dtype=x.dtype, device=x.device) if out is None else out
         gate = down[:, self.gate_col : self.gate_col + self.gate_cols] if self.has_gate else None
         if self.gate_cols == H * V:  # a gate per output element: behind the product that leaves the latent space
             ops.headwise_linear(mixed_latent, R, self._uv, mixed, V)
-            mixed = ops.gate_mul(mixed, gate, "sigmoid")
+            mixed = ops.gate_mul(mixed, gate, "sigmoid", out=out)
         else:
             ops.headwise_linear(mixed_latent, R, self._uv, mixed, V, gate=gate)
         return BranchOutput(mixed, self.o)

@@ -10,23 +10,25 @@ carry the side's name.
 
 from __future__ import annotations
 
+from typing import Optional
+
 import torch
 
 from ..cache import StateNeed
-from .base import BranchOutput, Mixer, make_part, register_part
-from .linear import Linear
+from .base import BranchOutput, Mixer, make_part, register_part, split_normed
+from .linear import JointProjection
 
 
 class ParallelMixers(Mixer):
     def __init__(self, width: int, left: dict, right: dict, left_scale: float = 1.0, right_scale: float = 1.0, position_encoder=None):
         """left, right: {"kind": a registered mixer, "args": its arguments}.  The position encoding goes to the sides that
-        say `"positional": True`."""
+        say `"positional": True`; with encodings of their own it is a dictionary from a side's name to its encoding."""
         super().__init__()
         self.width = width
         self.scales = (float(left_scale), float(right_scale))
         self.sides = []
         for name, spec in (("left", left), ("right", right)):
-            pos = position_encoder if spec.get("positional") else None
+            pos = position_encoder.get(name) if isinstance(position_encoder, dict) else (position_encoder if spec.get("positional") else None)
             side = make_part("mixer", spec["kind"], width=width, position_encoder=pos, **spec.get("args", {}))
             if not hasattr(side, "forward_branch"):
                 raise TypeError(f"mixer {spec['kind']!r} cannot run beside another: it has no forward_branch")
@@ -34,8 +36,11 @@ class ParallelMixers(Mixer):
             self.sides.append(self.add_child(name, side))
         if sum(side.kv_need() is not None for side in self.sides) > 1:
             raise ValueError("at most one of two parallel mixers can keep keys and values in the cache")
-        self._joint: Linear = None
-        self._widths = None
+        outs = self.output_projections()
+        if any(o.has_bias for o in outs):
+            raise NotImplementedError("parallel mixers join output projections without biases")
+        self._joint: Optional[JointProjection] = JointProjection(outs)
+        self._widths = [o.in_features for o in outs]
 
     def kv_need(self):
         for side in self.sides:
@@ -55,6 +60,10 @@ class ParallelMixers(Mixer):
     def graph_safe(self) -> bool:
         return all(getattr(side, "graph_safe", True) for side in self.sides)
 
+    @property
+    def writes_padding_rows(self) -> bool:
+        return all(side.writes_padding_rows for side in self.sides)
+
     def check_step(self, max_position: int) -> None:
         for side in self.sides:
             side.check_step(max_position)
@@ -62,32 +71,33 @@ class ParallelMixers(Mixer):
     def prefill_qblock(self, n_tokens: int, dtype) -> int:
         return max(side.prefill_qblock(n_tokens, dtype) for side in self.sides)
 
+    def output_projections(self) -> list:
+        return [side.output_projection() for side in self.sides]
+
+    def leaves_output_to_caller(self) -> None:
+        self._joint = None  # the caller's joint projection holds the sides' weights
+
     def finalize(self, device, dtype) -> None:
-        # the sides' output projections as one weight [width, K_left + K_right]; the sides' own tensors become views of it
-        outs = [side.output_projection() for side in self.sides]
-        if any(o.has_bias for o in outs):
-            raise NotImplementedError("parallel mixers join output projections without biases")
-        self._widths = [o.in_features for o in outs]
-        joint = torch.cat([o.w["weight"] for o in outs], dim=1).contiguous()
-        self._joint = Linear(sum(self._widths), self.width)
-        self._joint.w["weight"] = joint
-        at = 0
-        for o in outs:
-            o.w["weight"] = joint[:, at : at + o.in_features]
-            at += o.in_features
+        if self._joint is not None:
+            self._joint.join()
+
+    def accepts_normed_rows(self, rows: int, dtype, batch) -> bool:
+        return all(side.accepts_normed_rows(rows, dtype, batch) for side in self.sides)
 
     def forward(self, x: torch.Tensor, batch, cache) -> torch.Tensor:
         return self.forward_branch(x, batch, cache).value()
 
-    def forward_branch(self, x: torch.Tensor, batch, cache) -> BranchOutput:
-        both = torch.empty(x.shape[0], sum(self._widths), dtype=x.dtype, device=x.device)
-        if batch.is_decode:
-            both.zero_()  # a decode step may hold padding rows, which nobody writes and the joint product reads
+    def forward_branch(self, x, batch, cache, out: Optional[torch.Tensor] = None) -> BranchOutput:
+        """out (rows of any stride): where the inputs of the sides' output projections are written, for a caller that runs
+        those itself."""
+        if out is None:
+            rows = split_normed(x)[0]
+            out = self._joint.input_rows(rows.shape[0], rows.dtype, rows.device, batch, self.writes_padding_rows)
         at = 0
         for side, scale, k in zip(self.sides, self.scales, self._widths):
-            side.forward_branch(x, batch, cache, out=both[:, at : at + k], out_scale=scale)
+            side.forward_branch(x, batch, cache, out=out[:, at : at + k], out_scale=scale)
             at += k
-        return BranchOutput(both, self._joint)
+        return BranchOutput(out, self._joint)
 
 
 register_part("mixer", "parallel", ParallelMixers)

@@ -10,7 +10,7 @@ twice or let an entry read the cache of an earlier entry.
 from __future__ import annotations
 
 import dataclasses
-from typing import Dict, List, Optional, Tuple
+from typing import Dict, List, Optional, Tuple, Union
 
 
 @dataclasses.dataclass
@@ -25,7 +25,8 @@ class LayerSpec:
     feed_forward: Optional[PartSpec]  # None: the layer has none (its block must take that)
     norm: Optional[PartSpec] = None  # the spec of every norm the block asks for ...
     block: PartSpec = dataclasses.field(default_factory=lambda: PartSpec("pre_norm"))
-    position: Optional[str] = None  # key into ModelSpec.positions, handed to the mixer
+    # key into ModelSpec.positions, handed to the mixer; for a mixer of several sides a key for each (side -> key)
+    position: Union[None, str, Dict[str, str]] = None
     norms: Optional[List[PartSpec]] = None  # ... or one spec for each, in the order of the block's `norm_arguments`
 
 
