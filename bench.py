@@ -30,6 +30,7 @@ distance, and over a latent; layer norms on both sides of every branch) beside L
 gated feed-forward; every attention call is priced by the keys its own mask shows.
 
     python bench.py --zimorax [--layers N]
+    python bench.py --kapuvik [--layers N]
 
 is the same comparison for Zimorax (the Mamba-2 recurrence, a gated delta rule, windowed attention whose scores are mixed
 over the heads, looped layers, a plain feed-forward) beside Defapel, the closest model of the library (windowed attention
@@ -85,6 +86,8 @@ def main() -> int:
                     help="another workload: Zodolorn beside Llama at equal layer sizes, with every kernel class's distance from its roofline")
     ap.add_argument("--basopel", action="store_true", help="another workload: Basopel beside Llama at equal layer sizes, likewise")
     ap.add_argument("--zimorax", action="store_true", help="another workload: Zimorax beside Defapel at equal layer sizes, likewise")
+    ap.add_argument("--kapuvik", action="store_true",
+                    help="another workload: Kapuvik beside Defapel (and Zodolorn, for its latent attention) at equal layer sizes, likewise")
     ap.add_argument("--defapel", action="store_true", help="another workload: Defapel beside Llama at equal layer sizes, likewise")
     ap.add_argument("--sidalorn", action="store_true", help="another workload: Sidalorn beside Zodolorn at equal layer sizes, likewise")
     args = ap.parse_args()
@@ -98,7 +101,7 @@ def main() -> int:
         print(f"bench.py measures one GPU: this library runs on a single MI355X, --gpus {args.gpus} is not supported")
         return 2
 
-    for design in ("zodolorn", "defapel", "sidalorn", "basopel", "zimorax"):
+    for design in ("zodolorn", "defapel", "sidalorn", "basopel", "zimorax", "kapuvik"):
         if getattr(args, design):
             return design_comparison(args, design)
 
@@ -351,6 +354,15 @@ ZIMORAX_SIZES = [
 ]
 
 
+# (name, width, layer pattern (p: attention beside retention, g: gated linear attention, l: latent attention), heads, kv heads,
+#  head size, feed-forward, heads of the recurrences, their key channels, their value channels, [dim, rot, vdim, kv_rank] of the
+#  latent attention; of the models beside it: window, experts, top, expert ff, q_rank), vocabulary
+KAPUVIK_SIZES = [
+    ("w2048", 2048, "pglg", 16, 4, 128, 5632, 16, 128, 128, (128, 64, 128, 512), (8192, 32, 4, 1024, 768), 32768),
+    ("w4096", 4096, "pglg", 32, 8, 128, 8192, 32, 128, 128, (128, 64, 128, 512), (8192, 64, 6, 1536, 1536), 32768),
+]
+
+
 # (name, width, layer pattern, heads, [dim, vdim, kv_rank], recurrent channels, blocks, dense ff, experts, identity experts, top,
 #  expert ff, shared ff, groups, groups kept, norm groups, vocabulary)
 SIDALORN_SIZES = [
@@ -436,6 +448,11 @@ def design_comparison(args, design) -> int:
             channels = H * P + 2 * a[16] * N
             state_bytes = 2 * n_seqs * (st.numel() // st.shape[0]) * 4 + (n_seqs * (conv.numel() // conv.shape[0]) * 4 if conv is not None else 0)
             return state_bytes + a[0].shape[0] * 4 * channels + nbytes(a[3], a[4], out), 5.0 * n_seqs * H * P * N * mfma_flops / PEAK_FLOPS["fp32"]
+        if name == "linear_recurrence":  # like ssd; the projection's columns are read where they lie
+            _, cols, H, D, V, st = a[:6]
+            T, n_seqs = a[0].shape[0], a[9]
+            vector_flops = 5.0 * T * H * D * V
+            return T * 4 * a[0].shape[1] + nbytes(kw.get("up_t"), out) + 2 * n_seqs * (st.numel() // st.shape[0]) * 4, vector_flops * mfma_flops / PEAK_FLOPS["fp32"]
         if name == "latent_attention":  # one row of rank + rot a key, and the latent once more as values
             H, R, P = a[6], a[7], a[8]
             read, loaded = keys_of_call(a, kw)
@@ -462,11 +479,11 @@ def design_comparison(args, design) -> int:
                "latent_kv_write", "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "norm_add_norm_affine",
                "delta_rule", "delta_prepare", "gated_head_norm", "qk_projection_norm", "gate_mul", "scale_", "cast", "cast_cols",
                "rglru_gates", "rglru_scan", "short_conv", "group_norm_chain", "poly_norm", "moe_route_grouped", "talking_attention", "ssd", "ssd_step",
-               "gated_group_norm", "value_head_norm", "stream_rows"]
+               "gated_group_norm", "value_head_norm", "stream_rows", "linear_recurrence", "stream_enter", "soft_cap_"]
     small = {"moe_route", "moe_combine", "add_norm", "norm_add_norm", "norm_add_norm_affine", "rms_norm_cols", "rope_kv_write", "latent_kv_write",
              "latent_q_rotate", "activation", "clamped_gated_act", "gated_act", "embed", "delta_prepare", "gated_head_norm",
              "qk_projection_norm", "gate_mul", "scale_", "cast", "cast_cols", "short_conv", "group_norm_chain", "poly_norm",
-             "moe_route_grouped", "gated_group_norm", "value_head_norm", "stream_rows"}
+             "moe_route_grouped", "gated_group_norm", "value_head_norm", "stream_rows", "stream_enter", "soft_cap_"}
 
     def classes_of_a_step(run):
         """{class: (ms, ms at the roofline)} of the kernels of `run()`, by events around every call into the library."""
@@ -564,7 +581,7 @@ def design_comparison(args, design) -> int:
             torch.cuda.empty_cache()
         return out
 
-    beside = {"sidalorn": "zodolorn", "zimorax": "defapel"}.get(design, "llama")
+    beside = {"sidalorn": "zodolorn", "zimorax": "defapel", "kapuvik": "defapel"}.get(design, "llama")
     record = {"workload": f"{design} beside {beside} at equal layer sizes", "layers": layers, "dtype": "bf16",
               "data": "synthetic: random weights N(0, 0.02), uniform random token ids",
               "peak_measured": {"read_gbs": round(read_bps / 1e9, 1), "mfma_tflops": round(mfma_flops / 1e12, 1)}, "sizes": {}}
@@ -596,6 +613,37 @@ def design_comparison(args, design) -> int:
                                                                    vocab=vocab), **mine),
                                      "defapel": dict(config=dict(width=width, heads=heads, kv_heads=kv, dim=dim, window=window, delta_heads=dheads,
                                                                    experts=experts, top=top, expert_ff=expert_ff, vocab=vocab), **theirs)}
+        print(json.dumps(record))
+        return 0
+    if design == "kapuvik":
+        from fms_amd.architectures.defapel import make_config as make_defapel
+        from fms_amd.architectures.kapuvik import make_config as make_kapuvik
+
+        for (name, width, pattern, heads, kv, dim, ff, rheads, rdim, rvdim, (ldim, lrot, lvdim, rank),
+             (window, experts, top, expert_ff, q_rank), vocab) in KAPUVIK_SIZES:
+            pattern = (pattern * layers)[:layers]
+            loop = {"start": 1, "stop": layers, "times": 1} if layers > 1 else None  # every layer runs once, as the other models' do
+            configs = {
+                "kapuvik": make_kapuvik(width=width, vocab=vocab, pattern=pattern, heads=heads, kv_heads=kv, dim=dim, vdim=dim, ff=ff,
+                                        latent_heads=heads, latent_dim=ldim, rot_dim=lrot, latent_vdim=lvdim, kv_rank=rank, ret_heads=rheads,
+                                        ret_dim=rdim, ret_vdim=rvdim, gla_heads=rheads, gla_dim=rdim, gla_vdim=rvdim, loop=loop,
+                                        max_positions=context),
+                "defapel": make_defapel(width=width, vocab=vocab, pattern=("pcpc" * layers)[:layers], heads=heads, kv_heads=kv, dim=dim, vdim=dim,
+                                        window=window, delta_heads=rheads, delta_kv_heads=rheads, delta_dim=rdim, delta_vdim=rvdim, experts=experts,
+                                        top=top, expert_ff=expert_ff, max_positions=context),
+                "zodolorn": make_config(width=width, vocab=vocab, nlayers=layers, heads=heads, dim=ldim, rot_dim=lrot, vdim=lvdim, q_rank=q_rank,
+                                        kv_rank=rank, dense_ff=ff, experts=experts, top=top, expert_ff=expert_ff, shared_ff=2 * expert_ff,
+                                        max_positions=context),
+            }
+            sizes = dict(width=width, pattern=pattern, heads=heads, kv_heads=kv, dim=dim, ff=ff, recurrence_heads=rheads, key_channels=rdim,
+                         value_channels=rvdim, latent=(ldim, lrot, lvdim, rank), experts=experts, top=top, expert_ff=expert_ff, vocab=vocab)
+            record["sizes"][name] = {"config": sizes}
+            for which, config in configs.items():
+                model = fms_amd.from_config(config, which, data_type="bf16", random_seed=args.seed)
+                record["sizes"][name][which] = measure(model, vocab, per_call_masks=True)
+                del model
+                torch.cuda.empty_cache()
+                print(f"bench: {name} {which} measured", file=sys.stderr, flush=True)
         print(json.dumps(record))
         return 0
     if design == "basopel":

@@ -374,13 +374,29 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const BiasT* __restri
 #pragma unroll
       for (int e = 0; e < VEC; ++e) gv[e] = g[j + e], uv[e] = u[j + e];
     }
+    float bg[VEC], bu[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) bg[e] = bu[e] = 0.f;
+    if (bias) {  // uniform; rows of vectors have biases of vectors (the host checks the address)
+      if constexpr (VEC > 1) {
+#pragma unroll
+        for (int e = 0; e < VEC; e += 4) {
+          float x[4];
+          load_vec<4>(bias + j + e, x);
+          bg[e] = x[0], bg[e + 1] = x[1], bg[e + 2] = x[2], bg[e + 3] = x[3];
+          load_vec<4>(bias + hidden + j + e, x);
+          bu[e] = x[0], bu[e + 1] = x[1], bu[e + 2] = x[2], bu[e + 3] = x[3];
+        }
+      } else {
+        bg[0] = to_f32(bias[j]);
+        bu[0] = to_f32(bias[hidden + j]);
+      }
+    }
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
       float a = to_f32(gv[e]), b = to_f32(uv[e]);
-      if (bias) {
-        a += to_f32(bias[j + e]);
-        b += to_f32(bias[hidden + j + e]);
-      }
+      a += bg[e];
+      b += bu[e];
       ov[e] = from_f32<T>(act == FMS_ACT_CLAMPED_GATE ? clamped_gate(a, b, clamp.limit, clamp.alpha, clamp.shift) : activate(a, act) * b);
     }
     if constexpr (VEC * sizeof(T) == 16) {
@@ -396,7 +412,7 @@ template <typename T, typename BiasT>
 static void launch_gated_act(const void* gu, const void* bias, void* out, long ldo, int n_tokens, int hidden, int act,
                              fmsamd_gate_clamp clamp, hipStream_t stream) {
   constexpr int VEC = 16 / sizeof(T);
-  const bool wide = hidden % VEC == 0 && ldo % VEC == 0 && (((size_t)gu | (size_t)out) & 15) == 0;
+  const bool wide = hidden % VEC == 0 && ldo % VEC == 0 && (((size_t)gu | (size_t)out | (size_t)bias) & 15) == 0;
   const int per_thread = wide ? VEC : 1;
   const int blocks = ceil_div(hidden, 256 * per_thread);
   dim3 grid(blocks > 64 ? 64 : blocks, n_tokens);

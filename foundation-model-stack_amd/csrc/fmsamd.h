@@ -422,8 +422,9 @@ int fmsamd_gated_group_norm(const float* y, const float* z, long ldz, const void
 // k (heads * dim entries from col_q, col_k on), v and gate logits (heads * vdim from col_v, col_g on).  Decays: a = exp(log_decay)
 // per head, or (up_t) sigmoid(z)^inv_tau per head and key channel, z = up (the rank numbers from col_low on) + up_bias with
 // up_t [rank][heads * dim].  rot_dim > 0: the first rot_dim channels of q and k are rotated in neighbouring pairs by the
-// token's position.  q is multiplied by q_scale.  The walk writes o / rms(o) * norm_w (or no weight) * act(gate) * out_scale to
-// rows of out (ldo apart, zeros for padding rows); the chunked form (long steps) writes o itself.
+// token's position.  q is multiplied by q_scale.  Rows of out (ldo apart) get o / rms(o) * norm_w (or no weight) * act(gate) *
+// out_scale per head; padding rows (the walk only) get zeros.  The walk goes token by token, the chunked form (long steps, at
+// most 256 value channels) in chunks of 64 tokens.
 typedef struct fmsamd_linear_recurrence {
   const float* proj;
   long ld;
@@ -446,9 +447,9 @@ typedef struct fmsamd_linear_recurrence {
   long ldo;
 } fmsamd_linear_recurrence;
 int fmsamd_linear_recurrence_walk(const fmsamd_linear_recurrence* args, hipStream_t stream);
-long fmsamd_linear_recurrence_workspace(int n_tokens, int n_seqs, int heads, int dim);
-int fmsamd_linear_recurrence_chunked(const fmsamd_linear_recurrence* args, float* y, int longest, float* workspace,
-                                     long workspace_bytes, hipStream_t stream);
+long fmsamd_linear_recurrence_workspace(int n_tokens, int n_seqs, int heads, int dim, int vdim);
+int fmsamd_linear_recurrence_chunked(const fmsamd_linear_recurrence* args, int longest, float* workspace, long workspace_bytes,
+                                     hipStream_t stream);
 
 // out[t] = resid[t] + branch[t] * branch_scale + base[t] + shift, float32 rows (branch in the activation type; branch,
 // branch_scale, base and shift (width entries) may be null)

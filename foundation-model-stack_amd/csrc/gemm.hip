@@ -1,8 +1,9 @@
 // Matrix products y = x W^T (+ bias) for weights stored [N, K] with K contiguous,
 // which is how every linear layer of a checkpoint is stored.
 //
-//   * sgemm_nt_kernel: float32 in, float32 FMA accumulation, float32 out.  The
-//     true 32-bit path: no matrix-core shortcut, no reduced-precision inputs.
+//   * sgemm_nt_kernel: float32 in, float32 FMA over runs of 16, float64 over the
+//     runs, float32 out.  The true 32-bit path: no matrix-core shortcut, no
+//     reduced-precision inputs.
 //   * gemm_bf16_kernel: bfloat16 in, MFMA 16x16x32 with float32 accumulation,
 //     bfloat16 or float32 out; LDS-tiled 128x128x32.  Any M and N; K % 8 == 0.
 //   * skinny_bf16_kernel: M <= 16 rows of x (decode).  Weight-streaming: a
@@ -34,8 +35,11 @@ __global__ void __launch_bounds__(256)
   const int ty = threadIdx.x / 16;  // m direction
   const int m0 = blockIdx.y * SG_BM;
   const int n0 = blockIdx.x * SG_BN;
-  float acc[4][4] = {};
+  // Sums of 16 products each in float32, added up in float64: what a long K costs is the rounding of short sums, not of every
+  // partial sum on the way.
+  double total[4][4] = {};
   for (int k0 = 0; k0 < K; k0 += SG_BK) {
+    float acc[4][4] = {};
     for (int i = threadIdx.x; i < SG_BM * SG_BK; i += 256) {
       const int row = i / SG_BK, kk = i % SG_BK;
       const int m = m0 + row, k = k0 + kk;
@@ -57,6 +61,10 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(av[i], wv[j], acc[i][j]);
     }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) total[i][j] += acc[i][j];
     __syncthreads();
   }
 #pragma unroll
@@ -66,7 +74,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) c[(size_t)m * ldc + n] = from_f32<OutT>(acc[i][j] + (bias ? to_f32(bias[n]) : 0.f));
+      if (n < N) c[(size_t)m * ldc + n] = from_f32<OutT>((float)(total[i][j] + (bias ? to_f32(bias[n]) : 0.f)));
     }
   }
 }

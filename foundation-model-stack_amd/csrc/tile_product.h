@@ -48,12 +48,15 @@ __device__ __forceinline__ void tile_product_fma(ARow a_row, WRow w_row, int K, 
 #pragma unroll
     for (int i = 0; i < 8; ++i) Ws[lr + 8 * i][lk] = (in && wrow[i]) ? to_f32(wrow[i][k0 + lk]) : 0.f;
     __syncthreads();
+    float run[4] = {0.f, 0.f, 0.f, 0.f};  // a run of K in a sum of its own: fewer roundings of the whole sum
 #pragma unroll
     for (int k = 0; k < BK; ++k) {
       const float w = Ws[n][k];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) acc[i] = fmaf(As[mg * 4 + i][k], w, acc[i]);
+      for (int i = 0; i < 4; ++i) run[i] = fmaf(As[mg * 4 + i][k], w, run[i]);
     }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] += run[i];
     __syncthreads();
   }
 }

@@ -88,7 +88,7 @@ _SIGNATURES = {
     "fmsamd_ssd_step": [P, L, I, I, P, P, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
     "fmsamd_gated_group_norm": [P, P, L, P, I, I, F, P, I, P, I, I, P, L, I, I, P, P, P],
     "fmsamd_linear_recurrence_walk": [P, P],
-    "fmsamd_linear_recurrence_chunked": [P, P, I, P, L, P],
+    "fmsamd_linear_recurrence_chunked": [P, I, P, L, P],
     "fmsamd_stream_enter": [P, P, I, P, P, P, P, I, I, P],
     "fmsamd_soft_cap_f32": [P, L, F, P],
     "fmsamd_probe_read": [P, L, I, I, P, P],
@@ -137,7 +137,7 @@ def load(verbose: bool = True) -> ctypes.CDLL:
         lib.fmsamd_ssd_chunk_workspace.restype = c_long
         lib.fmsamd_ssd_chunk_workspace.argtypes = [I, I, I]
         lib.fmsamd_linear_recurrence_workspace.restype = c_long
-        lib.fmsamd_linear_recurrence_workspace.argtypes = [I, I, I, I]
+        lib.fmsamd_linear_recurrence_workspace.argtypes = [I, I, I, I, I]
         lib.fmsamd_talking_attn_workspace.restype = c_long
         lib.fmsamd_talking_attn_workspace.argtypes = [I, I, I, I]
         lib.fmsamd_moe_max_tiles.restype = c_int

@@ -1693,6 +1693,7 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, par
 # linear attention with a decay
 # --------------------------------------------------------------------------
 LINEAR_MAX_DIM = 256
+LINEAR_CHUNK_MAX_VDIM = 256
 LINEAR_CHUNK_FROM = 32  # tokens a sequence: from there on a step runs the recurrence in chunks
 
 
@@ -1768,12 +1769,11 @@ def linear_recurrence(proj: torch.Tensor, cols, heads: int, dim: int, vdim: int,
         state.data_ptr(), seq_starts.data_ptr(), seq_of_token.data_ptr(), slot_ids.data_ptr(), int(n_seqs), T, _ptr(norm_weight), float(eps),
         float(scale), ACTIVATIONS[activation], out.data_ptr(), _code(out_dtype), out.stride(0))
     lib = load()
-    if longest >= LINEAR_CHUNK_FROM if chunked is None else chunked:
-        ws_bytes = lib.fmsamd_linear_recurrence_workspace(T, int(n_seqs), heads, dim)
+    if (longest >= LINEAR_CHUNK_FROM and vdim <= LINEAR_CHUNK_MAX_VDIM) if chunked is None else chunked:
+        ws_bytes = lib.fmsamd_linear_recurrence_workspace(T, int(n_seqs), heads, dim, vdim)
         ws = torch.empty(ws_bytes // 4, dtype=torch.float32, device=proj.device)
-        y = torch.empty(T, HV, dtype=torch.float32, device=proj.device)
-        check(lib.fmsamd_linear_recurrence_chunked(ctypes.byref(arg), y.data_ptr(), int(longest), ws.data_ptr(), ws_bytes, _stream()))
-        return gated_head_norm(y, proj[:, cols[3] : cols[3] + HV], norm_weight, eps, activation, heads, vdim, out_dtype, seq_of_token, scale, out)
+        check(lib.fmsamd_linear_recurrence_chunked(ctypes.byref(arg), int(longest), ws.data_ptr(), ws_bytes, _stream()))
+        return out
     check(lib.fmsamd_linear_recurrence_walk(ctypes.byref(arg), _stream()))
     return out
 
