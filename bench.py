@@ -420,7 +420,7 @@ def design_comparison(args, design) -> int:
         return sum(t.numel() * t.element_size() for t in tensors if t is not None)
 
     def cost(name, a, kw, out):
-        if name in ("linear", "gated_linear", "linear_into_stream"):
+        if name in ("linear", "gated_linear", "linear_into_stream", "qkv_rope_write"):
             x, w = a[0], a[1]
             return nbytes(x, w) + (nbytes(out) if torch.is_tensor(out) else 0), 2.0 * x.shape[0] * w.shape[0] * w.shape[1]
         if name == "headwise_linear":
