@@ -282,7 +282,7 @@ __global__ void __launch_bounds__(DELTA_THREADS) delta_rule_kernel(DeltaArgs a) 
   }
 }
 
-// out[t, h, j] = o / rms_j(o) * weight[j] (or no weight) * act(gate[t, h, j]) * out_scale; one wave per (token, head)
+// out[t, h, j] = o / rms_j(o) * weight[j] * act(gate[t, h, j]) * out_scale; one wave per (token, head)
 template <typename T, typename W>
 __global__ void __launch_bounds__(256)
     gated_head_norm_kernel(const float* __restrict__ o, const float* __restrict__ gate, long ldg, const W* __restrict__ weight,
@@ -300,7 +300,7 @@ __global__ void __launch_bounds__(256)
   const float inv = 1.f / sqrtf(s / (float)Dv + eps);
   for (int j = lane; j < Dv; j += WAVE) {
     const float g = fms_activate(gate[(size_t)t * ldg + (size_t)h * Dv + j], act);
-    out[(size_t)t * ldo + (size_t)h * Dv + j] = from_f32<T>(row[j] * inv * (weight ? to_f32(weight[j]) : 1.f) * g * out_scale);
+    out[(size_t)t * ldo + (size_t)h * Dv + j] = from_f32<T>(row[j] * inv * to_f32(weight[j]) * g * out_scale);
   }
 }
 

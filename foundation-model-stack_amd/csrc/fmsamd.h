@@ -322,7 +322,7 @@ int fmsamd_delta_prepare(const float* proj, long ld, int col_b, const float* a, 
 int fmsamd_delta_rule(const float* qkv, const float* beta, const float* decay, const float* kq, float* state, float* out,
                       const int* seq_starts, const int* seq_of_token, const int* slot_ids, int n_seqs, int heads,
                       int kv_heads, int dim, int vdim, int per_channel, int single_tokens, hipStream_t stream);
-// out[t, h, :] = o[t, h, :] / rms * weight (null: no weight) * act(gate[t, h, :]) * out_scale
+// out[t, h, :] = o[t, h, :] / rms * weight * act(gate[t, h, :]) * out_scale
 int fmsamd_gated_head_norm(const float* o, const float* gate, long ldg, const void* weight, int weight_dtype, float eps,
                            int act, float out_scale, void* out, int out_dtype, long ldo, const int* seq_of_token,
                            int n_tokens, int heads, int vdim, hipStream_t stream);

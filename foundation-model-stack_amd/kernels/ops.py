@@ -1541,9 +1541,9 @@ def delta_rule(qkv: torch.Tensor, beta: torch.Tensor, decay: torch.Tensor, kq: t
     return out
 
 
-def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], eps: float, activation: str, heads: int, vdim: int,
+def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, activation: str, heads: int, vdim: int,
                     out_dtype: torch.dtype, seq_of_token: torch.Tensor, scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """o float32 [T, heads*vdim]: every head divided by its root mean square, times weight [vdim] (None: no weight), times act(gate)
+    """o float32 [T, heads*vdim]: every head divided by its root mean square, times weight [vdim], times act(gate)
     (float32 logits [T, heads*vdim], rows of any stride), times scale -> out_dtype (into `out`, rows of any stride)."""
     _need_cuda(o, gate, weight, seq_of_token, out)
     _rows2d("gate", gate)
@@ -1553,14 +1553,14 @@ def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.
         raise ValueError(f"o is contiguous float32 [T, {heads * vdim}]")
     if gate.dtype != torch.float32 or tuple(gate.shape) != (T, heads * vdim):
         raise ValueError(f"the gate is float32 [{T}, {heads * vdim}]")
-    if weight is not None and (tuple(weight.shape) != (vdim,) or not weight.is_contiguous()):
+    if tuple(weight.shape) != (vdim,) or not weight.is_contiguous():
         raise ValueError(f"the norm weight is a contiguous [{vdim}] tensor")
     if out is None:
         out = torch.empty(T, heads * vdim, dtype=out_dtype, device=o.device)
     _rows2d("out", out)
     if out.dtype != out_dtype or tuple(out.shape) != (T, heads * vdim):
         raise ValueError(f"out is [{T}, {heads * vdim}] of {out_dtype}")
-    check(load().fmsamd_gated_head_norm(o.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(weight), _code(weight.dtype) if weight is not None else F32, float(eps),
+    check(load().fmsamd_gated_head_norm(o.data_ptr(), gate.data_ptr(), gate.stride(0), weight.data_ptr(), _code(weight.dtype), float(eps),
                                         ACTIVATIONS[activation], float(scale), out.data_ptr(), _code(out_dtype), out.stride(0),
                                         seq_of_token.data_ptr(), T, heads, vdim, _stream()))
     return out
